@@ -7,6 +7,7 @@ from .malusun import MalusunConfig
 from .mazanex import MazanexConfig
 from .qwen3 import Qwen3Config
 from .rekezen import RekezenConfig
+from .talapel import TalapelConfig
 
 __all__ = ["ConfigError", "DubizenConfig", "EngineConfig", "MalusunConfig", "MazanexConfig", "ModelConfig", "Qwen3Config", "RekezenConfig", "SchedulerConfig",
-           "load_model_config"]
+           "TalapelConfig", "load_model_config"]

@@ -5,7 +5,7 @@
 //   * a sink per query head: exp(sink_h) joins the softmax's denominator, with no key and no value
 //     (the running maximum starts at sink_h and the running sum at 1);
 //   * values of another width than keys;
-//   * an output gate: the result times sigmoid(gate), a gate per element or one per query head;
+//   * an output gate: the result times sigmoid(gate), a gate per element or one per query head; a constant factor;
 //   * a soft cap: scores, after the scale, become cap * tanh(score / cap);
 //   * a penalty on distance: slope_h * (p - j) comes off head h's score of key j (after scale and cap);
 //   * a bias by distance: table[h][min(p - j, span - 1)] is added to head h's score of key j (after the scale,
@@ -24,7 +24,7 @@
 template <typename T, int TK, int DPT>
 __global__ __launch_bounds__(256) void masked_attention_kernel(
     const T* __restrict__ q, size_t q_stride, const T* __restrict__ key_pages, const T* __restrict__ value_pages,
-    T* __restrict__ out, const T* __restrict__ gate, size_t gate_stride, const float* __restrict__ sink,
+    T* __restrict__ out, size_t out_stride, float factor, const T* __restrict__ gate, size_t gate_stride, const float* __restrict__ sink,
     const int* __restrict__ cu_q, const int* __restrict__ ctx_len, const int* __restrict__ block_table,
     int table_stride, int kv_heads, int groups, int D, int Dv, int block_size, int num_blocks, int window,
     int chunk, float scale, float softcap, int head_gate, const float* __restrict__ slopes,
@@ -169,9 +169,9 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
   if (row_ok) {
     const float inv = l > 0.f ? 1.f / l : 0.f;
     const size_t at = (size_t)head * Dv;
-    T* orow = out + (size_t)(q0 + my_tok) * ((size_t)kv_heads * groups * Dv) + at;
+    T* orow = out + (size_t)(q0 + my_tok) * out_stride + at;
     const T* grow = gate ? gate + (size_t)(q0 + my_tok) * gate_stride + (head_gate ? (size_t)head : at) : nullptr;
-    const float whole = (grow && head_gate) ? 1.f / (1.f + expf(-load_as_float(grow))) : 1.f;
+    const float whole = factor * ((grow && head_gate) ? 1.f / (1.f + expf(-load_as_float(grow))) : 1.f);
 #pragma unroll
     for (int i = 0; i < DPT; ++i) {
       const int d = c + 16 * i;
@@ -186,7 +186,7 @@ __global__ __launch_bounds__(256) void masked_attention_kernel(
 
 template <typename T>
 static int launch_masked(const void* q, long long q_stride, const void* key_pages, const void* value_pages, void* out,
-                         const void* gate, long long gate_stride, const float* sink, const int* cu_q,
+                         long long out_stride, float factor, const void* gate, long long gate_stride, const float* sink, const int* cu_q,
                          const int* ctx_len, const int* block_table, int table_stride, int num_seqs, int max_q_len,
                          int q_heads, int kv_heads, int D, int Dv, int block_size, int num_blocks, int window,
                          int chunk, float scale, float softcap, int head_gate, const float* slopes, const float* dist_bias,
@@ -204,7 +204,7 @@ static int launch_masked(const void* q, long long q_stride, const void* key_page
                             (int)lds) != hipSuccess)                                                             \
       return FE_BAD_ARGUMENT;                                                                                    \
     masked_attention_kernel<T, TK, DPT><<<grid, 256, lds, stream>>>(                                             \
-        (const T*)q, (size_t)q_stride, (const T*)key_pages, (const T*)value_pages, (T*)out, (const T*)gate,      \
+        (const T*)q, (size_t)q_stride, (const T*)key_pages, (const T*)value_pages, (T*)out, (size_t)out_stride, factor, (const T*)gate, \
         (size_t)gate_stride, sink, cu_q, ctx_len, block_table, table_stride, kv_heads, groups, D, Dv, block_size, \
         num_blocks, window, chunk, scale, softcap, head_gate, slopes, dist_bias, span);                          \
   } while (0)
@@ -225,7 +225,7 @@ static int launch_masked(const void* q, long long q_stride, const void* key_page
 }
 
 extern "C" int fe_masked_attention(const void* q, int dtype, long long q_stride, const void* key_pages,
-                                   const void* value_pages, void* out, const void* gate, long long gate_stride,
+                                   const void* value_pages, void* out, long long out_stride, float factor, const void* gate, long long gate_stride,
                                    const float* sink, const int* cu_q, const int* ctx_len, const int* block_table,
                                    int table_stride, int num_seqs, int max_q_len, int q_heads, int kv_heads,
                                    int head_dim, int value_dim, int block_size, int num_blocks, int window, int chunk,
@@ -236,15 +236,15 @@ extern "C" int fe_masked_attention(const void* q, int dtype, long long q_stride,
       value_dim > 512 || (!value_pages && value_dim > head_dim) || (dist_bias && span < 1) || block_size <= 0 || num_blocks <= 0 || max_q_len < 1 || window < 0 || chunk < 0 ||
       num_seqs > 65535 || kv_heads > 65535)
     return FE_BAD_ARGUMENT;
-  if (q_stride < (long long)q_heads * head_dim || softcap < 0.f ||
+  if (q_stride < (long long)q_heads * head_dim || softcap < 0.f || out_stride < (long long)q_heads * value_dim ||
       (gate && gate_stride < (long long)q_heads * (head_gate ? 1 : value_dim)))
     return FE_BAD_ARGUMENT;
   if (dtype == FE_F32)
-    return launch_masked<float>(q, q_stride, key_pages, value_pages, out, gate, gate_stride, sink, cu_q, ctx_len,
+    return launch_masked<float>(q, q_stride, key_pages, value_pages, out, out_stride, factor, gate, gate_stride, sink, cu_q, ctx_len,
                                 block_table, table_stride, num_seqs, max_q_len, q_heads, kv_heads, head_dim, value_dim,
                                 block_size, num_blocks, window, chunk, scale, softcap, head_gate, slopes, dist_bias, span, stream);
   if (dtype == FE_BF16)
-    return launch_masked<bf16_t>(q, q_stride, key_pages, value_pages, out, gate, gate_stride, sink, cu_q, ctx_len,
+    return launch_masked<bf16_t>(q, q_stride, key_pages, value_pages, out, out_stride, factor, gate, gate_stride, sink, cu_q, ctx_len,
                                  block_table, table_stride, num_seqs, max_q_len, q_heads, kv_heads, head_dim, value_dim,
                                  block_size, num_blocks, window, chunk, scale, softcap, head_gate, slopes, dist_bias, span, stream);
   return FE_BAD_ARGUMENT;

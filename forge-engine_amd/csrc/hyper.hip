@@ -2,7 +2,8 @@
 //
 // fe_hyper_norm: one block per row.  With S streams x_0 .. x_(S-1) of a token (S = 1: the plain
 // residual stream) and a pending update y (float32, maybe in parts that are added up in order):
-//   x_t <- sum_s mix[s][t] x_s + share[t] y      (mix absent: the identity; share absent: ones)
+//   x_t <- sum_s mix[s][t] x_s + share[t] y      (mix absent: the identity; share absent: ones; y may be a bias
+//                                                 per channel, alone or on top of the update)
 //   u    = sum_t read[t] x_t                      (read absent: ones, the plain sum)
 //   out  = (u - mean) / sqrt(var + eps) * w + b   (layer norm; RMS norm: no mean, no bias)
 // all in float32 with one rounding at the store.  The new streams are written back unless the call
@@ -17,7 +18,7 @@
 template <typename TO, int S, int VEC, int THREADS>
 __global__ __launch_bounds__(THREADS) void hyper_norm_kernel(
     float* __restrict__ streams, long long stream_stride, const float* __restrict__ update, int parts,
-    long long part_stride, const float* __restrict__ mix, const float* __restrict__ share,
+    long long part_stride, const float* __restrict__ shift, const float* __restrict__ mix, const float* __restrict__ share,
     const float* __restrict__ read, const float* __restrict__ weight, const float* __restrict__ bias, float eps,
     int rms, TO* __restrict__ out, const int* __restrict__ rows, int W, int store) {
   extern __shared__ float u_row[];      // the row of u, W floats
@@ -45,7 +46,7 @@ __global__ __launch_bounds__(THREADS) void hyper_norm_kernel(
         x[s][0] = *p;
       }
     }
-    if (update) {
+    if (update || shift) {
 #pragma unroll
       for (int i = 0; i < VEC; ++i) y[i] = 0.f;
       for (int part = 0; part < parts; ++part) {
@@ -56,6 +57,10 @@ __global__ __launch_bounds__(THREADS) void hyper_norm_kernel(
         } else {
           y[0] += *p;
         }
+      }
+      if (shift) {
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) y[i] += shift[c + i];
       }
       float fresh[S][VEC];
 #pragma unroll
@@ -113,7 +118,7 @@ __global__ __launch_bounds__(THREADS) void hyper_norm_kernel(
 
 template <typename TO, int S>
 static void launch_hyper(float* streams, long long stream_stride, const float* update, int parts, long long part_stride,
-                         const float* mix, const float* share, const float* read, const float* weight,
+                         const float* shift, const float* mix, const float* share, const float* read, const float* weight,
                          const float* bias, float eps, int rms, void* out, const int* rows, int n_rows, int W, int store,
                          hipStream_t stream) {
   const size_t lds = out ? (size_t)W * sizeof(float) : 0;
@@ -121,24 +126,24 @@ static void launch_hyper(float* streams, long long stream_stride, const float* u
                    (!update || ((uintptr_t)update % 16 == 0 && part_stride % 4 == 0));
   // a step of few rows is a matter of round trips, not of bytes: more threads a row then (one round of loads a thread)
   if (vec && n_rows <= 512 && W >= 2048)
-    hyper_norm_kernel<TO, S, 4, 1024><<<n_rows, 1024, lds, stream>>>(streams, stream_stride, update, parts, part_stride, mix,
+    hyper_norm_kernel<TO, S, 4, 1024><<<n_rows, 1024, lds, stream>>>(streams, stream_stride, update, parts, part_stride, shift, mix,
                                                                      share, read, weight, bias, eps, rms, (TO*)out, rows, W, store);
   else if (vec)
-    hyper_norm_kernel<TO, S, 4, 256><<<n_rows, 256, lds, stream>>>(streams, stream_stride, update, parts, part_stride, mix, share,
+    hyper_norm_kernel<TO, S, 4, 256><<<n_rows, 256, lds, stream>>>(streams, stream_stride, update, parts, part_stride, shift, mix, share,
                                                                    read, weight, bias, eps, rms, (TO*)out, rows, W, store);
   else
-    hyper_norm_kernel<TO, S, 1, 256><<<n_rows, 256, lds, stream>>>(streams, stream_stride, update, parts, part_stride, mix, share,
+    hyper_norm_kernel<TO, S, 1, 256><<<n_rows, 256, lds, stream>>>(streams, stream_stride, update, parts, part_stride, shift, mix, share,
                                                                    read, weight, bias, eps, rms, (TO*)out, rows, W, store);
 }
 
 template <typename TO>
 static int dispatch_hyper(int S, float* streams, long long stream_stride, const float* update, int parts,
-                          long long part_stride, const float* mix, const float* share, const float* read,
+                          long long part_stride, const float* shift, const float* mix, const float* share, const float* read,
                           const float* weight, const float* bias, float eps, int rms, void* out, const int* rows,
                           int n_rows, int W, int store, hipStream_t stream) {
 #define CASE(N)                                                                                                       \
   case N:                                                                                                             \
-    launch_hyper<TO, N>(streams, stream_stride, update, parts, part_stride, mix, share, read, weight, bias, eps, rms, \
+    launch_hyper<TO, N>(streams, stream_stride, update, parts, part_stride, shift, mix, share, read, weight, bias, eps, rms, \
                         out, rows, n_rows, W, store, stream);                                                         \
     break;
   switch (S) {
@@ -150,18 +155,18 @@ static int dispatch_hyper(int S, float* streams, long long stream_stride, const 
 }
 
 extern "C" int fe_hyper_norm(float* streams, long long stream_stride, int num_streams, const float* update, int parts,
-                             long long part_stride, const float* mix, const float* share, const float* read,
+                             long long part_stride, const float* shift, const float* mix, const float* share, const float* read,
                              const float* weight, const float* bias, float eps, int rms, void* out, int out_dtype,
                              const int* rows, int n_rows, int width, int store, hipStream_t stream) {
   if (n_rows <= 0) return FE_OK;
   if (!streams || width <= 0 || width > 16384 || num_streams < 1 || num_streams > MAX_STREAMS || parts < 0 ||
-      (update && parts < 1) || (out && !weight) || (!out && !update))
+      (update ? parts < 1 : parts != 0) || (out && !weight) || (!out && !update && !shift))
     return FE_BAD_ARGUMENT;
   if (!out || out_dtype == FE_F32)
-    return dispatch_hyper<float>(num_streams, streams, stream_stride, update, parts, part_stride, mix, share, read, weight,
+    return dispatch_hyper<float>(num_streams, streams, stream_stride, update, parts, part_stride, shift, mix, share, read, weight,
                                  bias, eps, rms, out, rows, n_rows, width, store, stream);
   if (out_dtype == FE_BF16)
-    return dispatch_hyper<bf16_t>(num_streams, streams, stream_stride, update, parts, part_stride, mix, share, read, weight,
+    return dispatch_hyper<bf16_t>(num_streams, streams, stream_stride, update, parts, part_stride, shift, mix, share, read, weight,
                                   bias, eps, rms, out, rows, n_rows, width, store, stream);
   return FE_BAD_ARGUMENT;
 }

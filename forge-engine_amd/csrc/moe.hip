@@ -4,9 +4,12 @@
 //   fe_moe_select:   from router logits (float32): bias added, the `top` largest per token, softmax over those alone
 //                    (or, scoring 1, each chosen logit's own sigmoid)
 //   fe_moe_plan:     counts per expert, their prefix sums, and the pairs ordered by expert
+//   fe_moe_plan_table: the same where a table of token ids names every token's experts and no router is asked;
+//                    also the pairs' weights, all alike
 //   fe_moe_gate_up:  for every pair, act = min(g, L) * sigmoid(alpha min(g, L)) * (clamp(u, -L, L) + 1) with
 //                    g = W_gate[e] x, u = W_up[e] x of the pair's token and expert (form 1: silu(g) * u; with
-//                    input weights, g and u are first multiplied by the pair's routing weight)
+//                    input weights, g and u are first multiplied by the pair's routing weight); form 2: one matrix
+//                    an expert, act = max(u, 0)^2
 //   fe_moe_down:     out[choice][token] = weight * W_down[e] act   (float32; one part per choice, so
 //                    that the reader adds a token's experts up in a fixed order; the first choice's part
 //                    also takes what every token gets beside its experts, a shared expert's output)
@@ -144,14 +147,14 @@ extern "C" int fe_moe_select_grouped(const float* logits, long long stride, cons
 
 // One block: offsets[e] = pairs of experts below e, order[offsets[e] ..] = the pairs of expert e.
 // Within an expert the pairs come in no fixed order; a pair's results do not depend on its row.
-__global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ chosen, int pairs, int E,
-                                                        int* __restrict__ offsets, int* __restrict__ order) {
+template <typename Choice>
+__device__ __forceinline__ void plan_pairs(Choice choice, int pairs, int E, int* __restrict__ offsets, int* __restrict__ order) {
   extern __shared__ int counts[];   // [E] counts, then [E] cursors
   int* cursor = counts + E;
   for (int e = threadIdx.x; e < E; e += blockDim.x) counts[e] = 0;
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
-    const int e = chosen[i];
+    const int e = choice(i);
     if (e >= 0 && e < E) atomicAdd(&counts[e], 1);
   }
   __syncthreads();
@@ -165,9 +168,25 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   }
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
-    const int e = chosen[i];
+    const int e = choice(i);
     if (e >= 0 && e < E) order[atomicAdd(&cursor[e], 1)] = i;
   }
+}
+
+__global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ chosen, int pairs, int E,
+                                                        int* __restrict__ offsets, int* __restrict__ order) {
+  plan_pairs([&](int i) { return chosen[i]; }, pairs, E, offsets, order);
+}
+
+// Pair i is choice i % top of token i / top: column i % top of the table's row for the token's id.
+__global__ __launch_bounds__(1024) void moe_plan_table_kernel(const int* __restrict__ ids, const int* __restrict__ table, int vocab,
+                                                              int top, int pairs, int E, int* __restrict__ offsets,
+                                                              int* __restrict__ order, float* __restrict__ weights, float weight) {
+  plan_pairs([&](int i) {
+    const int id = ids[i / top];
+    return table[(size_t)(id >= 0 && id < vocab ? id : 0) * top + i % top];
+  }, pairs, E, offsets, order);
+  for (int i = threadIdx.x; i < pairs; i += blockDim.x) weights[i] = weight;
 }
 
 extern "C" int fe_moe_plan(const int* chosen, int pairs, int experts, int* offsets, int* order, hipStream_t stream) {
@@ -177,15 +196,26 @@ extern "C" int fe_moe_plan(const int* chosen, int pairs, int experts, int* offse
   return fe_check_launch();
 }
 
+// ids [tokens]; table [vocab][top] (expert numbers below `experts`); weights [tokens][top] all become `weight`
+extern "C" int fe_moe_plan_table(const int* ids, const int* table, int vocab, int tokens, int top, int experts, int* offsets,
+                                 int* order, float* weights, float weight, hipStream_t stream) {
+  if (tokens <= 0) return FE_OK;
+  if (experts <= 0 || experts > 1024 || top < 1 || top > 16 || vocab < 1 || (long long)tokens * top > 0x7fffffffLL) return FE_BAD_ARGUMENT;
+  moe_plan_table_kernel<<<1, 1024, 2 * (size_t)experts * sizeof(int), stream>>>(ids, table, vocab, top, tokens * top, experts,
+                                                                               offsets, order, weights, weight);
+  return fe_check_launch();
+}
+
 #define BM 32
 #define BN 64
 #define BK 32
 
-// form 0: the bounded activation above; form 1: silu(g) * u.  `w` scales both products first (a router's weight
+// form 0: the bounded activation above; form 1: silu(g) * u; form 2: max(g, 0)^2.  `w` scales both products first (a router's weight
 // on the expert's input: W (w x) = w (W x)).
 __device__ __forceinline__ float gated(float g, float u, float limit, float alpha, int form, float w) {
   g *= w;
   u *= w;
+  if (form == 2) return fmaxf(g, 0.f) * fmaxf(g, 0.f);      // one matrix an expert: g alone
   if (form == 1) return g / (1.f + expf(-g)) * u;
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
@@ -223,7 +253,8 @@ __device__ __forceinline__ bool find_tile(const int* __restrict__ offsets, int E
 
 // MODE 0: rows are tokens' x gathered through the sorted pairs, the weight is [E][2N][K] (gate rows, then
 // up rows), the ending is the gated activation into act [pairs, N].  MODE 1: rows are act's sorted rows,
-// the weight is [E][N][K], and the result times the pair's routing weight goes to out[choice][token][N].
+// the weight is [E][N][K], and the result times the pair's routing weight goes to out[choice][token][N].  MODE 2: as
+// MODE 0 with one matrix an expert, [E][N][K].
 template <typename T, int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const T* __restrict__ a, const T* __restrict__ w, const int* __restrict__ offsets, const int* __restrict__ order,
@@ -254,7 +285,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
       float v = 0.f;
       const int pair = pair_of[r];
       if (pair >= 0 && k0 + k < K) {
-        const size_t src = MODE == 0 ? (size_t)(pair / top) : (size_t)(row0 + r);
+        const size_t src = MODE != 1 ? (size_t)(pair / top) : (size_t)(row0 + r);
         v = load_as_float(a + src * K + k0 + k);
       }
       As[r][k] = v;
@@ -293,7 +324,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx + 16 * j;
       if (n >= N) continue;
-      if (MODE == 0) {
+      if (MODE != 1) {
         store_from_float(act + (size_t)(row0 + r) * N + n, gated(acc_g[i][j], acc_u[i][j], limit, alpha, form, pair_weight ? pair_weight[pair] : 1.f));
       } else {
         const int token = pair / top, choice = pair - token * top;
@@ -368,7 +399,7 @@ __global__ __launch_bounds__(256) void moe_grouped_mfma_kernel(
     my_row[j] = tid / 4 + 64 * j;
     const int pair = pair_of[my_row[j]];
     my_live[j] = pair >= 0;
-    const size_t src = pair < 0 ? 0 : (MODE == 0 ? (size_t)(pair / top) : (size_t)(row0 + my_row[j]));
+    const size_t src = pair < 0 ? 0 : (MODE != 1 ? (size_t)(pair / top) : (size_t)(row0 + my_row[j]));
     a_at[j] = a + src * K + my_chunk * 8;
   }
   const size_t w_rows = MODE == 0 ? 2 * (size_t)N : (size_t)N;
@@ -452,7 +483,7 @@ __global__ __launch_bounds__(256) void moe_grouped_mfma_kernel(
         const int r = mt * 16 + lq * 4 + i;
         const int pair = pair_of[r];
         if (pair < 0) continue;
-        if (MODE == 0) {
+        if (MODE != 1) {
           act[(size_t)(row0 + r) * N + n[nt]] = float_to_bf16(gated(acc_g[nt][mt][i], acc_u[nt][mt][i], limit, alpha, form, pair_weight ? pair_weight[pair] : 1.f));
         } else {
           const int token = pair / top, choice = pair - token * top;
@@ -500,7 +531,7 @@ __global__ __launch_bounds__(256) void moe_grouped_staged_kernel(
   // matrix, k chunk tid % 4
   const int my_row = tid / 4, my_chunk = tid % 4;
   const int my_pair = pair_of[my_row];
-  const size_t src = my_pair < 0 ? 0 : (MODE == 0 ? (size_t)(my_pair / top) : (size_t)(row0 + my_row));
+  const size_t src = my_pair < 0 ? 0 : (MODE != 1 ? (size_t)(my_pair / top) : (size_t)(row0 + my_row));
   const bf16_t* a_at = a + src * K + my_chunk * 8;
   const size_t w_rows = MODE == 0 ? 2 * (size_t)N : (size_t)N;
   const bf16_t* w_at[MATS][2];
@@ -586,7 +617,7 @@ __global__ __launch_bounds__(256) void moe_grouped_staged_kernel(
         const int r = mt * 16 + lq * 4 + i;
         const int pair = pair_of[r];
         if (pair < 0) continue;
-        if (MODE == 0) {
+        if (MODE != 1) {
           act[(size_t)(row0 + r) * N + n] = float_to_bf16(gated(acc[0][nt][mt][i], acc[MATS - 1][nt][mt][i], limit, alpha, form, pair_weight ? pair_weight[pair] : 1.f));
         } else {
           const int token = pair / top, choice = pair - token * top;
@@ -628,11 +659,25 @@ extern "C" int fe_moe_gate_up(const void* x, const void* gate_up, int dtype, con
                               int tokens, int top, int experts, int hidden, int inner, float limit, float alpha, int form,
                               const float* input_weight, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
-  if (top < 1 || experts < 1 || experts > 1024 || hidden <= 0 || inner <= 0 || form < 0 || form > 1 ||
+  if (top < 1 || experts < 1 || experts > 1024 || hidden <= 0 || inner <= 0 || form < 0 || form > 2 ||
       (form == 0 && !(limit > 0.f)))
     return FE_BAD_ARGUMENT;
   const long long pairs = (long long)tokens * top;
   const dim3 grid((unsigned)(pairs / BM + experts), (unsigned)((inner + BN - 1) / BN));
+  if (form == 2) {       // one matrix an expert: `gate_up` is [experts][inner][hidden]
+    if (dtype == FE_F32)
+      moe_grouped_kernel<float, 2><<<grid, 256, 0, stream>>>((const float*)x, (const float*)gate_up, offsets, order, input_weight,
+                                                             (float*)act, nullptr, experts, inner, hidden, top, tokens, limit, alpha, form, nullptr, 0);
+    else if (dtype == FE_BF16 && mfma_fits(x, gate_up, hidden)) {
+      MFMA_LAUNCH(2, inner, (const bf16_t*)x, (const bf16_t*)gate_up, input_weight, (bf16_t*)act, nullptr, inner, hidden, limit, alpha, form, nullptr, 0);
+    } else if (dtype == FE_BF16)
+      moe_grouped_kernel<bf16_t, 2><<<grid, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, offsets, order, input_weight,
+                                                              (bf16_t*)act, nullptr, experts, inner, hidden, top, tokens, limit,
+                                                              alpha, form, nullptr, 0);
+    else
+      return FE_BAD_ARGUMENT;
+    return fe_check_launch();
+  }
   if (dtype == FE_F32)
     moe_grouped_kernel<float, 0><<<grid, 256, 0, stream>>>((const float*)x, (const float*)gate_up, offsets, order, input_weight,
                                                            (float*)act, nullptr, experts, inner, hidden, top, tokens, limit, alpha, form, nullptr, 0);

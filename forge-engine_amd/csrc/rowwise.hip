@@ -222,24 +222,26 @@ extern "C" int fe_add_rows(float* h, const void* delta, int delta_dtype, long lo
 // gate_up is [T, 2*inter] with gate in the first half of each row:
 //   out[t, i] = silu(gate[t, i]) * up[t, i],  silu(z) = z / (1 + exp(-z)),  in float32.
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int inter, size_t total) {
+__global__ void swiglu_kernel(const T* __restrict__ gate_up, size_t in_stride, T* __restrict__ out, size_t out_stride, int inter,
+                              size_t total) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / inter;
     const int c = (int)(i - t * inter);
-    const T* row = gate_up + t * 2 * (size_t)inter;
+    const T* row = gate_up + t * in_stride;
     const float g = load_as_float(row + c);
     const float u = load_as_float(row + inter + c);
-    store_from_float(out + i, g / (1.f + expf(-g)) * u);
+    store_from_float(out + t * out_stride + c, g / (1.f + expf(-g)) * u);
   }
 }
 
 // bfloat16 rows whose width is a multiple of 8: eight elements (16 bytes) of gate and of up per thread.
-__global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __restrict__ gate_up,
-                                                            bf16_t* __restrict__ out, int inter8, size_t total8) {
+__global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __restrict__ gate_up, size_t in_stride8,
+                                                            bf16_t* __restrict__ out, size_t out_stride8, int inter8,
+                                                            size_t total8) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total8; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / inter8;
     const int c = (int)(i - t * inter8);
-    const uint4* row = (const uint4*)gate_up + t * 2 * (size_t)inter8;
+    const uint4* row = (const uint4*)gate_up + t * in_stride8;
     const uint4 g = row[c];
     const uint4 u = row[inter8 + c];
     const uint32_t gw[4] = {g.x, g.y, g.z, g.w}, uw[4] = {u.x, u.y, u.z, u.w};
@@ -251,28 +253,31 @@ __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __rest
       ow[k] = (uint32_t)float_to_bf16(g0 / (1.f + expf(-g0)) * u0) |
               ((uint32_t)float_to_bf16(g1 / (1.f + expf(-g1)) * u1) << 16);
     }
-    ((uint4*)out)[i] = make_uint4(ow[0], ow[1], ow[2], ow[3]);
+    ((uint4*)out)[t * out_stride8 + c] = make_uint4(ow[0], ow[1], ow[2], ow[3]);
   }
 }
 
-extern "C" int fe_swiglu(const void* gate_up, void* out, int dtype, int tokens, int inter, hipStream_t stream) {
+// rows of gate_up (gate, then up) lie in_stride elements apart, rows of out out_stride
+extern "C" int fe_swiglu(const void* gate_up, long long in_stride, void* out, long long out_stride, int dtype, int tokens,
+                         int inter, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
-  if (inter <= 0) return FE_BAD_ARGUMENT;
+  if (inter <= 0 || in_stride < 2LL * inter || out_stride < inter) return FE_BAD_ARGUMENT;
   const size_t total = (size_t)tokens * inter;
   const int threads = 256;
-  if (dtype == FE_BF16 && inter % 8 == 0 && ((((uintptr_t)gate_up) | ((uintptr_t)out)) & 15) == 0) {
+  if (dtype == FE_BF16 && inter % 8 == 0 && in_stride % 8 == 0 && out_stride % 8 == 0 &&
+      ((((uintptr_t)gate_up) | ((uintptr_t)out)) & 15) == 0) {
     const size_t total8 = total / 8;
     const size_t want8 = (total8 + threads - 1) / threads;
     swiglu_bf16x8_kernel<<<(int)(want8 < 16384 ? want8 : 16384), threads, 0, stream>>>(
-        (const bf16_t*)gate_up, (bf16_t*)out, inter / 8, total8);
+        (const bf16_t*)gate_up, (size_t)in_stride / 8, (bf16_t*)out, (size_t)out_stride / 8, inter / 8, total8);
     return fe_check_launch();
   }
   size_t want = (total + threads - 1) / threads;
   const int blocks = (int)(want < 8192 ? want : 8192);
   if (dtype == FE_F32)
-    swiglu_kernel<float><<<blocks, threads, 0, stream>>>((const float*)gate_up, (float*)out, inter, total);
+    swiglu_kernel<float><<<blocks, threads, 0, stream>>>((const float*)gate_up, (size_t)in_stride, (float*)out, (size_t)out_stride, inter, total);
   else if (dtype == FE_BF16)
-    swiglu_kernel<bf16_t><<<blocks, threads, 0, stream>>>((const bf16_t*)gate_up, (bf16_t*)out, inter, total);
+    swiglu_kernel<bf16_t><<<blocks, threads, 0, stream>>>((const bf16_t*)gate_up, (size_t)in_stride, (bf16_t*)out, (size_t)out_stride, inter, total);
   else
     return FE_BAD_ARGUMENT;
   return fe_check_launch();

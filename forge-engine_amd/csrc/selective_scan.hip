@@ -5,6 +5,7 @@
 //                        step from the sequence's state slot (its last taps - 1 rows of u, float32),
 //                        rows before the sequence's start zeros (a slot is cleared when a request
 //                        begins).  The state is moved on afterwards by fe_conv_state_update.
+//   fe_causal_conv_step: the same for a step of single tokens, the state's move in the same launch.
 //   fe_selective_scan:   per sequence, channel c and state n, token after token,
 //                          dt   = softplus(dt_lin[t][c] + dt_bias[c])
 //                          S[c][n] <- exp(dt * A[c][n]) * S[c][n] + dt * x[t][c] * B[t][n]
@@ -147,6 +148,57 @@ extern "C" int fe_causal_conv_act(const void* u, int dtype, long long u_stride, 
     if (wide) LAUNCH(bf16_t, 4); else LAUNCH(bf16_t, 1);
   }
 #undef LAUNCH
+  return fe_check_launch();
+}
+
+// A step in which every sequence brings one token: a thread per (sequence, channel) reads the state's rows, writes the
+// output and moves the state on itself (nobody else reads its channel's rows), one launch in all.
+template <typename T>
+__global__ __launch_bounds__(SS_THREADS) void causal_conv_step_kernel(
+    const T* __restrict__ u, size_t u_stride, const float* __restrict__ w, const float* __restrict__ bias,
+    float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ state_slots, T* __restrict__ out,
+    int channels, int taps, int slots, int act, int tokens) {
+  const int seq = blockIdx.x;
+  const int c = blockIdx.y * SS_THREADS + threadIdx.x;
+  const int t = cu_q[seq];
+  const int slot = state_slots[seq];
+  if (cu_q[seq + 1] != t + 1 || t >= tokens || slot < 0 || slot >= slots || c >= channels) return;
+  float* kept = state + (size_t)slot * (taps - 1) * channels + c;
+  float row[CONV_MAX_TAPS];
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS; ++j)
+    row[j] = j < taps - 1 ? kept[(size_t)j * channels] : 0.f;
+  const float newest = load_as_float(u + (size_t)t * u_stride + c);
+  float acc = bias ? bias[c] : 0.f;
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS; ++j) {
+    if (j == taps - 1) row[j] = newest;
+    if (j < taps) acc = fmaf(w[(size_t)c * taps + j], row[j], acc);
+  }
+#pragma unroll
+  for (int j = 0; j + 1 < CONV_MAX_TAPS; ++j)
+    if (j < taps - 1) kept[(size_t)j * channels] = row[j + 1];
+  if (act == 1) acc = acc / (1.f + expf(-acc));
+  store_from_float(out + (size_t)t * channels + c, acc);
+}
+
+extern "C" int fe_causal_conv_step(const void* u, int dtype, long long u_stride, const float* w, const float* bias, float* state,
+                                   const int* cu_q, const int* state_slots, void* out, int tokens, int num_seqs, int channels,
+                                   int taps, int slots, int act, hipStream_t stream) {
+  if (tokens <= 0 || num_seqs <= 0) return FE_OK;
+  if (channels <= 0 || taps < 2 || taps > CONV_MAX_TAPS || u_stride < channels || !w || !state || slots < 1 || act < 0 || act > 1)
+    return FE_BAD_ARGUMENT;
+  const int channel_blocks = (channels + SS_THREADS - 1) / SS_THREADS;
+  if (channel_blocks > 65535) return FE_BAD_ARGUMENT;
+  const dim3 grid(num_seqs, channel_blocks);
+  if (dtype == FE_F32)
+    causal_conv_step_kernel<float><<<grid, SS_THREADS, 0, stream>>>((const float*)u, (size_t)u_stride, w, bias, state, cu_q,
+                                                                    state_slots, (float*)out, channels, taps, slots, act, tokens);
+  else if (dtype == FE_BF16)
+    causal_conv_step_kernel<bf16_t><<<grid, SS_THREADS, 0, stream>>>((const bf16_t*)u, (size_t)u_stride, w, bias, state, cu_q,
+                                                                     state_slots, (bf16_t*)out, channels, taps, slots, act, tokens);
+  else
+    return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }
 

@@ -425,27 +425,58 @@ extern "C" int fe_add_bias(float* update, const float* bias, int rows, int width
 }
 
 // ---------------------------------------------------------------- output gate
-// out[t][c] *= sigmoid(gate[t][c / share]), gate rows `gate_stride` elements apart; `share` consecutive
-// outputs take one gate (1: a gate per element; a head's width: a gate per head)
+// out[t][c] = x[t][c] * sigmoid(gate[t][c / share]) * factor, gate and out rows of any stride (out may be x itself);
+// `share` consecutive outputs take one gate (1: a gate per element; a head's width: a gate per head)
 template <typename T>
-__global__ void sigmoid_gate_kernel(T* __restrict__ out, const T* __restrict__ gate, size_t gate_stride, int width,
-                                    long long count, int share) {
+__global__ void sigmoid_gate_kernel(const T* x, const T* __restrict__ gate, size_t gate_stride, T* out, size_t out_stride,
+                                    int width, long long count, int share, float factor) {
   const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= count) return;
   const long long t = i / width;
   const int c = (int)(i - t * width);
   const float g = load_as_float(gate + (size_t)t * gate_stride + c / share);
-  store_from_float(out + i, load_as_float(out + i) / (1.f + expf(-g)));
+  store_from_float(out + (size_t)t * out_stride + c, load_as_float(x + i) / (1.f + expf(-g)) * factor);
 }
 
-extern "C" int fe_sigmoid_gate(void* out, const void* gate, long long gate_stride, int dtype, int rows, int width,
-                               int share, hipStream_t stream) {
+// bfloat16, a gate per element, everything in 16-byte pieces
+__global__ __launch_bounds__(256) void sigmoid_gate_bf16x8_kernel(const uint4* x, const bf16_t* __restrict__ gate, size_t gate_stride,
+                                                                  bf16_t* out, size_t out_stride, int width8, long long count8,
+                                                                  float factor) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= count8) return;
+  const long long t = i / width8;
+  const int c = (int)(i - t * width8) * 8;
+  const uint4 a = x[i], g = *(const uint4*)(gate + (size_t)t * gate_stride + c);
+  const uint32_t aw[4] = {a.x, a.y, a.z, a.w}, gw[4] = {g.x, g.y, g.z, g.w};
+  uint32_t ow[4];
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float lo = __uint_as_float(aw[k] << 16) / (1.f + expf(-__uint_as_float(gw[k] << 16))) * factor;
+    const float hi = __uint_as_float(aw[k] & 0xffff0000u) / (1.f + expf(-__uint_as_float(gw[k] & 0xffff0000u))) * factor;
+    ow[k] = (uint32_t)float_to_bf16(lo) | ((uint32_t)float_to_bf16(hi) << 16);
+  }
+  *(uint4*)(out + (size_t)t * out_stride + c) = make_uint4(ow[0], ow[1], ow[2], ow[3]);
+}
+
+extern "C" int fe_sigmoid_gate(const void* x, const void* gate, long long gate_stride, void* out, long long out_stride, int dtype,
+                               int rows, int width, int share, float factor, hipStream_t stream) {
   if (rows <= 0) return FE_OK;
-  if (width <= 0 || share < 1 || width % share || gate_stride < width / share) return FE_BAD_ARGUMENT;
+  if (width <= 0 || share < 1 || width % share || gate_stride < width / share || out_stride < width) return FE_BAD_ARGUMENT;
   const long long count = (long long)rows * width;
   const int blocks = (int)((count + 255) / 256);
-  if (dtype == FE_F32) sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)out, (const float*)gate, (size_t)gate_stride, width, count, share);
-  else if (dtype == FE_BF16) sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)gate, (size_t)gate_stride, width, count, share);
+  if (dtype == FE_BF16 && share == 1 && width % 8 == 0 && gate_stride % 8 == 0 && out_stride % 8 == 0 &&
+      (((uintptr_t)x | (uintptr_t)gate | (uintptr_t)out) & 15) == 0) {
+    const long long count8 = count / 8;
+    sigmoid_gate_bf16x8_kernel<<<(int)((count8 + 255) / 256), 256, 0, stream>>>(
+        (const uint4*)x, (const bf16_t*)gate, (size_t)gate_stride, (bf16_t*)out, (size_t)out_stride, width / 8, count8, factor);
+    return fe_check_launch();
+  }
+  if (dtype == FE_F32)
+    sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((const float*)x, (const float*)gate, (size_t)gate_stride, (float*)out,
+                                                           (size_t)out_stride, width, count, share, factor);
+  else if (dtype == FE_BF16)
+    sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)gate, (size_t)gate_stride, (bf16_t*)out,
+                                                            (size_t)out_stride, width, count, share, factor);
   else return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }
@@ -550,8 +581,8 @@ __device__ __forceinline__ float gate_act(float g, int act) {
 template <typename TO>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     const float* __restrict__ o, const float* __restrict__ weight, int weight_len, const TO* __restrict__ gate,
-    size_t gate_stride, TO* __restrict__ out, const float* __restrict__ floor_, int tokens, int heads, int dim,
-    int extra, float eps, int act) {
+    size_t gate_stride, TO* __restrict__ out, size_t out_stride, const float* __restrict__ floor_, int tokens, int heads,
+    int dim, int extra, float eps, int act) {
   const int lane = threadIdx.x & 63;
   const long long pair = (long long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (pair >= (long long)tokens * heads) return;
@@ -570,25 +601,151 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     float v = row[c] * inv;
     if (weight) v *= weight[weight_len == dim ? c : h * dim + c];
     if (gate) v *= gate_act(load_as_float(gate + (size_t)t * gate_stride + h * dim + c), act);
-    store_from_float(out + ((size_t)t * heads + h) * dim + c, v);
+    store_from_float(out + (size_t)t * out_stride + (size_t)h * dim + c, v);
   }
 }
 
 extern "C" int fe_head_norm_gate(const float* o, const float* weight, int weight_len, const void* gate,
-                                 long long gate_stride, void* out, int out_dtype, const float* floor_, int tokens,
+                                 long long gate_stride, void* out, long long out_stride, int out_dtype, const float* floor_, int tokens,
                                  int heads, int dim, int extra, float eps, int act, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
-  if (heads <= 0 || dim <= 0 || extra < 0 || extra > 1 || !(eps > 0.f) || act < 0 || act > 2) return FE_BAD_ARGUMENT;
+  if (heads <= 0 || dim <= 0 || extra < 0 || extra > 1 || !(eps > 0.f) || act < 0 || act > 2 || out_stride < (long long)heads * dim)
+    return FE_BAD_ARGUMENT;
   if (weight && weight_len != dim && weight_len != heads * dim) return FE_BAD_ARGUMENT;
   if (extra && floor_ == nullptr) return FE_BAD_ARGUMENT;
   const long long pairs = (long long)tokens * heads;
   const int blocks = (int)((pairs + 3) / 4);
   if (out_dtype == FE_F32)
     head_norm_gate_kernel<float><<<blocks, 256, 0, stream>>>(o, weight, weight_len, (const float*)gate, (size_t)gate_stride,
-                                                              (float*)out, floor_, tokens, heads, dim, extra, eps, act);
+                                                              (float*)out, (size_t)out_stride, floor_, tokens, heads, dim, extra, eps, act);
   else if (out_dtype == FE_BF16)
     head_norm_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>(o, weight, weight_len, (const bf16_t*)gate, (size_t)gate_stride,
-                                                               (bf16_t*)out, floor_, tokens, heads, dim, extra, eps, act);
+                                                               (bf16_t*)out, (size_t)out_stride, floor_, tokens, heads, dim, extra, eps, act);
+  else return FE_BAD_ARGUMENT;
+  return fe_check_launch();
+}
+
+// ---------------------------------------------------------------- gate, then a norm in equal parts of the row
+// u = y * silu(z);  out = u / sqrt(mean(u^2) + eps) * weight, the mean over each of `groups` equal parts of a row.
+// y float32 [rows][width] dense; z and out in the compute dtype, rows of any stride.  Block = one part of one row; a
+// part's first 4 x 4 elements a thread stay in registers between the passes.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ z, size_t z_stride,
+                                                               const float* __restrict__ weight, T* __restrict__ out,
+                                                               size_t out_stride, int width, int part, float eps) {
+  constexpr int KEEP = 4;
+  struct alignas(sizeof(T) * VEC) Pack { T e[VEC]; };
+  struct alignas(4 * VEC) PackF { float e[VEC]; };
+  __shared__ float scratch[16];
+  const size_t row = blockIdx.x;
+  const int first = blockIdx.y * part;
+  const float* yr = y + row * width + first;
+  const T* zr = z + row * z_stride + first;
+  T* orow = out + row * out_stride + first;
+  const float* wr = weight + first;
+  const int step = blockDim.x * VEC;
+  auto gated = [&](int c, float (&u)[VEC]) {
+    const PackF a = *(const PackF*)(yr + c);
+    const Pack g = *(const Pack*)(zr + c);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) {
+      const float v = load_as_float(&g.e[i]);
+      u[i] = a.e[i] * (v / (1.f + expf(-v)));
+    }
+  };
+  float kept[KEEP][VEC];
+  float squares = 0.f;
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int c = threadIdx.x * VEC + n * step;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) kept[n][i] = 0.f;
+    if (c < part) gated(c, kept[n]);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) squares = fmaf(kept[n][i], kept[n][i], squares);
+  }
+  for (int c = threadIdx.x * VEC + KEEP * step; c < part; c += step) {
+    float u[VEC];
+    gated(c, u);
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) squares = fmaf(u[i], u[i], squares);
+  }
+  const float inv = 1.f / sqrtf(block_sum<true>(squares, scratch) / (float)part + eps);
+  auto store = [&](int c, const float (&u)[VEC]) {
+    const PackF w = *(const PackF*)(wr + c);
+    Pack o;
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) store_from_float(&o.e[i], u[i] * inv * w.e[i]);
+    *(Pack*)(orow + c) = o;
+  };
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int c = threadIdx.x * VEC + n * step;
+    if (c < part) store(c, kept[n]);
+  }
+  for (int c = threadIdx.x * VEC + KEEP * step; c < part; c += step) {
+    float u[VEC];
+    gated(c, u);
+    store(c, u);
+  }
+}
+
+extern "C" int fe_gated_group_norm(const float* y, const void* z, long long z_stride, const float* weight, void* out,
+                                   long long out_stride, int dtype, int rows, int width, int groups, float eps, hipStream_t stream) {
+  if (rows <= 0) return FE_OK;
+  if (width <= 0 || groups < 1 || groups > 65535 || width % groups || z_stride < width || out_stride < width || !weight || !(eps > 0.f))
+    return FE_BAD_ARGUMENT;
+  const int part = width / groups;
+  const size_t element = dtype == FE_F32 ? 4 : 2;
+  const bool wide = part % 4 == 0 && z_stride % 4 == 0 && out_stride % 4 == 0 &&
+                    (((uintptr_t)y | (uintptr_t)weight) & 15) == 0 && ((uintptr_t)z | (uintptr_t)out) % (4 * element) == 0;
+  const dim3 grid(rows, groups);
+  const int vec = wide ? 4 : 1;
+  const int threads = part <= 64 * vec * 4 ? 64 : 256;
+#define LAUNCH(T, VEC)                                                                                                        \
+  gated_group_norm_kernel<T, VEC><<<grid, threads, 0, stream>>>(y, (const T*)z, (size_t)z_stride, weight, (T*)out, (size_t)out_stride, \
+                                                                width, part, eps)
+  if (dtype == FE_F32) {
+    if (wide) LAUNCH(float, 4); else LAUNCH(float, 1);
+  } else if (dtype == FE_BF16) {
+    if (wide) LAUNCH(bf16_t, 4); else LAUNCH(bf16_t, 1);
+  } else {
+    return FE_BAD_ARGUMENT;
+  }
+#undef LAUNCH
+  return fe_check_launch();
+}
+
+// ---------------------------------------------------------------- the stream, updates added, in the compute dtype
+// out[t][c] = h[t][c] + update (in parts that are added up in order, or none) + bias (or none); out rows of any stride
+template <typename T>
+__global__ void stream_sum_cast_kernel(const float* __restrict__ h, const float* __restrict__ update, int parts, size_t part_stride,
+                                       const float* __restrict__ bias, T* __restrict__ out, size_t out_stride, int width,
+                                       long long count) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= count) return;
+  const long long t = i / width;
+  const int c = (int)(i - t * width);
+  float v = h[i];
+  if (update) {
+    float sum = 0.f;
+    for (int p = 0; p < parts; ++p) sum += update[p * part_stride + i];
+    v += sum;
+  }
+  if (bias) v += bias[c];
+  store_from_float(out + (size_t)t * out_stride + c, v);
+}
+
+extern "C" int fe_stream_sum_cast(const float* h, const float* update, int parts, const float* bias, void* out, long long out_stride,
+                                  int dtype, int rows, int width, hipStream_t stream) {
+  if (rows <= 0) return FE_OK;
+  if (width <= 0 || out_stride < width || (update && parts < 1)) return FE_BAD_ARGUMENT;
+  const long long count = (long long)rows * width;
+  const int blocks = (int)((count + 255) / 256);
+  if (dtype == FE_F32)
+    stream_sum_cast_kernel<float><<<blocks, 256, 0, stream>>>(h, update, parts, (size_t)count, bias, (float*)out, (size_t)out_stride, width, count);
+  else if (dtype == FE_BF16)
+    stream_sum_cast_kernel<bf16_t><<<blocks, 256, 0, stream>>>(h, update, parts, (size_t)count, bias, (bf16_t*)out, (size_t)out_stride, width, count);
   else return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }

@@ -9,7 +9,7 @@ implementation: without a GPU or without the compiled library a call raises.
 from __future__ import annotations
 
 import threading
-from ctypes import c_float, c_int, c_longlong, c_void_p
+from ctypes import c_double, c_float, c_int, c_longlong, c_void_p
 
 import numpy as np
 import torch
@@ -133,14 +133,14 @@ def add_rows(h: Tensor, delta: Tensor) -> Tensor:
 
 
 def swiglu(gate_up: Tensor, out: Tensor) -> Tensor:
-    """out[t, i] = silu(gate_up[t, i]) * gate_up[t, I + i]."""
-    _gpu(gate_up, "gate_up")
-    _gpu(out, "out", gate_up.dtype)
+    """out[t, i] = silu(gate_up[t, i]) * gate_up[t, I + i]; rows of any stride."""
     tokens, two_inter = gate_up.shape
-    if two_inter % 2 or out.shape != (tokens, two_inter // 2):
-        raise KernelError(f"out must be [{tokens}, {two_inter // 2}], got {tuple(out.shape)}")
-    _call("rowwise", "fe_swiglu", _ptr(gate_up), _ptr(out), c_int(_code(out.dtype)), c_int(tokens),
-          c_int(two_inter // 2), _stream())
+    in_stride = _strided_rows(gate_up, "gate_up", two_inter)
+    if two_inter % 2 or out.shape != (tokens, two_inter // 2) or out.dtype != gate_up.dtype:
+        raise KernelError(f"out must be [{tokens}, {two_inter // 2}] in gate_up's dtype, got {tuple(out.shape)}")
+    out_stride = _strided_rows(out, "out", two_inter // 2)
+    _call("rowwise", "fe_swiglu", _ptr(gate_up), c_longlong(in_stride), _ptr(out), c_longlong(out_stride), c_int(_code(out.dtype)),
+          c_int(tokens), c_int(two_inter // 2), _stream())
     return out
 
 
@@ -1216,12 +1216,12 @@ def _strided_rows(t: Tensor, name: str, width: int) -> int:
 def head_norm_gate(o: Tensor, weight: Tensor | None, gate: Tensor | None, out: Tensor, *, heads: int, dim: int,
                    eps: float, act: str = "none", extra: int = 0, floor: Tensor | None = None) -> Tensor:
     """out[t, h] = o[t, h, :dim] / rms * weight * act(gate[t, h]) per head, rms over dim (epsilon
-    inside the root).  o float32 [T, heads, dim + extra]; with ``extra`` = 1 the last column is a
+    inside the root); out [T, heads * dim], rows of any stride.  o float32 [T, heads, dim + extra]; with ``extra`` = 1 the last column is a
     normaliser n and the head is first divided by max(|n|, floor[t, h]) + 1e-6.  weight float32
     of heads * dim entries, or of dim entries shared by the heads; gate [T, heads * dim] rows of
     any stride, in the compute dtype."""
     _gpu(o, "o", torch.float32)
-    _gpu(out, "out")
+    out_stride = _strided_rows(out, "out", heads * dim)
     tokens = o.shape[0]
     if o.shape != (tokens, heads, dim + extra) or extra not in (0, 1) or out.shape != (tokens, heads * dim):
         raise KernelError(f"o must be [T, {heads}, {dim + extra}] and out [T, {heads * dim}]")
@@ -1243,7 +1243,7 @@ def head_norm_gate(o: Tensor, weight: Tensor | None, gate: Tensor | None, out: T
         if floor.shape != (tokens, heads):
             raise KernelError(f"floor must be [T, {heads}]")
     _call("stream_ops", "fe_head_norm_gate", _ptr(o), _ptr(weight), c_int(weight_len), _ptr(gate), c_longlong(gate_stride),
-          _ptr(out), c_int(_code(out.dtype)), _ptr(floor if extra else None), c_int(tokens), c_int(heads), c_int(dim),
+          _ptr(out), c_longlong(out_stride), c_int(_code(out.dtype)), _ptr(floor if extra else None), c_int(tokens), c_int(heads), c_int(dim),
           c_int(extra), c_float(eps), c_int(_ACTS[act]), _stream())
     return out
 
@@ -1256,7 +1256,7 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
                          kv_heads: int, head_dim: int, value_dim: int, rotary_dim: int, unit_norm_eps: float | None,
                          taps: int, v_from: Tensor | None = None, v_mix: float = 0.0, v_keep: Tensor | None = None,
                          norm_weight_q: Tensor | None = None, norm_weight_k: Tensor | None = None,
-                         norm_first: bool = False) -> None:
+                         norm_first: bool = False, q_temp: tuple[float, float] | None = None) -> None:
     """From the projection's output to queries and cached keys and values in one kernel: a short
     projection's bias (float32 [channels] or None: the product before has none), a short causal
     convolution over time on every q, k and v channel (``taps`` > 0: y_t = sum_j c[:, j] *
@@ -1269,7 +1269,8 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
     the same tokens): the values become ``(1 - v_mix) v + v_mix v_from`` before they are stored; ``v_keep`` (same
     shape) receives the values as stored, for layers that lean on this one's.  ``norm_weight_q`` / ``norm_weight_k``
     (float32 [head_dim], shared by the heads): the unit norm's result times a weight per dim, an RMS norm;
-    ``norm_first``: the norm comes before the rotation instead of behind it."""
+    ``norm_first``: the norm comes before the rotation instead of behind it.  ``q_temp`` (coef, every): queries at
+    position p are multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)`` last of all."""
     channels = (q_heads + kv_heads) * head_dim + kv_heads * value_dim
     for name, w in (("norm_weight_q", norm_weight_q), ("norm_weight_k", norm_weight_k)):
         if w is not None:
@@ -1278,6 +1279,8 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
                 raise KernelError(f"{name} must be [{head_dim}] and comes with a unit norm")
     if norm_first and unit_norm_eps is None:
         raise KernelError("norm_first comes with a unit norm")
+    if q_temp is not None and not q_temp[1] > 0.0:
+        raise KernelError("a temperature's run of positions must be positive")
     _gpu(qkv, "qkv", contiguous=False)
     tokens = qkv.shape[0]
     if qkv.dim() != 2 or qkv.shape[1] < channels or qkv.stride(1) != 1:
@@ -1332,7 +1335,7 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
           c_int(value_dim), c_int(rotary_dim), c_float(unit_norm_eps if unit_norm_eps is not None else 0.0),
           c_int(1 if unit_norm_eps is not None else 0), c_int(taps), c_int(block_size), c_int(num_blocks), c_int(slots),
           _ptr(v_from), c_float(v_mix), _ptr(v_keep), _ptr(norm_weight_q), _ptr(norm_weight_k), c_int(1 if norm_first else 0),
-          _stream())
+          c_float(q_temp[0] if q_temp is not None else 0.0), c_double(q_temp[1] if q_temp is not None else 0.0), _stream())
     if taps > 1:
         _call("conv_rope", "fe_conv_state_update", _ptr(qkv), c_int(_code(qkv.dtype)), c_longlong(stride), _ptr(bias), _ptr(conv_state),
               _ptr(cu_q), _ptr(state_slots), c_int(num_seqs), c_int(channels), c_int(taps), c_int(slots), c_int(tokens),
@@ -1344,7 +1347,7 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
                      value_dim: int, scale: float, window: int | None = None, chunk: int | None = None,
                      sink: Tensor | None = None, gate: Tensor | None = None, num_decode: int | None = None,
                      max_ctx: int | None = None, softcap: float | None = None, head_gate: bool = False,
-                     slopes: Tensor | None = None, dist_bias: Tensor | None = None) -> Tensor:
+                     slopes: Tensor | None = None, dist_bias: Tensor | None = None, factor: float = 1.0) -> Tensor:
     """Paged grouped-query attention with the masks and softmax forms beyond the causal one: the
     query at position p reads keys j <= p with j > p - window (``window``) and j >= p - p % chunk
     (``chunk``); ``sink`` (float32 [Hq]) adds exp(sink_h) to head h's softmax denominator, with
@@ -1353,13 +1356,13 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     ``softcap``: scores, after the scale, become cap * tanh(score / cap); ``slopes`` (float32 [Hq]): head h's score
     of key j loses slopes[h] * (p - j); ``dist_bias`` (float32 [Hq, span]): head h's score of key j gains
     dist_bias[h, min(p - j, span - 1)] (after the scale, which does not multiply it); ``value_pages`` None: a key's
-    first ``value_dim`` dims are its value (a cache of keys only).  out [T, Hq * Dv].  Scores and softmax
+    first ``value_dim`` dims are its value (a cache of keys only).  out [T, Hq * Dv]; with a gate its rows may have any
+    stride, and ``factor`` multiplies the gated result.  Scores and softmax
     float32.  A bfloat16 cache with keys and values of 64 or 128 elements, groups up to 8 and pages of
     a power of two >= 16 goes to the matrix-core kernels of ``paged_attention`` (single tokens and
     portions each to its own), with the gate in a small kernel behind them; everything else, and
     the float32 mode, to the vector-ALU kernel that does all of it in one launch."""
     _gpu(q, "q", contiguous=False)
-    _gpu(out, "out", q.dtype)
     _gpu(key_pages, "key_pages", q.dtype)
     if value_pages is not None:
         _gpu(value_pages, "value_pages", q.dtype)
@@ -1368,8 +1371,11 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     _gpu(block_table, "block_table", torch.int32)
     tokens = q.shape[0]
     q_stride = _strided_rows(q, "q", q_heads * head_dim)
-    if out.shape != (tokens, q_heads * value_dim):
-        raise KernelError(f"out must be [{tokens}, {q_heads * value_dim}], got {tuple(out.shape)}")
+    out_stride = _strided_rows(out, "out", q_heads * value_dim)
+    if out.shape != (tokens, q_heads * value_dim) or out.dtype != q.dtype:
+        raise KernelError(f"out must be [{tokens}, {q_heads * value_dim}] in q's dtype, got {tuple(out.shape)}")
+    if gate is None and (factor != 1.0 or not out.is_contiguous()):
+        raise KernelError("a factor and rows of another stride come with a gate")
     if q_heads % kv_heads or not 1 <= head_dim <= MASKED_MAX_KEY_DIM or not 1 <= value_dim <= MASKED_MAX_VALUE_DIM:
         raise KernelError(f"query heads must be a multiple of kv heads, keys of up to {MASKED_MAX_KEY_DIM} and values of up to {MASKED_MAX_VALUE_DIM} dims")
     if value_pages is None and value_dim > head_dim:
@@ -1410,16 +1416,18 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
             and not (slopes is not None and softcap is not None) and value_pages is not None
             and not (dist_bias is not None and (slopes is not None or softcap is not None))
             and block_size >= 16 and block_size & (block_size - 1) == 0 and q.data_ptr() % 16 == 0 and q_stride % 8 == 0):
-        paged_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table, num_seqs=num_seqs, max_q_len=max_q_len,
+        attended = out if out.is_contiguous() else torch.empty_like(out, memory_format=torch.contiguous_format)
+        paged_attention(q, key_pages, value_pages, attended, cu_q, ctx_len, block_table, num_seqs=num_seqs, max_q_len=max_q_len,
                         q_heads=q_heads, kv_heads=kv_heads, head_dim=head_dim, scale=scale, window=window,
                         num_decode=num_decode, max_ctx=max_ctx, chunk=chunk, sink=sink, softcap=softcap, slopes=slopes,
                         dist_bias=dist_bias)
         if gate is not None:
-            _call("stream_ops", "fe_sigmoid_gate", _ptr(out), _ptr(gate), c_longlong(gate_stride), c_int(_code(out.dtype)),
-                  c_int(tokens), c_int(q_heads * value_dim), c_int(value_dim if head_gate else 1), _stream())
+            _call("stream_ops", "fe_sigmoid_gate", _ptr(attended), _ptr(gate), c_longlong(gate_stride), _ptr(out), c_longlong(out_stride),
+                  c_int(_code(out.dtype)), c_int(tokens), c_int(q_heads * value_dim), c_int(value_dim if head_gate else 1),
+                  c_float(factor), _stream())
         return out
     _call("attention_masked", "fe_masked_attention", _ptr(q), c_int(_code(q.dtype)), c_longlong(q_stride), _ptr(key_pages),
-          _ptr(value_pages), _ptr(out), _ptr(gate), c_longlong(gate_stride), _ptr(sink), _ptr(cu_q), _ptr(ctx_len),
+          _ptr(value_pages), _ptr(out), c_longlong(out_stride), c_float(factor), _ptr(gate), c_longlong(gate_stride), _ptr(sink), _ptr(cu_q), _ptr(ctx_len),
           _ptr(block_table), c_int(block_table.stride(0)), c_int(num_seqs), c_int(max_q_len), c_int(q_heads),
           c_int(kv_heads), c_int(head_dim), c_int(value_dim), c_int(block_size), c_int(num_blocks),
           c_int(window or 0), c_int(chunk or 0), c_float(scale), c_float(softcap or 0.0), c_int(1 if head_gate else 0),
@@ -1684,13 +1692,14 @@ def mlstm_gate_scan(gates: Tensor, bias: Tensor, cap: float, maximum: Tensor, cu
 
 def hyper_norm(streams: Tensor, update: Tensor | None, mix: Tensor | None, share: Tensor | None, read: Tensor | None,
                weight: Tensor | None, bias: Tensor | None, eps: float, out: Tensor | None, rows: Tensor | None = None,
-               store: bool = True, rms: bool = False) -> Tensor | None:
+               store: bool = True, rms: bool = False, shift: Tensor | None = None) -> Tensor | None:
     """The norm over S residual streams [S, T, W] (float32; S = 1: one plain stream), fused with the
     pending update (float32 [T, W] or [parts, T, W], added up in order):
     ``x_t <- sum_s mix[s, t] x_s + share[t] * update`` (mix None: the identity, share None: ones; written
     back unless ``store`` is False), ``u = sum_t read[t] x_t`` (None: the plain sum), and ``out`` =
     the layer norm of u with weight and bias (``rms``: the RMS norm, no mean, bias optional), of the
-    rows listed in ``rows`` if given.  ``out`` None: the update is applied and nothing else."""
+    rows listed in ``rows`` if given.  ``out`` None: the update is applied and nothing else.  ``shift`` (float32 [W]): a
+    bias on the update (or instead of one)."""
     _gpu(streams, "streams", torch.float32)
     if streams.dim() != 3 or not 1 <= streams.shape[0] <= 8:
         raise KernelError(f"streams must be [1..8, T, W], got {tuple(streams.shape)}")
@@ -1700,10 +1709,10 @@ def hyper_norm(streams: Tensor, update: Tensor | None, mix: Tensor | None, share
     parts = 0
     if update is not None:
         parts = _parts_of(update, total_rows, width, "update")
-    elif out is None:
+    elif out is None and shift is None:
         raise KernelError("nothing to do: neither an update nor an output")
     for name, t, shape in (("mix", mix, (count, count)), ("share", share, (count,)), ("read", read, (count,)),
-                           ("weight", weight, (width,)), ("bias", bias, (width,))):
+                           ("weight", weight, (width,)), ("bias", bias, (width,)), ("shift", shift, (width,))):
         if t is not None:
             _gpu(t, name, torch.float32)
             if tuple(t.shape) != shape:
@@ -1712,16 +1721,16 @@ def hyper_norm(streams: Tensor, update: Tensor | None, mix: Tensor | None, share
     if rows is not None:
         _gpu(rows, "rows", torch.int32)
         n_rows = rows.numel()
-        if store and update is not None:
+        if store and (update is not None or shift is not None):
             raise KernelError("store with a row list is not allowed (rows may repeat)")
     if out is not None:
         _gpu(out, "out")
         if out.shape != (n_rows, width) or weight is None or not eps > 0.0:
             raise KernelError(f"out must be [{n_rows}, {width}] and come with a weight and a positive eps")
     _call("hyper", "fe_hyper_norm", _ptr(streams), c_longlong(total_rows * width), c_int(count), _ptr(update), c_int(parts),
-          c_longlong(total_rows * width), _ptr(mix), _ptr(share), _ptr(read), _ptr(weight), _ptr(bias), c_float(eps),
+          c_longlong(total_rows * width), _ptr(shift), _ptr(mix), _ptr(share), _ptr(read), _ptr(weight), _ptr(bias), c_float(eps),
           c_int(1 if rms else 0), _ptr(out), c_int(_code(out.dtype) if out is not None else FE_F32), _ptr(rows),
-          c_int(n_rows), c_int(width), c_int(1 if (store and update is not None) else 0), _stream())
+          c_int(n_rows), c_int(width), c_int(1 if (store and (update is not None or shift is not None)) else 0), _stream())
     return out
 
 
@@ -1821,7 +1830,7 @@ def whole_norm_rope_write(qkv: Tensor, q_weight: Tensor, k_weight: Tensor | None
 # ------------------------------------------------- a mixture of experts
 
 _SCORINGS = {"softmax": 0, "sigmoid": 1}
-_GATED_FORMS = {"bounded": 0, "silu": 1}
+_GATED_FORMS = {"bounded": 0, "silu": 1, "relu_squared": 2}
 
 
 def moe_route(x: Tensor, router_weight: Tensor, router_bias: Tensor | None, top: int, scoring: str = "softmax") -> tuple[Tensor, Tensor]:
@@ -1876,42 +1885,73 @@ def moe_route_grouped(x: Tensor, router_weight: Tensor, correction: Tensor | Non
     return chosen, weights, logits
 
 
-def moe_experts(x: Tensor, chosen: Tensor, weights: Tensor, gate_up: Tensor, down: Tensor, out: Tensor, *, limit: float = 0.0,
-                alpha: float = 1.0, extra: Tensor | None = None, form: str = "bounded", weight_input: bool = False) -> Tensor:
+def moe_plan_table(ids: Tensor, table: Tensor, experts: int) -> tuple[Tensor, Tensor, Tensor]:
+    """The plan of ``moe_experts`` where no router is asked: row ``ids[t]`` of ``table`` (int32 [vocab, top], numbers below
+    ``experts``) names token t's experts, each weighing 1 / top.  Returns (offsets [experts + 1], order [T * top],
+    weights float32 [T, top])."""
+    _gpu(ids, "ids", torch.int32)
+    _gpu(table, "table", torch.int32)
+    if ids.dim() != 1 or table.dim() != 2 or not 1 <= table.shape[1] <= min(16, experts) or experts > 1024:
+        raise KernelError("ids must be [T] and table [vocab, top] with top between 1 and min(experts, 16)")
+    tokens, (vocab, top) = ids.numel(), table.shape
+    offsets = torch.empty(experts + 1, dtype=torch.int32, device=ids.device)
+    order = torch.empty(tokens * top, dtype=torch.int32, device=ids.device)
+    weights = torch.empty((tokens, top), dtype=torch.float32, device=ids.device)
+    _call("moe", "fe_moe_plan_table", _ptr(ids), _ptr(table), c_int(vocab), c_int(tokens), c_int(top), c_int(experts), _ptr(offsets),
+          _ptr(order), _ptr(weights), c_float(1.0 / top), _stream())
+    return offsets, order, weights
+
+
+def moe_experts(x: Tensor, chosen: Tensor | None, weights: Tensor, gate_up: Tensor, down: Tensor, out: Tensor, *, limit: float = 0.0,
+                alpha: float = 1.0, extra: Tensor | None = None, form: str = "bounded", weight_input: bool = False,
+                plan: tuple[Tensor, Tensor] | None = None) -> Tensor:
     """out[k, t] = weights[t, k] * down[e] @ act, e = chosen[t, k], with ``act = min(g, limit) *
     sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + 1)``, ``g = gate_up[e, :F] @ x[t]``,
     ``u = gate_up[e, F:] @ x[t]``.  x [T, H]; gate_up [E, 2F, H]; down [E, H, F]; out float32 [top, T, H]
     (one part per choice).  ``extra`` (float32 [T, H] or [parts, T, H], added up in order): what every
     token gets beside its experts; it joins the first choice's part.  ``form`` "silu": ``act = silu(g) * u``, no
     bounds.  ``weight_input``: the routing weight scales the expert's input instead of its output (g and u are
-    multiplied by it before the activation, which is the same as multiplying x).  The pairs are sorted by
-    expert on the device and two grouped products run over the sorted rows."""
+    multiplied by it before the activation, which is the same as multiplying x).  ``form`` "relu_squared": one matrix
+    an expert, gate_up [E, F, H], ``act = max(gate_up[e] @ x[t], 0)^2``.  The pairs are sorted by
+    expert on the device and two grouped products run over the sorted rows; ``plan`` (offsets, order): they are sorted
+    already (``chosen`` is then not read)."""
     _gpu(x, "x")
-    _gpu(chosen, "chosen", torch.int32)
+    if plan is None:
+        _gpu(chosen, "chosen", torch.int32)
     _gpu(weights, "weights", torch.float32)
     _gpu(gate_up, "gate_up", x.dtype)
     _gpu(down, "down", x.dtype)
     _gpu(out, "out", torch.float32)
     tokens, hidden = x.shape
-    top = chosen.shape[1] if chosen.dim() == 2 else 0
-    if gate_up.dim() != 3 or gate_up.shape[2] != hidden or gate_up.shape[1] % 2:
-        raise KernelError(f"gate_up must be [experts, 2F, {hidden}], got {tuple(gate_up.shape)}")
-    experts, inner = gate_up.shape[0], gate_up.shape[1] // 2
+    top = weights.shape[1] if weights.dim() == 2 else 0
+    if form not in _GATED_FORMS:
+        raise KernelError("forms: " + ", ".join(_GATED_FORMS))
+    matrices = 1 if form == "relu_squared" else 2
+    if gate_up.dim() != 3 or gate_up.shape[2] != hidden or gate_up.shape[1] % matrices:
+        raise KernelError(f"gate_up must be [experts, {matrices}F, {hidden}], got {tuple(gate_up.shape)}")
+    experts, inner = gate_up.shape[0], gate_up.shape[1] // matrices
     if down.shape != (experts, hidden, inner):
         raise KernelError(f"down must be [{experts}, {hidden}, {inner}], got {tuple(down.shape)}")
-    if chosen.shape != (tokens, top) or weights.shape != (tokens, top) or not 1 <= top <= 16 or experts > 1024:
+    if (plan is None and chosen.shape != (tokens, top)) or weights.shape != (tokens, top) or not 1 <= top <= 16 or experts > 1024:
         raise KernelError("chosen and weights must be [T, top <= 16] and experts at most 1,024")
     if out.shape != (top, tokens, hidden):
         raise KernelError(f"out must be [{top}, {tokens}, {hidden}], got {tuple(out.shape)}")
-    if form not in _GATED_FORMS or (form == "bounded" and not limit > 0.0):
-        raise KernelError("the bounded activation needs a positive limit; forms: " + ", ".join(_GATED_FORMS))
+    if form == "bounded" and not limit > 0.0:
+        raise KernelError("the bounded activation needs a positive limit")
     extra_parts = 0 if extra is None else _parts_of(extra, tokens, hidden, "extra")
     pairs = tokens * top
-    offsets = torch.empty(experts + 1, dtype=torch.int32, device=x.device)
-    order = torch.empty(pairs, dtype=torch.int32, device=x.device)
     act = torch.empty((pairs, inner), dtype=x.dtype, device=x.device)
     code = c_int(_code(x.dtype))
-    _call("moe", "fe_moe_plan", _ptr(chosen), c_int(pairs), c_int(experts), _ptr(offsets), _ptr(order), _stream())
+    if plan is None:
+        offsets = torch.empty(experts + 1, dtype=torch.int32, device=x.device)
+        order = torch.empty(pairs, dtype=torch.int32, device=x.device)
+        _call("moe", "fe_moe_plan", _ptr(chosen), c_int(pairs), c_int(experts), _ptr(offsets), _ptr(order), _stream())
+    else:
+        offsets, order = plan
+        _gpu(offsets, "offsets", torch.int32)
+        _gpu(order, "order", torch.int32)
+        if offsets.numel() != experts + 1 or order.numel() != pairs:
+            raise KernelError(f"the plan must hold {experts + 1} offsets and {pairs} pairs")
     _call("moe", "fe_moe_gate_up", _ptr(x), _ptr(gate_up), code, _ptr(offsets), _ptr(order), _ptr(act), c_int(tokens), c_int(top),
           c_int(experts), c_int(hidden), c_int(inner), c_float(limit), c_float(alpha), c_int(_GATED_FORMS[form]),
           _ptr(weights if weight_input else None), _stream())
@@ -1972,12 +2012,13 @@ def gate_rows(update: Tensor, logits: Tensor, column: int) -> Tensor:
 
 
 def causal_conv_act(u: Tensor, weight: Tensor, bias: Tensor | None, state: Tensor | None, token_seq: Tensor, cu_q: Tensor,
-                    state_slots: Tensor, *, num_seqs: int, act: str = "silu") -> Tensor:
+                    state_slots: Tensor, *, num_seqs: int, act: str = "silu", single_tokens: bool = False) -> Tensor:
     """A short causal convolution over time on every channel, then the activation: ``y_t = act(b + sum_j
     w[:, j] * u_(t - taps + 1 + j))``.  u [T, >= channels] with any row stride (its first ``channels`` columns
     are read); weight float32 [channels, taps], the last column the token's own; bias float32 [channels] or
     None; state float32 [slots, taps - 1, channels]: every sequence's last taps - 1 rows of u, read for the
-    rows before the step and moved on afterwards (None with one tap).  Returns [T, channels] in u's dtype."""
+    rows before the step and moved on afterwards (None with one tap).  ``single_tokens``: every sequence brings one
+    token (one launch then does both).  Returns [T, channels] in u's dtype."""
     _gpu(u, "u", contiguous=False)
     _gpu(weight, "weight", torch.float32)
     if weight.dim() != 2 or not 1 <= weight.shape[1] <= 8:
@@ -2002,6 +2043,13 @@ def causal_conv_act(u: Tensor, weight: Tensor, bias: Tensor | None, state: Tenso
     slots = state.shape[0] if taps > 1 else 0
     out = torch.empty((tokens, channels), dtype=u.dtype, device=u.device)
     code = c_int(_code(u.dtype))
+    if single_tokens and taps > 1:
+        if tokens != num_seqs:
+            raise KernelError("a step of single tokens has one token a sequence")
+        _call("selective_scan", "fe_causal_conv_step", _ptr(u), code, c_longlong(stride), _ptr(weight), _ptr(bias), _ptr(state),
+              _ptr(cu_q), _ptr(state_slots), _ptr(out), c_int(tokens), c_int(num_seqs), c_int(channels), c_int(taps), c_int(slots),
+              c_int(_ACTS[act]), _stream())
+        return out
     _call("selective_scan", "fe_causal_conv_act", _ptr(u), code, c_longlong(stride), _ptr(weight), _ptr(bias),
           _ptr(state if taps > 1 else None), _ptr(token_seq), _ptr(cu_q), _ptr(state_slots), _ptr(out), c_int(tokens),
           c_int(channels), c_int(taps), c_int(slots), c_int(_ACTS[act]), _stream())
@@ -2083,4 +2131,165 @@ def selective_scan(x: Tensor, dt_lin: Tensor, dt_bias: Tensor, a: Tensor, bc: Te
           c_longlong(bc_stride), _ptr(d), _ptr(z), c_longlong(z_stride), _ptr(state), _ptr(cu_q), _ptr(state_slots), _ptr(out),
           c_int(tokens), c_int(num_seqs), c_int(channels), c_int(states), c_int(state.shape[0]), c_int(lanes), c_int(per_lane),
           c_int(segment), _ptr(seg_start), _ptr(seg_dt), c_int(rows), _stream())
+    return out
+
+
+# ------------------------------------------------- recurrences with one decay a head and token
+
+def rotary_table(positions: Tensor, inv_freq: Tensor) -> Tensor:
+    """(cos, sin) of ``float(position) * inv_freq[i]`` for every token of the step: float32 [T, len(inv_freq), 2]."""
+    _gpu(positions, "positions", torch.int32)
+    _gpu(inv_freq, "inv_freq", torch.float32)
+    if positions.dim() != 1 or inv_freq.dim() != 1 or inv_freq.numel() < 1:
+        raise KernelError("positions and inv_freq must be vectors")
+    table = torch.empty((positions.numel(), inv_freq.numel(), 2), dtype=torch.float32, device=positions.device)
+    _call("head_recurrence", "fe_rotary_table", _ptr(positions), _ptr(inv_freq), _ptr(table), c_int(positions.numel()),
+          c_int(inv_freq.numel()), _stream())
+    return table
+
+
+HEAD_SEGMENT = 128              # tokens a segment when a step's sequences are cut up (a multiple of 32)
+HEAD_SEGMENT_MIN_TOKENS = 128   # ... which happens when a sequence of the step may be this much longer than one token
+HEAD_STEP_MAX_NORMED = 1024     # widest head whose norm and gate the kernel for single tokens takes along
+
+
+def head_recurrence_segment(tokens: int, num_seqs: int) -> int:
+    """Tokens a segment, or 0 for one walk a sequence."""
+    if HEAD_SEGMENT <= 0 or tokens - num_seqs < HEAD_SEGMENT_MIN_TOKENS:
+        return 0
+    return HEAD_SEGMENT
+
+
+def _head_recurrence_checked(q, k, v, state, cu_q, state_slots, *, num_seqs, heads, share, key_dim, value_dim, rate, table,
+                             dt, dt_bias, skip):
+    """The operands' strides after every check that both kernels rest on."""
+    if heads < 1 or share < 1 or heads % share or not 1 <= key_dim <= 256 or value_dim < 1:
+        raise KernelError("heads must be a multiple of the heads that share q and k, key sizes 1 to 256")
+    tokens = q.shape[0]
+    strides = [_strided_rows(q, "q", heads // share * key_dim), _strided_rows(k, "k", heads // share * key_dim),
+               _strided_rows(v, "v", heads * value_dim)]
+    if k.dtype != q.dtype or v.dtype != q.dtype or k.shape[0] != tokens or v.shape[0] != tokens:
+        raise KernelError("q, k and v must share dtype and token count")
+    _gpu(state, "state", torch.float32)
+    if state.dim() != 4 or state.shape[1:] != (heads, value_dim, key_dim):
+        raise KernelError(f"state must be [slots, {heads}, {value_dim}, {key_dim}], got {tuple(state.shape)}")
+    _sequences(cu_q, state_slots, num_seqs)
+    for name, t in (("rate", rate), ("dt_bias", dt_bias), ("skip", skip)):
+        if t is not None:
+            _gpu(t, name, torch.float32)
+            if t.shape != (heads,):
+                raise KernelError(f"{name} must be [{heads}]")
+    rotary_dim = 0
+    if table is not None:
+        _gpu(table, "table", torch.float32)
+        rotary_dim = 2 * table.shape[1]
+        if table.dim() != 3 or table.shape[0] != tokens or table.shape[2] != 2 or rotary_dim > key_dim:
+            raise KernelError(f"table must be [{tokens}, <= {key_dim // 2}, 2]")
+    dt_stride = 0
+    if dt is not None:
+        dt_stride = _strided_rows(dt, "dt", heads)
+        if dt.dtype != q.dtype or dt.shape[0] != tokens or dt_bias is None:
+            raise KernelError("dt must be [T, heads] in q's dtype and comes with its bias")
+    return tokens, (*strides, dt_stride), rotary_dim
+
+
+def head_recurrence(q: Tensor, k: Tensor, v: Tensor, state: Tensor, cu_q: Tensor, state_slots: Tensor, *, num_seqs: int,
+                    heads: int, key_dim: int, value_dim: int, rate: Tensor, share: int = 1, table: Tensor | None = None,
+                    dt: Tensor | None = None, dt_bias: Tensor | None = None, skip: Tensor | None = None, q_scale: float = 1.0,
+                    k_scale: float = 1.0, single_tokens: bool = False, segment: int | None = None) -> Tensor:
+    """Per sequence and head: ``S_t = exp(l_t) S_(t-1) + b_t k_t v_t^T``, ``o_t = S_t^T q_t + skip_h v_t``; returns o,
+    float32 [T, heads, value_dim].  Without ``dt``: l_t = ``rate[h]``, b_t = 1.  With ``dt`` ([T, heads], q's dtype): the
+    step size ``softplus(dt + dt_bias[h])`` is b_t, and l_t is ``rate[h]`` times it.  q and k [T, heads // share *
+    key_dim] (``share`` neighbouring heads read the same ones), v [T, heads * value_dim], rows of any stride; q and k
+    are turned by ``table`` (``rotary_table``: dim i pairs with i + half, further dims pass) and multiplied by
+    ``q_scale`` / ``k_scale``.  ``state`` float32 [slots, heads, value_dim, key_dim], read at the step's start and
+    written at its end.  All of it is float32.  ``single_tokens``: every sequence brings one token.  ``segment``:
+    tokens a segment of long sequences (0: none, None: by the step's size)."""
+    tokens, strides, rotary_dim = _head_recurrence_checked(
+        q, k, v, state, cu_q, state_slots, num_seqs=num_seqs, heads=heads, share=share, key_dim=key_dim, value_dim=value_dim,
+        rate=rate, table=table, dt=dt, dt_bias=dt_bias, skip=skip)
+    out = torch.empty((tokens, heads, value_dim), dtype=torch.float32, device=q.device)
+    lead = (_ptr(q), _ptr(k), _ptr(v), _ptr(dt), c_int(_code(q.dtype)), *(c_longlong(s) for s in strides), _ptr(table),
+            c_int(rotary_dim), _ptr(rate), _ptr(dt_bias), _ptr(skip), c_float(q_scale), c_float(k_scale), _ptr(state),
+            c_int(state.shape[0]), _ptr(out))
+    if single_tokens:
+        if tokens != num_seqs:
+            raise KernelError("a step of single tokens has one token a sequence")
+        _call("head_recurrence", "fe_head_recurrence_step", *lead, _ptr(None), c_longlong(0), _ptr(None), c_longlong(0),
+              c_float(1.0), _ptr(cu_q), _ptr(state_slots), c_int(num_seqs), c_int(heads), c_int(share), c_int(key_dim),
+              c_int(value_dim), c_int(tokens), _stream())
+        return out
+    if segment is None:
+        segment = head_recurrence_segment(tokens, num_seqs)
+    seg_state = seg_sum = None
+    slots = 0
+    if segment:
+        if segment % 32:
+            raise KernelError("segments are multiples of 32 tokens")
+        slots = tokens // segment + num_seqs
+        seg_state = torch.empty((slots, heads, value_dim, key_dim), dtype=torch.float32, device=q.device)
+        seg_sum = torch.empty((slots, heads), dtype=torch.float64, device=q.device)
+    else:
+        segment = -(-tokens // 32) * 32
+    _call("head_recurrence", "fe_head_recurrence", *lead, _ptr(cu_q), _ptr(state_slots), c_int(num_seqs), c_int(heads),
+          c_int(share), c_int(key_dim), c_int(value_dim), c_int(tokens), c_int(segment), _ptr(seg_state), _ptr(seg_sum),
+          c_int(slots), _stream())
+    return out
+
+
+def head_recurrence_gated(q: Tensor, k: Tensor, v: Tensor, state: Tensor, cu_q: Tensor, state_slots: Tensor, gate: Tensor,
+                          out: Tensor, *, eps: float, num_seqs: int, heads: int, key_dim: int, value_dim: int, rate: Tensor,
+                          share: int = 1, table: Tensor | None = None, q_scale: float = 1.0, k_scale: float = 1.0) -> Tensor:
+    """``head_recurrence`` for a step of single tokens with its ending in the same launch: every head's o divided by its
+    root mean square (epsilon inside the root), times silu(gate), into ``out`` [T, heads * value_dim] (rows of any
+    stride, q's dtype)."""
+    tokens, strides, rotary_dim = _head_recurrence_checked(
+        q, k, v, state, cu_q, state_slots, num_seqs=num_seqs, heads=heads, share=share, key_dim=key_dim, value_dim=value_dim,
+        rate=rate, table=table, dt=None, dt_bias=None, skip=None)
+    gate_stride = _strided_rows(gate, "gate", heads * value_dim)
+    out_stride = _strided_rows(out, "out", heads * value_dim)
+    if tokens != num_seqs or gate.dtype != q.dtype or out.dtype != q.dtype or gate.shape[0] != tokens or out.shape[0] != tokens:
+        raise KernelError("gate and out must be in q's dtype with one token a sequence")
+    if value_dim > HEAD_STEP_MAX_NORMED:
+        raise KernelError(f"heads of up to {HEAD_STEP_MAX_NORMED} values")
+    _call("head_recurrence", "fe_head_recurrence_step", _ptr(q), _ptr(k), _ptr(v), _ptr(None), c_int(_code(q.dtype)),
+          *(c_longlong(s) for s in strides), _ptr(table), c_int(rotary_dim), _ptr(rate), _ptr(None), _ptr(None), c_float(q_scale),
+          c_float(k_scale), _ptr(state), c_int(state.shape[0]), _ptr(None), _ptr(gate), c_longlong(gate_stride), _ptr(out),
+          c_longlong(out_stride), c_float(eps), _ptr(cu_q), _ptr(state_slots), c_int(num_seqs), c_int(heads), c_int(share),
+          c_int(key_dim), c_int(value_dim), c_int(tokens), _stream())
+    return out
+
+
+def gated_group_norm(y: Tensor, z: Tensor, weight: Tensor, out: Tensor, *, groups: int, eps: float) -> Tensor:
+    """``u = y * silu(z)``, then every one of ``groups`` equal parts of a row divided by its own root mean square (epsilon
+    inside the root), times ``weight``.  y float32 [T, W]; z and out [T, W] in the compute dtype, rows of any stride;
+    weight float32 [W]."""
+    _gpu(y, "y", torch.float32)
+    _gpu(weight, "weight", torch.float32)
+    tokens, width = y.shape
+    z_stride, out_stride = _strided_rows(z, "z", width), _strided_rows(out, "out", width)
+    if z.shape[0] != tokens or out.shape[0] != tokens or z.dtype != out.dtype or weight.shape != (width,):
+        raise KernelError(f"z and out must be [{tokens}, {width}] in one dtype and weight [{width}]")
+    if groups < 1 or width % groups or not eps > 0.0:
+        raise KernelError("the groups must divide the row and eps be positive")
+    _call("stream_ops", "fe_gated_group_norm", _ptr(y), _ptr(z), c_longlong(z_stride), _ptr(weight), _ptr(out), c_longlong(out_stride),
+          c_int(_code(out.dtype)), c_int(tokens), c_int(width), c_int(groups), c_float(eps), _stream())
+    return out
+
+
+def stream_sum_cast(h: Tensor, update: Tensor | None, shift: Tensor | None, out: Tensor) -> Tensor:
+    """out = h + update + shift in out's dtype (rows of any stride); h float32 [T, W] stays as it is, the update
+    (float32 [T, W] or [parts, T, W], added up in order) and the bias ``shift`` (float32 [W]) may be None."""
+    _gpu(h, "h", torch.float32)
+    tokens, width = h.shape
+    parts = 0 if update is None else _parts_of(update, tokens, width, "update")
+    if shift is not None:
+        _gpu(shift, "shift", torch.float32)
+        if shift.shape != (width,):
+            raise KernelError(f"shift must be [{width}]")
+    out_stride = _strided_rows(out, "out", width)
+    if out.shape[0] != tokens:
+        raise KernelError(f"out must be [{tokens}, {width}]")
+    _call("stream_ops", "fe_stream_sum_cast", _ptr(h), _ptr(update), c_int(parts), _ptr(shift), _ptr(out), c_longlong(out_stride),
+          c_int(_code(out.dtype)), c_int(tokens), c_int(width), _stream())
     return out

@@ -1,5 +1,5 @@
 """A decoder built from a ``ModelPlan``: embedding, layers run in the order of
-the plan's schedule, final norm, head.  It knows no architecture: which parts,
+the plan's schedule (ahead of some calls the stream may be replaced), final norm, head.  It knows no architecture: which parts,
 which sizes and which order all come from the plan.
 """
 
@@ -27,6 +27,7 @@ class DecoderModel:
             norms = {role: build_part("norm", norm_spec, ctx) for role, norm_spec in spec.norms.items()}
             extra = dict(spec.block_params, prefix=spec.prefix) if (spec.block_params or spec.prefix) else {}
             self.layers.append(part_class("block", spec.block)(ctx, mixer, feed_forward, norms, **extra))
+        self.entry = None if plan.entry is None else build_part("entry", plan.entry, ctx)
         self.final_norm = build_part("norm", plan.final_norm, ctx)
         self.head = build_part("head", plan.head, ctx)
         if getattr(self.head, "tied", False):
@@ -46,6 +47,8 @@ class DecoderModel:
         found: list[Part] = [self.embedding]
         for layer in self.layers:
             found.extend(layer.children())
+        if self.entry is not None:
+            found.append(self.entry)
         found.extend([self.final_norm, self.head])
         return found
 
@@ -70,6 +73,8 @@ class DecoderModel:
             raise ValueError(f"tensors never loaded: {missing[:5]}")
         for part in self.parts():
             part.finalize()
+        for layer in self.layers:
+            layer.assemble()
 
     @property
     def graph_safe(self) -> bool:
@@ -104,8 +109,13 @@ class DecoderModel:
         """Run the step's tokens through every scheduled layer; float32 logits
         [len(batch.want_rows), vocab] at the wanted rows.  ``embedding_view``: the states of an
         embedding that keeps some."""
+        batch.carry.clear()      # a batch that is run again (ahead of a capture, say) carries nothing over
         residual = self.embedding.forward(batch) if embedding_view is None else self.embedding.forward(batch, embedding_view)
+        if self.entry is not None:
+            self.entry.begin(residual, batch)
         for index, call in enumerate(self.schedule):
+            if call.enters:
+                self.entry.forward(residual, batch)
             self.layers[call.layer].forward(residual, batch, cache_views[index], call.writes_cache)
         if batch.num_wanted == 0:
             residual.flush()

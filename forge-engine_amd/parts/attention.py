@@ -34,6 +34,9 @@ B / 2, else ``min(B - 1, B / 2 + floor(ln(n / (B / 2)) / ln(D / (B / 2)) * (B - 
 at first, logarithmic steps beyond, the last row from distance D on; the rows are laid out by distance
 once, when the table is loaded); ``qk_norm_eps`` on the general path (the weighted RMS norm of every q
 and k head, before the rotation, in the kernel that writes the pages);
+``query_temperature`` (``{"coef": c, "every": n}``: queries at position p times
+``1 + c ln(floor((p + 1) / n) + 1)``); ``output_scale`` (a factor on the layer's output, its bias included; it comes
+with an output gate, whose kernel applies it in float32);
 ``force_general`` (take the general path whatever the options).  A position part may scale its
 cosines and sines (``magnitude``).  With any of them the step takes the general path:
 one product for q, k, v (and the gate), one kernel for convolution, rotation, norms and the
@@ -48,7 +51,7 @@ from torch import Tensor
 from ..cache.spec import CacheNeeds, CacheView, FixedState, PagedKV
 from ..kernels import ops
 from ..registry import register_part
-from .base import BuildContext, Mixer, ParamSpec, build_part
+from .base import BuildContext, JointEnds, Mixer, ParamSpec, build_part
 from .plan import PartSpec
 
 
@@ -62,8 +65,10 @@ class GroupedQueryAttention(Mixer):
                  own_kv: bool = True, names: dict[str, str] | None = None, output_bias: bool | None = None,
                  fixed_sink: float | None = None, distance_slope_bits: float | None = None,
                  value_mix: str | None = None, value_mix_key: str = "values", force_general: bool = False,
-                 bias_init: str = "zeros", distance_bias: dict | None = None) -> None:
+                 bias_init: str = "zeros", distance_bias: dict | None = None, query_temperature: dict | None = None,
+                 output_scale: float = 1.0, output_bias_init: str = "zeros") -> None:
         super().__init__(ctx, prefix)
+        self.output_bias_init = output_bias_init
         self.bias_init = bias_init      # how random models draw the biases of q, k and v ("small": so that they show)
         if num_heads % num_kv_heads:
             raise ValueError("query heads must be a multiple of kv heads")
@@ -104,6 +109,12 @@ class GroupedQueryAttention(Mixer):
             if rows < 2 or not reach > rows // 2:
                 raise ValueError(f"a table of biases by distance needs two rows or more and a reach beyond half its rows, not {rows} and {reach}")
             self.distance_bias = (rows, reach)
+        self.query_temperature = None if query_temperature is None else (float(query_temperature["coef"]), float(query_temperature["every"]))
+        self.output_scale = float(output_scale)
+        if self.output_scale != 1.0 and not self.output_gate:
+            raise ValueError("a factor on the output comes with an output gate")
+        if self.query_temperature is not None and (whole_norm_eps is not None or not self.query_temperature[1] > 0.0):
+            raise ValueError("a query temperature needs a positive run of positions and is not combined with the whole-projection norm")
         self.bias_table: Tensor | None = None       # as loaded [rows, heads]; by distance [heads, span] after finalize
         self.mix_weight: float | None = None
         self.slopes: Tensor | None = None
@@ -120,7 +131,8 @@ class GroupedQueryAttention(Mixer):
                             or chunk is not None or sink or self.output_gate or whole_norm_eps is not None
                             or softcap is not None or not own_kv or fixed_sink is not None
                             or distance_slope_bits is not None or value_mix is not None
-                            or self.output_bias != bool(bias) or force_general or distance_bias is not None)
+                            or self.output_bias != bool(bias) or force_general or distance_bias is not None
+                            or query_temperature is not None)
         if (value_mix is not None or fixed_sink is not None or distance_slope_bits is not None) and whole_norm_eps is not None:
             raise ValueError("value mixing, fixed sinks and distance slopes are not combined with the whole-projection norm")
         if self.general and qk_norm_eps is not None and (whole_norm_eps is not None or unit_norm_eps is not None):
@@ -180,7 +192,7 @@ class GroupedQueryAttention(Mixer):
             specs[n["k_bias"]] = ParamSpec((self.kv_size,), kind="vector", init=drawn)
             specs[n["v_bias"]] = ParamSpec((self.v_size,), kind="vector", init=drawn)
             if self.output_bias:
-                specs[n["o_bias"]] = ParamSpec((self.hidden_size,), kind="vector", init="zeros")
+                specs[n["o_bias"]] = ParamSpec((self.hidden_size,), kind="vector", init=self.output_bias_init)
         if self.qk_norm_eps is not None:
             specs[n["q_norm"]] = ParamSpec((self.head_dim,), kind="vector", init="norm")
             specs[n["k_norm"]] = ParamSpec((self.head_dim,), kind="vector", init="norm")
@@ -248,7 +260,7 @@ class GroupedQueryAttention(Mixer):
             self.bias_table = self._bias_by_distance(self.bias_table).to(device)
         # the general path adds biases in float32 behind the products, which then take the kernels for few rows
         self.conv_bias = None if self.qkv_bias is None else self.qkv_bias[:self.conv_channels].float().contiguous()
-        self.o_bias_f32 = None if self.o_bias is None else self.o_bias.float().contiguous()
+        self.o_bias_f32 = None if self.o_bias is None else (self.o_bias.float() * self.output_scale).contiguous()
         if self.qkv_bias is not None and self.qkv_weight.dtype != torch.float32:
             self.qkv_bias = self.qkv_bias.to(self.qkv_weight.dtype)
         if self.o_bias is not None and self.o_weight.dtype != torch.float32:
@@ -335,7 +347,27 @@ class GroupedQueryAttention(Mixer):
             raise ValueError("the general attention path writes its own keys and values, except for a layer that "
                              "has none and reads another call's")
         qkv = ops.linear(x, self.qkv_weight)        # [T, q | k | v (| gate)]; the bias is added by the kernel below
-        q = torch.empty((x.shape[0], self.q_size), dtype=x.dtype, device=x.device)
+        attn = torch.empty((x.shape[0], self.out_size), dtype=x.dtype, device=x.device)
+        self._attend(qkv, attn, batch, cache, writes_cache, inv_freq, rotary_dim)
+        update = ops.linear_update(attn, self.o_weight)
+        return update if self.o_bias_f32 is None else ops.add_bias(update, self.o_bias_f32)
+
+    def joint_ends(self) -> JointEnds | None:
+        if not (self.general and self.own_kv and self.output_gate):
+            return None
+        return JointEnds(self.qkv_weight, self.o_weight, self.o_bias_f32)
+
+    def release_ends(self) -> None:
+        self.qkv_weight = self.o_weight = None
+
+    def forward_joint(self, z: Tensor, out: Tensor, batch, cache: CacheView, writes_cache: bool = True) -> None:
+        rotary = self.position.rotary()
+        inv_freq, rotary_dim = rotary if rotary is not None else (None, 0)
+        self._attend(z, out, batch, cache, writes_cache, inv_freq, rotary_dim)
+
+    def _attend(self, qkv: Tensor, attn: Tensor, batch, cache: CacheView, writes_cache: bool, inv_freq, rotary_dim: int) -> None:
+        """From the projections to the gated heads, side by side."""
+        q = torch.empty((qkv.shape[0], self.q_size), dtype=qkv.dtype, device=qkv.device)
         magnitude = self.position.magnitude()
         if self.whole_norm_eps is not None:
             ops.whole_norm_rope_write(
@@ -347,16 +379,13 @@ class GroupedQueryAttention(Mixer):
             raise ValueError("scaled cosines and sines come with the whole-projection norm's kernel only")
         else:
             self._conv_rope(qkv, q, batch, cache, inv_freq, rotary_dim)
-        attn = torch.empty((x.shape[0], self.out_size), dtype=x.dtype, device=x.device)
         ops.masked_attention(
             q, cache.key_pages, cache.value_pages, attn, batch.cu_q, batch.ctx_len, cache.block_table,
             num_seqs=batch.num_seqs, max_q_len=batch.max_q_len, q_heads=self.num_heads,
             kv_heads=self.num_kv_heads, head_dim=self.head_dim, value_dim=self.value_dim, scale=self.scale,
             window=self.window, chunk=self.chunk, sink=self.sink_weight, slopes=self.slopes, dist_bias=self.bias_table,
             gate=qkv[:, self.conv_channels:] if self.output_gate else None, num_decode=batch.num_decode,
-            max_ctx=batch.max_ctx, softcap=self.softcap, head_gate=self.head_gate)
-        update = ops.linear_update(attn, self.o_weight)
-        return update if self.o_bias_f32 is None else ops.add_bias(update, self.o_bias_f32)
+            max_ctx=batch.max_ctx, softcap=self.softcap, head_gate=self.head_gate, factor=self.output_scale)
 
     def _conv_rope(self, qkv: Tensor, q: Tensor, batch, cache: CacheView, inv_freq, rotary_dim: int) -> None:
         mixing = {}
@@ -376,7 +405,7 @@ class GroupedQueryAttention(Mixer):
             rotary_dim=rotary_dim, unit_norm_eps=self.unit_norm_eps if self.qk_norm_eps is None else self.qk_norm_eps,
             taps=self.conv_taps, norm_weight_q=self.q_norm if self.qk_norm_eps is not None else None,
             norm_weight_k=self.k_norm if self.qk_norm_eps is not None else None,
-            norm_first=self.qk_norm_eps is not None, **mixing)
+            norm_first=self.qk_norm_eps is not None, q_temp=self.query_temperature, **mixing)
 
     def _single_tokens_only(self, batch, x: Tensor, cache: CacheView, rotary_dim: int) -> bool:
         """Every sequence of the step brings one token, and the sizes are ones that the

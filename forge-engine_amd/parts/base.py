@@ -10,6 +10,7 @@ which model it is in.  Roles:
 * ``FeedForward``:  activations [T, H] -> update [T, H]
 * ``PositionEncoding``: what a mixer needs to encode positions
 * ``Block``:        the arrangement of the above in one layer
+* ``StreamEntry``:  what happens to the stream ahead of a pass through a run of layers
 * ``Head``:         normalised rows -> float32 logits
 """
 
@@ -34,13 +35,15 @@ class ParamSpec:
     ``init``: how the random-weights mode draws it: ``normal`` N(0, 0.02),
     ``norm`` 1 + N(0, 0.05), ``zeros``, ``unit`` N(0, 0.25), ``uniform`` U(0, 1), ``taps`` (a short
     convolution: N(0, 0.04) with one added to the newest tap), ``small`` N(0, 0.01), ``router``
-    N(0, 0.25), ``identity`` (the identity plus N(0, 0.01)).
+    N(0, 0.25), ``identity`` (the identity plus N(0, 0.01)); an ``int_table`` with ``choices`` gets rows of
+    different numbers below that.
     """
 
     shape: tuple[int, ...]
     kind: str = "matrix"
     init: str = "normal"
     optional: bool = False
+    choices: int = 0
 
 
 @dataclass
@@ -65,14 +68,28 @@ class Residual:
         self.pending: Tensor | None = None
         self.streams: Tensor | None = None
         self.pending_mix: tuple[Tensor, Tensor] | None = None    # (mix [S, S] indexed [from, to], share [S])
+        self.pending_bias: Tensor | None = None                   # float32 [W]: added with the pending update, or alone
         self.pending_norm: tuple[Tensor, float] | None = None    # (weight, eps): the update is RMS-normed before it is added
         self.in_compute_dtype: Tensor | None = None               # the stream as a norm of updates last stored it beside h (the same values)
 
-    def add(self, update: Tensor | None) -> None:
-        """Leave an update pending; None: the part has added it into the stream itself."""
+    def add(self, update: Tensor | None, bias: Tensor | None = None) -> None:
+        """Leave an update pending; None: the part has added it into the stream itself.  ``bias``: one number a
+        channel that comes on top."""
         self.flush()
         self.in_compute_dtype = None
-        self.pending = update
+        self.pending, self.pending_bias = update, bias
+
+    def take_biased(self) -> tuple[Tensor | None, Tensor | None]:
+        """(update, bias) of what is pending, which the caller now applies itself."""
+        update, bias = self.pending, self.pending_bias
+        self.pending = self.pending_bias = None
+        return update, bias
+
+    def replace(self, h: Tensor, update: Tensor | None = None) -> None:
+        """The stream is another tensor from here on (nothing of the old one, or pending on it, counts any more)."""
+        self.h = h
+        self.in_compute_dtype = None
+        self.pending, self.pending_bias = update, None
 
     def add_normed(self, update: Tensor, weight: Tensor, eps: float) -> None:
         """Leave ``h += update * rsqrt(mean(update^2) + eps) * weight`` pending (a norm behind a
@@ -124,7 +141,12 @@ class Residual:
         return out
 
     def flush(self) -> Tensor:
-        if self.pending is not None:
+        if self.pending_bias is not None:
+            if self.streams is not None:
+                raise ValueError("a bias on an update needs a model with one residual stream")
+            update, bias = self.take_biased()
+            ops.hyper_norm(self.h.unsqueeze(0), update, None, None, None, None, None, 0.0, None, shift=bias)
+        elif self.pending is not None:
             if self.streams is not None:
                 update, mix, share = self.take_pending()
                 ops.hyper_norm(self.streams, update, mix, share, None, None, None, 0.0, None)
@@ -211,6 +233,22 @@ class PositionEncoding(Part):
         """A factor on every cosine and sine of the rotation (1: a plain rotation)."""
         return 1.0
 
+    def table(self, batch) -> Tensor | None:
+        """(cos, sin) of the step's tokens, float32 [T, rotary_dim / 2, 2], for mixers that turn q and k inside a
+        kernel that is not theirs alone; None where nothing turns."""
+        return None
+
+
+@dataclass
+class JointEnds:
+    """The first and the last matrix of a part that is an inner function between two products.  Parts that read
+    the same input and whose outputs are added up can share both products: the first matrices stacked, the last
+    ones side by side (the sum of the products is one product over the concatenated inner activations)."""
+
+    first: Tensor                # [N, W]: everything that reads the part's input
+    last: Tensor                 # [W, K]: what its inner activations go through
+    bias: Tensor | None = None   # float32 [W] on the last product
+
 
 class Mixer(Part):
     role = "mixer"
@@ -218,6 +256,18 @@ class Mixer(Part):
     # it may add its update into the stream itself, where its last product can do so for free, and
     # then returns None instead of the update.
     takes_stream = False
+
+    def joint_ends(self) -> JointEnds | None:
+        """The part's outer matrices, if it can run between products that it shares with others (``forward_joint``)."""
+        return None
+
+    def release_ends(self) -> None:
+        """The outer matrices live in shared ones now: the part's own copies go, and ``forward`` is not called any more."""
+
+    def forward_joint(self, z: Tensor, out: Tensor, batch, cache: CacheView | None, writes_cache: bool = True) -> None:
+        """From ``z`` [T, N], its columns of the shared first product, to its inner activations ``out`` [T, K] (both
+        strided views)."""
+        raise NotImplementedError
 
     def cache_needs(self) -> CacheNeeds:
         return CacheNeeds()
@@ -229,6 +279,16 @@ class Mixer(Part):
 class FeedForward(Part):
     role = "feed_forward"
     takes_stream = False   # as for a mixer
+    takes_extra = False    # True: ``forward`` takes ``extra=``, an update of the same tokens that joins its own
+
+    def joint_ends(self) -> JointEnds | None:
+        return None        # as for a mixer
+
+    def release_ends(self) -> None:
+        """As for a mixer."""
+
+    def forward_joint(self, z: Tensor, out: Tensor, batch) -> None:
+        raise NotImplementedError
 
     def forward(self, x: Tensor, batch) -> Tensor | None:
         raise NotImplementedError
@@ -238,6 +298,17 @@ class Head(Part):
     role = "head"
 
     def forward(self, z: Tensor) -> Tensor:
+        raise NotImplementedError
+
+
+class StreamEntry(Part):
+    role = "entry"
+
+    def begin(self, residual: Residual, batch) -> None:
+        """Once a step, right behind the embedding: keep what the passes need of it (in ``batch.carry``)."""
+
+    def forward(self, residual: Residual, batch) -> None:
+        """Ahead of the first layer of a pass: replace the stream."""
         raise NotImplementedError
 
 
@@ -259,6 +330,9 @@ class Block(Part):
         if self.feed_forward is not None:
             found.append(self.feed_forward)
         return [*found, *self.norms.values()]
+
+    def assemble(self) -> None:
+        """Called once after every part of the model was finalized: an arrangement may join its parts' matrices."""
 
     def cache_needs(self) -> CacheNeeds:
         """What one call of the layer asks of the cache: the mixer's needs, and whatever

@@ -117,6 +117,76 @@ class SandwichNormBlock(Block):
         return {"stream_ops"}
 
 
+class ParallelBlock(Block):
+    """One norm, and both sublayers read its output: ``x = norm(h); h += mixer(x) + ffn(x)``.  Sublayers
+    that offer their outer matrices (``joint_ends``) share two products: one from x to everything they read of it,
+    one from their inner activations, side by side, to the update.  A feed-forward that does not (experts) takes
+    the mixer's update along as its ``extra``.  A layer may have no feed-forward."""
+
+    NORMS = ("input",)
+
+    def __init__(self, ctx: BuildContext, mixer, feed_forward, norms, prefix: str = "") -> None:
+        super().__init__(ctx, mixer, feed_forward, norms, prefix)
+        self.first: Tensor | None = None       # the shared matrices, once assembled
+        self.last: Tensor | None = None
+        self.bias: Tensor | None = None
+        self.mixer_ends = (0, 0)               # columns of the first product, and of the inner activations, that are the mixer's
+        self.joint_feed_forward = False
+
+    def assemble(self) -> None:
+        ends = self.mixer.joint_ends()
+        if ends is None:
+            return
+        joint = [ends]
+        other = None if self.feed_forward is None else self.feed_forward.joint_ends()
+        if other is not None and other.first.dtype == ends.first.dtype and other.last.dtype == ends.last.dtype:
+            joint.append(other)
+            self.joint_feed_forward = True
+        self.mixer_ends = (ends.first.shape[0], ends.last.shape[1])
+        self.first = ends.first if len(joint) == 1 else torch.cat([e.first for e in joint])
+        self.last = ends.last if len(joint) == 1 else torch.cat([e.last for e in joint], dim=1)
+        biases = [e.bias for e in joint if e.bias is not None]
+        self.bias = None if not biases else sum(biases[1:], biases[0])
+        self.mixer.release_ends()
+        if self.joint_feed_forward:
+            self.feed_forward.release_ends()
+
+    def forward(self, residual: Residual, batch, cache: CacheView | None, writes_cache: bool = True) -> None:
+        x = self.norms["input"].forward(residual)
+        if self.first is None:
+            self._forward_apart(x, residual, batch, cache, writes_cache)
+            return
+        z = ops.linear(x, self.first)
+        inner = torch.empty((x.shape[0], self.last.shape[1]), dtype=x.dtype, device=x.device)
+        columns, width = self.mixer_ends
+        self.mixer.forward_joint(z[:, :columns], inner[:, :width], batch, cache, writes_cache)
+        if self.joint_feed_forward:
+            self.feed_forward.forward_joint(z[:, columns:], inner[:, width:], batch)
+        update = ops.linear_update(inner, self.last, stream=residual.open())
+        if self.feed_forward is not None and not self.joint_feed_forward:
+            update = self._with_feed_forward(x, update, batch)
+        residual.add(update, self.bias)
+
+    def _with_feed_forward(self, x: Tensor, update: Tensor | None, batch) -> Tensor:
+        if self.feed_forward.takes_extra:
+            return self.feed_forward.forward(x, batch, extra=update)
+        return _side_by_side(update, self.feed_forward.forward(x, batch))
+
+    def _forward_apart(self, x: Tensor, residual: Residual, batch, cache, writes_cache: bool) -> None:
+        update = self.mixer.forward(x, batch, cache, writes_cache)
+        residual.add(update if self.feed_forward is None else self._with_feed_forward(x, update, batch))
+
+    def kernel_libraries(self):
+        return {"gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide", "rowwise"}
+
+
+def _side_by_side(a: Tensor | None, b: Tensor | None) -> Tensor | None:
+    """Two updates as one in parts."""
+    if a is None or b is None:
+        return a if b is None else b
+    return torch.cat([u if u.dim() == 3 else u.unsqueeze(0) for u in (a, b)])
+
+
 class HyperConnectionBlock(Block):
     """Pre-norm sublayers over ``streams`` residual streams instead of one.  Sublayer q (the mixer,
     then the feed-forward) reads ``u = sum_s in_q[s] x_s``, computes ``y = sublayer(norm_q(u))``, and
@@ -177,6 +247,7 @@ class HyperConnectionBlock(Block):
 
 
 register_part("block", "hyper_connections", HyperConnectionBlock)
+register_part("block", "parallel", ParallelBlock)
 register_part("block", "pre_norm", PreNormBlock)
 register_part("block", "sandwich_norm", SandwichNormBlock)
 register_part("block", "output_norm", OutputNormBlock)

@@ -9,36 +9,40 @@ from torch import Tensor
 
 from ..kernels import ops
 from ..registry import register_part
-from .base import BuildContext, FeedForward, ParamSpec
+from .base import BuildContext, FeedForward, JointEnds, ParamSpec
 
 
 class SwiGLU(FeedForward):
-    def __init__(self, ctx: BuildContext, prefix: str, *, hidden_size: int, intermediate_size: int) -> None:
+    DEFAULT_NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
+
+    def __init__(self, ctx: BuildContext, prefix: str, *, hidden_size: int, intermediate_size: int,
+                 names: dict[str, str] | None = None) -> None:
         super().__init__(ctx, prefix)
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
+        self.names = dict(self.DEFAULT_NAMES, **(names or {}))
         self.gate_up_weight: Tensor | None = None
         self.down_weight: Tensor | None = None
 
     def param_specs(self):
         inter, hidden = self.intermediate_size, self.hidden_size
         return {
-            self.name("gate_proj.weight"): ParamSpec((inter, hidden)),
-            self.name("up_proj.weight"): ParamSpec((inter, hidden)),
-            self.name("down_proj.weight"): ParamSpec((hidden, inter)),
+            self.name(self.names["gate"]): ParamSpec((inter, hidden)),
+            self.name(self.names["up"]): ParamSpec((inter, hidden)),
+            self.name(self.names["down"]): ParamSpec((hidden, inter)),
         }
 
     def set_param(self, name: str, tensor: Tensor) -> None:
         inter = self.intermediate_size
-        if name in (self.name("gate_proj.weight"), self.name("up_proj.weight")):
+        if name in (self.name(self.names["gate"]), self.name(self.names["up"])):
             if self.gate_up_weight is None:
                 self.gate_up_weight = torch.empty((2 * inter, self.hidden_size), dtype=tensor.dtype,
                                                   device=tensor.device)
             if tensor.dtype != self.gate_up_weight.dtype:
                 raise ValueError(f"{name}: gate and up projections must be stored in one dtype")
-            start = 0 if name == self.name("gate_proj.weight") else inter
+            start = 0 if name == self.name(self.names["gate"]) else inter
             self.gate_up_weight[start:start + inter].copy_(tensor)
-        elif name == self.name("down_proj.weight"):
+        elif name == self.name(self.names["down"]):
             self.down_weight = tensor
         else:
             raise KeyError(name)
@@ -48,6 +52,15 @@ class SwiGLU(FeedForward):
     def forward(self, x: Tensor, batch=None, stream: Tensor | None = None) -> Tensor | None:
         act = ops.linear_swiglu(x, self.gate_up_weight)
         return ops.linear_update(act, self.down_weight, stream=stream)   # the update stays float32 for the residual sum
+
+    def joint_ends(self) -> JointEnds:
+        return JointEnds(self.gate_up_weight, self.down_weight)
+
+    def release_ends(self) -> None:
+        self.gate_up_weight = self.down_weight = None
+
+    def forward_joint(self, z: Tensor, out: Tensor, batch=None) -> None:
+        ops.swiglu(z, out)
 
     def kernel_libraries(self):
         return {"rowwise", "gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide", "gemm_tile"}

@@ -17,7 +17,9 @@ expert, within the ``keep_groups`` best of ``groups`` equal runs of neighbouring
 being as good as its best corrected score; a chosen expert's weight is its own score over the
 sum of the chosen scores, times ``route_scale``); ``shared_gate`` (the shared expert's output times
 ``sigmoid(w_g . x)``, one number a token, w_g a tensor of one row; its logit is formed with the
-router's, in float32).
+router's, in float32); ``scoring`` "table" (no router at all: row ``token id`` of an integer table
+[vocab, top] names the token's experts, each weighing 1 / top; the plan of such a step is made once for all
+passes through the layer); ``form`` "relu_squared" (no gate: ``y = W_down max(W_up x, 0)^2``).
 
 A step sorts its (token, choice) pairs by expert on the device and runs two grouped products over
 the sorted rows (gate and up with the activation as their ending, then down, weighted by the
@@ -41,7 +43,7 @@ class RoutedExperts(FeedForward):
                  intermediate_size: int, limit: float | None = None, alpha: float = 1.702, shared_size: int | None = None,
                  shared_limit: float | None = None, names: dict[str, str] | None = None, scoring: str = "softmax",
                  form: str = "bounded", weight_input: bool = False, router_bias: bool = True, groups: int = 1,
-                 keep_groups: int = 1, route_scale: float = 1.0, shared_gate: bool = False) -> None:
+                 keep_groups: int = 1, route_scale: float = 1.0, shared_gate: bool = False, vocab_size: int | None = None) -> None:
         """``names``: what the tensors are called behind the prefix; ``expert`` is a pattern with
         ``{e}`` for the expert's number."""
         super().__init__(ctx, prefix)
@@ -52,7 +54,7 @@ class RoutedExperts(FeedForward):
         self.hidden_size = hidden_size
         self.experts, self.top = experts, top
         self.intermediate_size = intermediate_size
-        if scoring not in ("softmax", "sigmoid", "softmax_all") or form not in ("bounded", "silu"):
+        if scoring not in ("softmax", "sigmoid", "softmax_all", "table") or form not in ("bounded", "silu", "relu_squared"):
             raise ValueError(f"unknown scoring '{scoring}' or form '{form}'")
         if scoring == "softmax_all":
             if not 1 <= groups <= 64 or experts % groups or not 1 <= keep_groups <= groups or top > experts // groups * keep_groups:
@@ -61,6 +63,13 @@ class RoutedExperts(FeedForward):
                 raise ValueError("scores over all experts come without a router bias and weigh the experts' outputs")
         elif groups != 1 or keep_groups != 1 or route_scale != 1.0:
             raise ValueError("groups and a factor on the weights come with scoring 'softmax_all'")
+        if scoring == "table" and (router_bias or weight_input or shared_gate or not vocab_size):
+            raise ValueError("a table of experts needs the vocabulary's size and comes without a router's options")
+        if form == "relu_squared" and shared_size:
+            raise ValueError("experts without a gate are not combined with a shared expert")
+        self.vocab_size = vocab_size
+        self.table: Tensor | None = None
+        self.matrices = 1 if form == "relu_squared" else 2      # first matrices of an expert
         if shared_gate and not shared_size:
             raise ValueError("a gate on the shared expert needs a shared expert")
         self.groups, self.keep_groups, self.route_scale, self.shared_gate = int(groups), int(keep_groups), float(route_scale), bool(shared_gate)
@@ -71,7 +80,8 @@ class RoutedExperts(FeedForward):
         self.shared_size = shared_size
         self.shared_limit = float(self.limit if shared_limit is None else shared_limit)
         self.names = dict({"expert": "experts.{e}", "shared": "shared", "router": "router.weight", "router_bias": "router.bias",
-                           "gate": "gate", "up": "up", "down": "down", "correction": "correction", "shared_gate": "shared.gate_proj"},
+                           "gate": "gate", "up": "up", "down": "down", "correction": "correction", "shared_gate": "shared.gate_proj",
+                           "table": "table"},
                           **(names or {}))
         self.correction: Tensor | None = None
         self.router_rows: Tensor | None = None      # with a gate on the shared expert: the router's rows, then the gate's row
@@ -82,13 +92,18 @@ class RoutedExperts(FeedForward):
         self.shared_gate_up: Tensor | None = None   # [2 Fs, H]
         self.shared_down: Tensor | None = None
 
+    takes_extra = True
+
     def _expert_name(self, expert: int | None, which: str) -> str:
         owner = self.names["shared"] if expert is None else self.names["expert"].format(e=expert)
         return self.name(f"{owner}.{self.names[which]}")
 
     def param_specs(self):
         f, h = self.intermediate_size, self.hidden_size
-        specs = {self.name(self.names["router"]): ParamSpec((self.experts, h), init="router")}
+        if self.scoring == "table":
+            specs = {self.name(self.names["table"]): ParamSpec((self.vocab_size, self.top), kind="int_table", choices=self.experts)}
+        else:
+            specs = {self.name(self.names["router"]): ParamSpec((self.experts, h), init="router")}
         if self.scoring == "softmax_all":     # a checkpoint without it: no correction
             specs[self.name(self.names["correction"])] = ParamSpec((self.experts,), kind="vector", init="small", optional=True)
         if self.shared_gate:
@@ -96,7 +111,8 @@ class RoutedExperts(FeedForward):
         if self.has_router_bias:
             specs[self.name(self.names["router_bias"])] = ParamSpec((self.experts,), kind="vector", init="small")
         for expert in range(self.experts):
-            specs[self._expert_name(expert, "gate")] = ParamSpec((f, h))
+            if self.matrices == 2:
+                specs[self._expert_name(expert, "gate")] = ParamSpec((f, h))
             specs[self._expert_name(expert, "up")] = ParamSpec((f, h))
             specs[self._expert_name(expert, "down")] = ParamSpec((h, f))
         if self.shared_size:
@@ -105,13 +121,16 @@ class RoutedExperts(FeedForward):
             specs[self._expert_name(None, "down")] = ParamSpec((h, self.shared_size))
         self._owners = {}
         for expert in [*range(self.experts), None] if self.shared_size else range(self.experts):
-            for which in ("gate", "up", "down"):
+            for which in ("gate", "up", "down")[2 - self.matrices:]:
                 self._owners[self._expert_name(expert, which)] = (expert, which)
         return specs
 
     def set_param(self, name: str, tensor: Tensor) -> None:
         f, h = self.intermediate_size, self.hidden_size
-        if name == self.name(self.names["router"]) or (self.shared_gate and name == self.name(self.names["shared_gate"])):
+        if self.scoring == "table" and name == self.name(self.names["table"]):
+            self.table = tensor.contiguous()
+            return
+        if (self.scoring != "table" and name == self.name(self.names["router"])) or (self.shared_gate and name == self.name(self.names["shared_gate"])):
             if not self.shared_gate:
                 self.router_weight = tensor.contiguous()
                 return
@@ -151,18 +170,32 @@ class RoutedExperts(FeedForward):
             self.down[expert].copy_(tensor)
             return
         if self.gate_up is None:
-            self.gate_up = torch.empty((self.experts, 2 * f, h), dtype=tensor.dtype, device=tensor.device)
-        start = 0 if which == "gate" else f
+            self.gate_up = torch.empty((self.experts, self.matrices * f, h), dtype=tensor.dtype, device=tensor.device)
+        start = 0 if which == "gate" or self.matrices == 1 else f
         self.gate_up[expert, start:start + f].copy_(tensor)
 
     def finalize(self) -> None:
-        if self.gate_up.dtype != self.down.dtype or self.gate_up.dtype != self.router_weight.dtype:
+        if self.scoring == "table":
+            rows = self.table.sort(dim=1).values
+            if int(rows.min()) < 0 or int(rows.max()) >= self.experts or bool((rows[:, 1:] == rows[:, :-1]).any()):
+                raise ValueError(f"{self.prefix}: every row of the table must name different experts below {self.experts}")
+        if self.gate_up.dtype != self.down.dtype or (self.router_weight is not None and self.gate_up.dtype != self.router_weight.dtype):
             raise ValueError(f"{self.prefix}: the experts' matrices and the router must be stored in one dtype")
 
-    def forward(self, x: Tensor, batch=None) -> Tensor:
+    def _table_plan(self, batch) -> tuple[Tensor, Tensor, Tensor]:
+        key = ("expert plan", self.prefix)
+        if key not in batch.carry:      # token ids stay the same through a step: so does who goes where
+            batch.carry[key] = ops.moe_plan_table(batch.token_ids, self.table, self.experts)
+        return batch.carry[key]
+
+    def forward(self, x: Tensor, batch=None, extra: Tensor | None = None) -> Tensor:
+        """``extra`` (float32 [T, H] or in parts): an update of the same tokens that joins the first choice's part."""
         tokens = x.shape[0]
         gate_logits, gate_column = None, 0
-        if self.scoring == "softmax_all":
+        chosen = plan = None
+        if self.scoring == "table":
+            *plan, weights = self._table_plan(batch)
+        elif self.scoring == "softmax_all":
             chosen, weights, logits = ops.moe_route_grouped(
                 x, self.router_rows if self.shared_gate else self.router_weight, self.correction, experts=self.experts,
                 top=self.top, groups=self.groups, keep=self.keep_groups, scale=self.route_scale)
@@ -180,9 +213,13 @@ class RoutedExperts(FeedForward):
             shared = ops.linear_update(act, self.shared_down)
             if self.shared_gate:
                 ops.gate_rows(shared, gate_logits, gate_column)
+        if shared is not None and extra is not None:
+            extra = torch.cat([u if u.dim() == 3 else u.unsqueeze(0) for u in (shared, extra)])
+        elif extra is None:
+            extra = shared
         update = torch.empty((self.top, tokens, self.hidden_size), dtype=torch.float32, device=x.device)
         return ops.moe_experts(x, chosen, weights, self.gate_up, self.down, update, limit=self.limit, alpha=self.alpha,
-                               extra=shared, form=self.form, weight_input=self.weight_input)
+                               extra=extra, form=self.form, weight_input=self.weight_input, plan=plan)
 
     def kernel_libraries(self):
         return {"moe", "rowwise", "stream_ops", "gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide", "gemm_tile"}

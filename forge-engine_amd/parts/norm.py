@@ -38,6 +38,8 @@ class RMSNorm(Norm):
         self.weight = tensor + self.offset if self.offset else tensor
 
     def forward(self, residual: Residual, rows: Tensor | None = None) -> Tensor:
+        if residual.pending_bias is not None:    # this kernel knows no bias on the update
+            residual.flush()
         if residual.pending_norm is not None:    # a norm behind the sublayer before: both norms in one pass over the row
             if rows is not None:                 # the chosen rows alone; stream and pending update are left as they are
                 update, (weight, eps) = residual.pending, residual.pending_norm
@@ -82,7 +84,7 @@ class LayerNorm(Norm):
     squared deviations; float32 inside, fused with the add of the pending update like the other
     norms.  It also serves models with several residual streams (``reads_streams``): its input is
     then ``sum_s read[s] x_s`` (``read`` None: the plain sum), taken after the pending update went
-    into the streams through its mixing matrix, all in the same kernel."""
+    into the streams through its mixing matrix, all in the same kernel (which also adds a bias on the update)."""
 
     reads_streams = True
 
@@ -117,9 +119,11 @@ class LayerNorm(Norm):
         out = torch.empty((count, self.size), dtype=self.ctx.dtype, device=streams.device)
         if rows is not None:     # the chosen rows alone; stream and pending update are left as they are
             update, mixed = residual.pending, residual.pending_mix or (None, None)
-            return ops.hyper_norm(streams, update, *mixed, read, self.weight, self.bias, self.eps, out, rows=rows, store=False)
+            return ops.hyper_norm(streams, update, *mixed, read, self.weight, self.bias, self.eps, out, rows=rows, store=False,
+                                  shift=residual.pending_bias)
+        shift, residual.pending_bias = residual.pending_bias, None
         update, mix, share = residual.take_pending()
-        return ops.hyper_norm(streams, update, mix, share, read, self.weight, self.bias, self.eps, out)
+        return ops.hyper_norm(streams, update, mix, share, read, self.weight, self.bias, self.eps, out, shift=shift)
 
     def kernel_libraries(self):
         return {"hyper"}

@@ -37,11 +37,13 @@ class LayerCall:
     """One entry of the run order.  ``layer`` indexes ``ModelPlan.layers`` (a
     layer may be named more than once).  ``cache`` names the cache slot the
     call uses: by default its own, else that of an earlier call, in which case
-    ``writes_cache`` is False and the mixer only reads what the other wrote."""
+    ``writes_cache`` is False and the mixer only reads what the other wrote.  A layer that is named several times
+    has a cache slot and state of its own for every call."""
 
     layer: int
     cache: int | None = None
     writes_cache: bool = True
+    enters: bool = False    # the stream passes the plan's ``entry`` right ahead of this call
 
 
 @dataclass(frozen=True)
@@ -55,6 +57,7 @@ class ModelPlan:
     head: PartSpec
     eos_token_ids: frozenset = frozenset()
     max_positions: int | None = None
+    entry: PartSpec | None = None              # what replaces the stream ahead of the calls that say ``enters``
     ignorable_names: frozenset = frozenset()   # tensors that a checkpoint may hold and the model does not read
 
     def resolved_schedule(self) -> tuple[LayerCall, ...]:
@@ -69,5 +72,7 @@ class ModelPlan:
                     raise ValueError(f"schedule entry {index} shares cache slot {slot} and must not write it")
                 if not (0 <= slot < index) or not calls[slot].writes_cache:
                     raise ValueError(f"schedule entry {index} reads cache slot {slot}, which no earlier entry writes")
-            calls.append(LayerCall(call.layer, slot, call.writes_cache))
+            if call.enters and self.entry is None:
+                raise ValueError(f"schedule entry {index} enters a pass, but the plan names no entry")
+            calls.append(LayerCall(call.layer, slot, call.writes_cache, call.enters))
         return tuple(calls)

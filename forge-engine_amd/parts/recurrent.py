@@ -1,12 +1,12 @@
 """Mixers that carry a matrix state per head from token to token instead of a cache of keys.
 
-All three are the linear recurrence
+All of them are the linear recurrence
 
     S_t = diag(a_t) S_(t-1) + b_t k_t v_t^T            (S: [key dim, value dim] per head, float32)
 
 read by a query, and differ in where the decay a_t and the input scale b_t come from, whether the
 query reads the state before or after the token's own update, and how the read-out is
-normalised.  One kernel runs the recurrence for all of them (``ops.linear_recurrence``), for
+normalised.  One kernel runs the recurrence for the first three (``ops.linear_recurrence``), for
 prompt portions and single tokens alike; the state of every live request lives in a fixed-size
 slot, so a request may be cut into steps anywhere.  Decays, gates, the state and the read-out
 are float32 in both compute modes; the projections run in the compute dtype.
@@ -24,9 +24,15 @@ are float32 in both compute modes; the projections run in the compute dtype.
   b_t = exp(i - m_t); a normaliser n_t follows the same recurrence with k alone (kept as one more
   column of the state, fed by v = 1); read-out ``S_t^T q / (max(|n_t . q|, exp(-m_t)) + 1e-6)``,
   heads normalised to unit root mean square, times a weight, times sigmoid(gate).
+* ``retention``: one constant decay per head; q and k turned by rotary positions, k times dim^-1/2;
+  the query reads S_t; heads normalised to unit root mean square (no weight), times silu(gate).  With one
+  decay a head a prompt is walked in chunks as matrix products (``ops.head_recurrence``), and a step of
+  single tokens ends with the norm and the gate in the recurrence's own launch.
 """
 
 from __future__ import annotations
+
+import math
 
 import torch
 from torch import Tensor
@@ -34,7 +40,8 @@ from torch import Tensor
 from ..cache.spec import CacheNeeds, CacheView, FixedState
 from ..kernels import ops
 from ..registry import register_part
-from .base import BuildContext, Mixer, ParamSpec
+from .base import BuildContext, JointEnds, Mixer, ParamSpec, build_part
+from .plan import PartSpec
 
 
 class _RecurrentMixer(Mixer):
@@ -247,6 +254,58 @@ class MLSTM(_RecurrentMixer):
         return ops.linear_update(y, t["o"])
 
 
+class Retention(_RecurrentMixer):
+    DEFAULT_NAMES = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o"}
+
+    def __init__(self, ctx: BuildContext, prefix: str, *, hidden_size: int, heads: int, dim: int, value_dim: int, eps: float,
+                 decay: list[float], position: PartSpec, names: dict[str, str] | None = None) -> None:
+        """``decay``: what a head's state is multiplied by from token to token, one positive number a head."""
+        super().__init__(ctx, prefix, hidden_size=hidden_size, heads=heads, key_dim=dim, value_dim=value_dim, eps=eps, names=names)
+        if len(decay) != heads or not all(d > 0.0 for d in decay):
+            raise ValueError(f"{heads} heads need as many positive decays, not {decay}")
+        if not 1 <= dim <= 256:
+            raise ValueError(f"key sizes of 1 to 256, not {dim}")
+        self.position = build_part("position", position, ctx)
+        self.rate = torch.tensor([math.log(d) for d in decay], dtype=torch.float64).to(torch.float32).to(ctx.device)
+        self.fuse("qkvg", [("q", heads * dim), ("k", heads * dim), ("v", heads * value_dim), ("g", heads * value_dim)])
+
+    def shapes(self):
+        keys, values, width = self.heads * self.key_dim, self.heads * self.value_dim, self.hidden_size
+        return {"q": ((keys, width), "matrix", "normal"), "k": ((keys, width), "matrix", "normal"),
+                "v": ((values, width), "matrix", "normal"), "g": ((values, width), "matrix", "normal"),
+                "o": ((width, values), "matrix", "normal")}
+
+    def forward(self, x: Tensor, batch, cache: CacheView, writes_cache: bool = True) -> Tensor:
+        out = torch.empty((x.shape[0], self.heads * self.value_dim), dtype=x.dtype, device=x.device)
+        self.forward_joint(ops.linear(x, self.tensors["qkvg"]), out, batch, cache, writes_cache)
+        return ops.linear_update(out, self.tensors["o"])
+
+    def joint_ends(self) -> JointEnds:
+        return JointEnds(self.tensors["qkvg"], self.tensors["o"])
+
+    def release_ends(self) -> None:
+        self.tensors = {}
+
+    def forward_joint(self, z: Tensor, out: Tensor, batch, cache: CacheView, writes_cache: bool = True) -> None:
+        q, k, v, gate = (self.columns(z, key) for key in ("q", "k", "v", "g"))
+        sizes = {"num_seqs": batch.num_seqs, "heads": self.heads, "key_dim": self.key_dim, "value_dim": self.value_dim,
+                 "rate": self.rate, "table": self.position.table(batch), "k_scale": self.key_dim ** -0.5}
+        state = cache.states[self.STATE]
+        single = batch.num_decode is not None and batch.num_decode == batch.num_seqs == z.shape[0]
+        if single and self.value_dim <= ops.HEAD_STEP_MAX_NORMED:
+            ops.head_recurrence_gated(q, k, v, state, batch.cu_q, batch.state_slots, gate, out, eps=self.eps, **sizes)
+            return
+        o = ops.head_recurrence(q, k, v, state, batch.cu_q, batch.state_slots, single_tokens=single, **sizes)
+        ops.head_norm_gate(o, None, gate, out, heads=self.heads, dim=self.value_dim, eps=self.eps, act="silu")
+
+    def token_inputs(self):
+        return self.position.token_inputs()
+
+    def kernel_libraries(self):
+        return {"head_recurrence", "stream_ops", "gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide"}
+
+
+register_part("mixer", "retention", Retention)
 register_part("mixer", "rwkv_time_mix", RWKVTimeMix)
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
 register_part("mixer", "mlstm", MLSTM)

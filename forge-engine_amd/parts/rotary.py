@@ -14,6 +14,7 @@ import math
 
 import torch
 
+from ..kernels import ops
 from ..registry import register_part
 from .base import BuildContext, PositionEncoding
 
@@ -24,6 +25,7 @@ class RotaryPosition(PositionEncoding):
         """``precise``: the table is computed in 64-bit and rounded once, instead of with the
         reference's float32 expression."""
         super().__init__(ctx, prefix)
+        self.theta = float(theta)
         self.rotary_dim = head_dim if rotary_dim is None else rotary_dim
         if self.rotary_dim % 2 or not 0 < self.rotary_dim <= head_dim:
             raise ValueError(f"rotary_dim {self.rotary_dim} must be even and at most head_dim {head_dim}")
@@ -35,6 +37,13 @@ class RotaryPosition(PositionEncoding):
 
     def rotary(self):
         return self.inv_freq, self.rotary_dim
+
+    def table(self, batch):
+        """Formed once a step for all parts that turn alike."""
+        key = ("rotary", type(self), self.theta, self.rotary_dim)
+        if key not in batch.carry:
+            batch.carry[key] = ops.rotary_table(batch.positions, self.inv_freq)
+        return batch.carry[key]
 
 
 class YarnRotaryPosition(RotaryPosition):
@@ -64,6 +73,9 @@ class YarnRotaryPosition(RotaryPosition):
 
     def magnitude(self) -> float:
         return self._magnitude
+
+    def table(self, batch):
+        raise ValueError("stretched frequencies come with a magnitude, which the table does not hold")
 
 
 class NoPosition(PositionEncoding):

@@ -23,6 +23,9 @@ NORM_STD = 0.05
 
 
 def _draw(spec: ParamSpec, generator: torch.Generator, device) -> torch.Tensor:
+    if spec.kind == "int_table" and spec.choices:
+        scores = torch.rand((spec.shape[0], spec.choices), generator=generator, dtype=torch.float32, device=device)
+        return scores.argsort(dim=1)[:, :spec.shape[1]].to(torch.int32)
     if spec.kind == "int_table":
         return torch.zeros(spec.shape, dtype=torch.int32, device=device)
     if spec.init == "zeros":

@@ -382,7 +382,7 @@ def add_bias(update, bias):
 def conv_rope_norm_write(qkv, bias, conv_weight, conv_state, inv_freq, positions, token_seq, cu_q, state_slots, block_table,
                          key_pages, value_pages, q_out, *, num_seqs, q_heads, kv_heads, head_dim, value_dim, rotary_dim,
                          unit_norm_eps, taps, v_from=None, v_mix=0.0, v_keep=None, norm_weight_q=None, norm_weight_k=None,
-                         norm_first=False):
+                         norm_first=False, q_temp=None):
     tokens = qkv.shape[0]
     q_size, k_size, v_size = q_heads * head_dim, kv_heads * head_dim, kv_heads * value_dim
     channels = q_size + k_size + v_size
@@ -417,6 +417,9 @@ def conv_rope_norm_write(qkv, bias, conv_weight, conv_state, inv_freq, positions
         return x
 
     q = rotate_norm(y[:, :q_size].view(tokens, q_heads, head_dim), norm_weight_q)
+    if q_temp is not None:
+        runs = torch.floor((positions.double() + 1) / q_temp[1])
+        q = q * (1.0 + q_temp[0] * torch.log(runs + 1.0)).float().view(-1, 1, 1)
     k = rotate_norm(y[:, q_size:q_size + k_size].view(tokens, kv_heads, head_dim), norm_weight_k).to(qkv.dtype)
     v = y[:, q_size + k_size:]
     if v_from is not None:
@@ -436,7 +439,7 @@ def conv_rope_norm_write(qkv, bias, conv_weight, conv_state, inv_freq, positions
 
 def masked_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table, *, num_seqs, max_q_len, q_heads, kv_heads,
                      head_dim, value_dim, scale, window=None, chunk=None, sink=None, gate=None, num_decode=None, max_ctx=None,
-                     softcap=None, head_gate=False, slopes=None, dist_bias=None):
+                     softcap=None, head_gate=False, slopes=None, dist_bias=None, factor=1.0):
     block_size = key_pages.shape[2]
     groups = q_heads // kv_heads
     for s in range(num_seqs):
@@ -477,7 +480,7 @@ def masked_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table,
                     o = o * torch.sigmoid(gate[a + i, h].float())
                 elif gate is not None:
                     o = o * torch.sigmoid(gate[a + i, h * value_dim:(h + 1) * value_dim].float())
-                out[a + i, h * value_dim:(h + 1) * value_dim] = o.to(out.dtype)
+                out[a + i, h * value_dim:(h + 1) * value_dim] = (o * factor).to(out.dtype)
     return out
 
 
@@ -536,11 +539,13 @@ def mlstm_gate_scan(gates, bias, cap, maximum, cu_q, state_slots, out, *, num_se
     return out
 
 
-def hyper_norm(streams, update, mix, share, read, weight, bias, eps, out, rows=None, store=True, rms=False):
+def hyper_norm(streams, update, mix, share, read, weight, bias, eps, out, rows=None, store=True, rms=False, shift=None):
     count = streams.shape[0]
     x = streams
-    if update is not None:
-        y = _sum_parts(update)
+    if update is not None or shift is not None:
+        y = torch.zeros_like(streams[0]) if update is None else _sum_parts(update)
+        if shift is not None:
+            y = y + shift
         m = torch.eye(count) if mix is None else mix
         sh = torch.ones(count) if share is None else share
         x = torch.einsum("sr,stw->rtw", m, streams) + sh[:, None, None] * y[None]
@@ -629,15 +634,30 @@ def _gated(g, u, limit, alpha, form="bounded"):
     return g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + 1.0)
 
 
-def moe_experts(x, chosen, weights, gate_up, down, out, *, limit=0.0, alpha=1.0, extra=None, form="bounded", weight_input=False):
-    inner = gate_up.shape[1] // 2
+def moe_plan_table(ids, table, experts):
+    chosen = table[ids.long()]
+    order = torch.argsort(chosen.reshape(-1), stable=True).to(torch.int32)
+    counts = torch.bincount(chosen.reshape(-1).long(), minlength=experts)
+    offsets = torch.cat([torch.zeros(1, dtype=torch.long), torch.cumsum(counts, 0)]).to(torch.int32)
+    return offsets, order, torch.full(chosen.shape, 1.0 / table.shape[1])
+
+
+def moe_experts(x, chosen, weights, gate_up, down, out, *, limit=0.0, alpha=1.0, extra=None, form="bounded", weight_input=False, plan=None):
+    if plan is not None:
+        offsets, order = plan
+        flat = torch.empty(order.numel(), dtype=torch.int32, device=order.device)
+        for e in range(gate_up.shape[0]):
+            flat[order[int(offsets[e]):int(offsets[e + 1])].long()] = e
+        chosen = flat.view(weights.shape)
+    inner = gate_up.shape[1] // (1 if form == "relu_squared" else 2)
     for t in range(x.shape[0]):
         for k in range(chosen.shape[1]):
             e = int(chosen[t, k])
             gu = gate_up[e].float() @ x[t].float()
             if weight_input:
                 gu = gu * weights[t, k]
-            act = _gated(gu[:inner], gu[inner:], limit, alpha, form).to(x.dtype).float()
+            act = torch.relu(gu).square() if form == "relu_squared" else _gated(gu[:inner], gu[inner:], limit, alpha, form)
+            act = act.to(x.dtype).float()
             out[k, t] = (1.0 if weight_input else weights[t, k]) * (down[e].float() @ act)
     if extra is not None:
         out[0] += _sum_parts(extra)
@@ -654,7 +674,7 @@ def relu_squared(x):
     return torch.relu(x.float()).square().to(x.dtype)
 
 
-def causal_conv_act(u, weight, bias, state, token_seq, cu_q, state_slots, *, num_seqs, act="silu"):
+def causal_conv_act(u, weight, bias, state, token_seq, cu_q, state_slots, *, num_seqs, act="silu", single_tokens=False):
     channels, taps = weight.shape
     rows = u[:, :channels].float()
     out = torch.empty((u.shape[0], channels), dtype=u.dtype, device=u.device)
@@ -694,6 +714,65 @@ def selective_scan(x, dt_lin, dt_bias, a, bc, d, z, state, cu_q, state_slots, *,
             zt = z[t, :channels].double()
             out[t] = (y * zt * torch.sigmoid(zt)).to(out.dtype)
         state[slot] = memory.float()
+    return out
+
+
+def rotary_table(positions, inv_freq):
+    angle = positions.float()[:, None] * inv_freq[None, :]
+    return torch.stack([angle.cos(), angle.sin()], dim=-1)
+
+
+def head_recurrence(q, k, v, state, cu_q, state_slots, *, num_seqs, heads, key_dim, value_dim, rate, share=1, table=None, dt=None,
+                    dt_bias=None, skip=None, q_scale=1.0, k_scale=1.0, single_tokens=False, segment=None):
+    tokens = q.shape[0]
+
+    def rows(x, scale):
+        x = x.double().reshape(tokens, heads // share, key_dim)
+        if table is not None:
+            half = table.shape[1]
+            cos, sin = table[:, None, :, 0].double(), table[:, None, :, 1].double()
+            lo, hi = x[..., :half], x[..., half:2 * half]
+            x = torch.cat((lo * cos - hi * sin, hi * cos + lo * sin, x[..., 2 * half:]), dim=-1)
+        return (x * scale).repeat_interleave(share, dim=1)
+
+    qd, kd, vd = rows(q, q_scale), rows(k, k_scale), v.double().reshape(tokens, heads, value_dim)
+    step = torch.ones(tokens, heads, dtype=torch.float64, device=q.device)
+    if dt is not None:
+        step = torch.nn.functional.softplus(dt.double() + dt_bias.double())
+    decay = torch.exp(rate.double() * step)
+    out = torch.zeros((tokens, heads, value_dim), dtype=torch.float64, device=q.device)
+    for s in range(num_seqs):
+        lo, hi = int(cu_q[s]), int(cu_q[s + 1])
+        if hi == lo:
+            continue
+        slot = int(state_slots[s])
+        memory = state[slot].double()                       # [heads, value, key]
+        for t in range(lo, hi):
+            memory = decay[t][:, None, None] * memory + step[t][:, None, None] * vd[t][:, :, None] * kd[t][:, None, :]
+            out[t] = (memory * qd[t][:, None, :]).sum(-1)
+            if skip is not None:
+                out[t] += skip.double()[:, None] * vd[t]
+        state[slot] = memory.float()
+    return out.float()
+
+
+def head_recurrence_gated(q, k, v, state, cu_q, state_slots, gate, out, *, eps, num_seqs, heads, key_dim, value_dim, rate, share=1,
+                          table=None, q_scale=1.0, k_scale=1.0):
+    o = head_recurrence(q, k, v, state, cu_q, state_slots, num_seqs=num_seqs, heads=heads, key_dim=key_dim, value_dim=value_dim,
+                        rate=rate, share=share, table=table, q_scale=q_scale, k_scale=k_scale)
+    return head_norm_gate(o, None, gate, out, heads=heads, dim=value_dim, eps=eps, act="silu")
+
+
+def gated_group_norm(y, z, weight, out, *, groups, eps):
+    u = y * (z.float() * torch.sigmoid(z.float()))
+    u = _unit(u.view(u.shape[0], groups, -1), eps).reshape(u.shape)
+    out.copy_((u * weight).to(out.dtype))
+    return out
+
+
+def stream_sum_cast(h, update, shift, out):
+    total = h if update is None else h + _sum_parts(update)
+    out.copy_((total if shift is None else total + shift).to(out.dtype))
     return out
 
 
@@ -819,7 +898,8 @@ NAMES = ("decode_prepare_supported", "linear_in_parts", "embed_rows", "add_rmsno
          "conv_rope_norm_write", "masked_attention", "linear_recurrence", "mlstm_gate_scan",
          "hyper_norm", "embed_token_pairs", "scale_rows", "whole_norm_rope_write", "moe_route", "moe_experts", "linear_gated",
          "relu_squared", "causal_conv_act", "selective_scan", "rmsnorm_update_norm", "layernorm_update", "activate", "gate_rows",
-         "latent_norm_rope_write", "latent_query_pack", "latent_attention", "heads_product", "moe_route_grouped")
+         "latent_norm_rope_write", "latent_query_pack", "latent_attention", "heads_product", "moe_route_grouped",
+         "rotary_table", "head_recurrence", "head_recurrence_gated", "gated_group_norm", "stream_sum_cast", "moe_plan_table")
 
 
 def install(monkeypatch):
