@@ -112,8 +112,9 @@ def parse_args():
     parser.add_argument("--points", default=None, help="other decode batch sizes to report")
     parser.add_argument("--widths", default="1024,2048,4096",
                         help="--phase design: model widths at which Mazanex and Qwen3 are measured side by side")
-    parser.add_argument("--design", choices=("mazanex", "rekezen", "malusun", "dubizen"), default="mazanex",
+    parser.add_argument("--design", choices=("mazanex", "rekezen", "malusun", "dubizen", "talapel"), default="mazanex",
                         help="--phase design: which design is measured beside Qwen3")
+    parser.add_argument("--only", default="", help="--phase design: measure this model of the comparison alone")
     parser.add_argument("--phase", choices=("all", "decode", "prefill", "micro", "check", "design"), default="all",
                         help="run one phase only (for profiles); the record then holds that phase alone")
     parser.add_argument("--through", choices=("step", "scheduler"), default="step",
@@ -380,11 +381,36 @@ def dubizen_configs(width: int, layers: int) -> dict:
     return {"Dubizen": dubizen, "Rekezen": others["Rekezen"], "Qwen3": others["Qwen3"]}
 
 
-DESIGN_CONFIGS = {"mazanex": design_configs, "rekezen": rekezen_configs, "malusun": malusun_configs, "dubizen": dubizen_configs}
+def talapel_configs(width: int, layers: int) -> dict:
+    """Talapel beside Mazanex (mixers side by side, recurrences over a matrix state), Malusun (a state-space scan, a
+    mixture of experts) and Qwen3, at one width: heads of 128 in groups of four, the same vocabulary, as many layer
+    runs as the others have layers.  Talapel passes twice through half as many layers: capped attention beside a
+    state-space recurrence (twice the width inside, heads of 64, 128 states, eight groups) with the dense feed-forward
+    of three widths, retention (keys of 128, values of 256), attention beside the recurrence again, both with eight
+    experts as wide as the model of which a token's id names two."""
+    heads = max(4, width // 128)
+    side = {"left": {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                     "q_temp": {"coef": 0.5, "every": 512}},
+            "right": {"heads": width // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8},
+            "left_scale": 1.2, "right_scale": 0.8}
+    keep = {"heads": heads, "dim": 128, "vdim": 256, "decay": [1.0 - 2.0 ** -(5 + h % 6) for h in range(heads)],
+            "rot": {"dims": 128, "base": 10000.0}}
+    moe = {"kind": "moe", "router": {"experts": 8, "top": 2}, "expert": {"ff": width}}
+    kinds = [("parallel", side, {"kind": "dense", "ff": 3 * width}), ("retention", keep, moe), ("parallel", side, moe)]
+    own = max(1, layers // 2)
+    talapel = {"architecture": "Talapel", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5},
+               "loop": {"start": 0, "stop": own, "times": 2},
+               "layers": [{"type": kinds[i % 3][0], "mixer": kinds[i % 3][1], "mlp": kinds[i % 3][2]} for i in range(own)]}
+    others = dict(design_configs(width, layers), Malusun=malusun_configs(width, layers)["Malusun"])
+    return {"Talapel": talapel, "Mazanex": others["Mazanex"], "Malusun": others["Malusun"], "Qwen3": others["Qwen3"]}
+
+
+DESIGN_CONFIGS = {"mazanex": design_configs, "rekezen": rekezen_configs, "malusun": malusun_configs, "dubizen": dubizen_configs,
+                  "talapel": talapel_configs}
 
 
 def design_comparison(args) -> int:
-    """Prefill and decode throughput of Mazanex (or, with ``--design``, Rekezen, Malusun or Dubizen) beside the closest existing models at equal
+    """Prefill and decode throughput of Mazanex (or, with ``--design``, Rekezen, Malusun, Dubizen or Talapel) beside the closest existing models at equal
     width, layer count, feed-forward size and vocabulary; random weights, one JSON line a model and width."""
     import torch
 
@@ -399,6 +425,8 @@ def design_comparison(args) -> int:
     generator = torch.Generator().manual_seed(args.seed)
     for width in (int(w) for w in args.widths.split(",")):
         for label, raw in DESIGN_CONFIGS[args.design](width, layers).items():
+            if args.only and label.lower() != args.only.lower():
+                continue
             config = load_model_config(raw)
             model = random_model(config, args.seed, dtype=dtype, device=device)
             pages = -(-(max(args.prefill_tokens, prompt_len) + args.steps + args.warmup + 16) // args.block_size)
@@ -433,7 +461,8 @@ def design_comparison(args) -> int:
             for name in names:
                 runner.begin(name)
                 runner.step([StepEntry(name, tokens(prompt_len), [])])
-            entries = [StepEntry(name, [1], [0]) for name in names]
+            # different tokens: a design may choose experts by the token's id
+            entries = [StepEntry(name, [token], [0]) for name, token in zip(names, tokens(batch))]
             decode_ms = time_ms(lambda: runner.step(entries), args.warmup, args.steps)
             print(json.dumps({
                 "phase": "design", "model": label, "width": width, "layers": layers, "dtype": args.dtype,

@@ -48,8 +48,6 @@ def _check_attention(raw: dict, where: str) -> None:
     for key in ("dim", "vdim"):
         if read.integer(key) > 256:
             raise ConfigError(f"{where}: '{key}' of up to 256")
-    if raw["dim"] % 2:
-        raise ConfigError(f"{where}: 'dim' must be even")
     _finite(raw, "scale", where)
     if raw.get("softcap") is not None:
         read.number("softcap")

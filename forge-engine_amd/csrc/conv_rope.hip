@@ -13,6 +13,8 @@
 // (an RMS norm); with `norm_first` the norm comes before the rotation instead of behind it.
 // Queries may be multiplied by a temperature that grows with the position, 1 + coef ln(floor((p + 1) / every) + 1),
 // as the last step ahead of their store.
+// Rows of q and of the key pages may be wider than a head, and value pages hold more dims than a value (sizes that
+// another kernel's tiles want): the rest of a q or key row is set to zero, the rest of a value is left alone.
 // Values may lean on another layer's values of the same tokens: v <- (1 - mix) v + mix * v_from
 // (v_from [T, kv_heads * value_dim], dense), after the bias and the convolution and before the page
 // write; a layer that others lean on leaves its values, as stored, in v_keep (same shape).
@@ -31,7 +33,8 @@ __global__ __launch_bounds__(64) void conv_rope_norm_write_kernel(
     T* __restrict__ key_pages, T* __restrict__ value_pages, T* __restrict__ q_out, int q_heads, int kv_heads,
     int head_dim, int value_dim, int rotary_dim, float eps, int unit_norm, int taps, int block_size,
     int num_blocks, int slots, const T* __restrict__ v_from, float v_mix, T* __restrict__ v_keep,
-    const float* __restrict__ norm_wq, const float* __restrict__ norm_wk, int norm_first, float temp_coef, double temp_every) {
+    const float* __restrict__ norm_wq, const float* __restrict__ norm_wk, int norm_first, float temp_coef, double temp_every,
+    int key_row, int value_row) {
   __shared__ float y[CR_HEAD_MAX];
   const int t = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
   const int seq = token_seq[t];
@@ -76,7 +79,7 @@ __global__ __launch_bounds__(64) void conv_rope_norm_write_kernel(
       float v = y[d];
       if (v_from) v = (1.f - v_mix) * v + v_mix * load_as_float(v_from + dense + d);
       if (v_keep) store_from_float(v_keep + dense + d, v);
-      if (paged) store_from_float(value_pages + (((size_t)page * kv_heads + hv) * value_dim + d) * block_size + place, v);
+      if (paged) store_from_float(value_pages + (((size_t)page * kv_heads + hv) * value_row + d) * block_size + place, v);
     }
     return;
   }
@@ -110,10 +113,12 @@ __global__ __launch_bounds__(64) void conv_rope_norm_write_kernel(
   if (late) inv = unit();
   if (is_q) {
     if (temp_every > 0.0) inv *= 1.f + temp_coef * logf((float)floor((double)(pos + 1) / temp_every) + 1.f);
-    T* dst = q_out + (size_t)t * q_size + head * head_dim;
+    T* dst = q_out + ((size_t)t * q_heads + head) * key_row;
     for (int d = lane; d < n; d += 64) store_from_float(dst + d, y[d] * inv * (late && norm_w ? norm_w[d] : 1.f));
+    for (int d = n + lane; d < key_row; d += 64) store_from_float(dst + d, 0.f);
   } else if (paged) {
-    T* dst = key_pages + (((size_t)page * kv_heads + (head - q_heads)) * block_size + place) * head_dim;
+    T* dst = key_pages + (((size_t)page * kv_heads + (head - q_heads)) * block_size + place) * key_row;
+    for (int d = n + lane; d < key_row; d += 64) store_from_float(dst + d, 0.f);
     for (int d = lane; d < n; d += 64) store_from_float(dst + d, y[d] * inv * (late && norm_w ? norm_w[d] : 1.f));
   }
 }
@@ -152,7 +157,7 @@ extern "C" int fe_conv_rope_norm_write(const void* qkv, int dtype, long long qkv
                                        int rotary_dim, float eps, int unit_norm, int taps, int block_size,
                                        int num_blocks, int slots, const void* v_from, float v_mix, void* v_keep,
                                        const float* norm_wq, const float* norm_wk, int norm_first, float temp_coef,
-                                       double temp_every, hipStream_t stream) {
+                                       double temp_every, int key_row, int value_row, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
   if (q_heads <= 0 || kv_heads <= 0 || head_dim <= 0 || value_dim <= 0 || block_size <= 0 || num_blocks <= 0)
     return FE_BAD_ARGUMENT;
@@ -160,7 +165,7 @@ extern "C" int fe_conv_rope_norm_write(const void* qkv, int dtype, long long qkv
   if (taps < 0 || taps > 8 || (taps && !conv_w) || (taps > 1 && (!conv_state || slots < 1))) return FE_BAD_ARGUMENT;
   if (unit_norm && !(eps > 0.f)) return FE_BAD_ARGUMENT;
   if (!unit_norm && (norm_wq || norm_wk || norm_first)) return FE_BAD_ARGUMENT;
-  if (temp_every < 0.0) return FE_BAD_ARGUMENT;
+  if (temp_every < 0.0 || key_row < head_dim || value_row < value_dim) return FE_BAD_ARGUMENT;
   const long long channels = (long long)(q_heads + kv_heads) * head_dim + (long long)kv_heads * value_dim;
   if (head_dim > CR_HEAD_MAX || value_dim > CR_HEAD_MAX || qkv_stride < channels || q_heads + 2 * kv_heads > 65535)
     return FE_BAD_ARGUMENT;      // a head lives in LDS
@@ -170,7 +175,7 @@ extern "C" int fe_conv_rope_norm_write(const void* qkv, int dtype, long long qkv
       (const T*)qkv, (size_t)qkv_stride, bias, conv_w, conv_state, inv_freq, positions, token_seq, cu_q, state_slots, \
       block_table, table_stride, (T*)key_pages, (T*)value_pages, (T*)q_out, q_heads, kv_heads, head_dim,       \
       value_dim, rotary_dim, eps, unit_norm, taps, block_size, num_blocks, slots, (const T*)v_from, v_mix, (T*)v_keep, \
-      norm_wq, norm_wk, norm_first, temp_coef, temp_every)
+      norm_wq, norm_wk, norm_first, temp_coef, temp_every, key_row, value_row)
   if (dtype == FE_F32) LAUNCH(float);
   else if (dtype == FE_BF16) LAUNCH(bf16_t);
   else return FE_BAD_ARGUMENT;

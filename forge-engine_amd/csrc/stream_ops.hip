@@ -426,27 +426,29 @@ extern "C" int fe_add_bias(float* update, const float* bias, int rows, int width
 
 // ---------------------------------------------------------------- output gate
 // out[t][c] = x[t][c] * sigmoid(gate[t][c / share]) * factor, gate and out rows of any stride (out may be x itself);
-// `share` consecutive outputs take one gate (1: a gate per element; a head's width: a gate per head)
+// `share` consecutive outputs take one gate (1: a gate per element; a head's width: a gate per head); runs of `run`
+// elements lie x_run elements apart in x (rows of x_run * (width / run)): heads that x holds wider than they are
 template <typename T>
 __global__ void sigmoid_gate_kernel(const T* x, const T* __restrict__ gate, size_t gate_stride, T* out, size_t out_stride,
-                                    int width, long long count, int share, float factor) {
+                                    int width, long long count, int share, float factor, int run, int x_run) {
   const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= count) return;
   const long long t = i / width;
   const int c = (int)(i - t * width);
   const float g = load_as_float(gate + (size_t)t * gate_stride + c / share);
-  store_from_float(out + (size_t)t * out_stride + c, load_as_float(x + i) / (1.f + expf(-g)) * factor);
+  const long long at = t * (width / run) * x_run + (long long)(c / run) * x_run + c % run;
+  store_from_float(out + (size_t)t * out_stride + c, load_as_float(x + at) / (1.f + expf(-g)) * factor);
 }
 
 // bfloat16, a gate per element, everything in 16-byte pieces
 __global__ __launch_bounds__(256) void sigmoid_gate_bf16x8_kernel(const uint4* x, const bf16_t* __restrict__ gate, size_t gate_stride,
                                                                   bf16_t* out, size_t out_stride, int width8, long long count8,
-                                                                  float factor) {
+                                                                  float factor, int run8, int x_run8) {
   const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= count8) return;
   const long long t = i / width8;
-  const int c = (int)(i - t * width8) * 8;
-  const uint4 a = x[i], g = *(const uint4*)(gate + (size_t)t * gate_stride + c);
+  const int c8 = (int)(i - t * width8), c = c8 * 8;
+  const uint4 a = x[t * (width8 / run8) * x_run8 + (long long)(c8 / run8) * x_run8 + c8 % run8], g = *(const uint4*)(gate + (size_t)t * gate_stride + c);
   const uint32_t aw[4] = {a.x, a.y, a.z, a.w}, gw[4] = {g.x, g.y, g.z, g.w};
   uint32_t ow[4];
 #pragma unroll
@@ -459,24 +461,27 @@ __global__ __launch_bounds__(256) void sigmoid_gate_bf16x8_kernel(const uint4* x
 }
 
 extern "C" int fe_sigmoid_gate(const void* x, const void* gate, long long gate_stride, void* out, long long out_stride, int dtype,
-                               int rows, int width, int share, float factor, hipStream_t stream) {
+                               int rows, int width, int share, float factor, int run, int x_run, hipStream_t stream) {
   if (rows <= 0) return FE_OK;
-  if (width <= 0 || share < 1 || width % share || gate_stride < width / share || out_stride < width) return FE_BAD_ARGUMENT;
+  if (width <= 0 || share < 1 || width % share || gate_stride < width / share || out_stride < width || run < 1 ||
+      width % run || x_run < run)
+    return FE_BAD_ARGUMENT;
   const long long count = (long long)rows * width;
   const int blocks = (int)((count + 255) / 256);
-  if (dtype == FE_BF16 && share == 1 && width % 8 == 0 && gate_stride % 8 == 0 && out_stride % 8 == 0 &&
+  if (dtype == FE_BF16 && share == 1 && width % 8 == 0 && run % 8 == 0 && x_run % 8 == 0 && gate_stride % 8 == 0 && out_stride % 8 == 0 &&
       (((uintptr_t)x | (uintptr_t)gate | (uintptr_t)out) & 15) == 0) {
     const long long count8 = count / 8;
     sigmoid_gate_bf16x8_kernel<<<(int)((count8 + 255) / 256), 256, 0, stream>>>(
-        (const uint4*)x, (const bf16_t*)gate, (size_t)gate_stride, (bf16_t*)out, (size_t)out_stride, width / 8, count8, factor);
+        (const uint4*)x, (const bf16_t*)gate, (size_t)gate_stride, (bf16_t*)out, (size_t)out_stride, width / 8, count8, factor,
+        run / 8, x_run / 8);
     return fe_check_launch();
   }
   if (dtype == FE_F32)
     sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((const float*)x, (const float*)gate, (size_t)gate_stride, (float*)out,
-                                                           (size_t)out_stride, width, count, share, factor);
+                                                           (size_t)out_stride, width, count, share, factor, run, x_run);
   else if (dtype == FE_BF16)
     sigmoid_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)gate, (size_t)gate_stride, (bf16_t*)out,
-                                                            (size_t)out_stride, width, count, share, factor);
+                                                            (size_t)out_stride, width, count, share, factor, run, x_run);
   else return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }

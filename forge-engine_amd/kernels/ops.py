@@ -254,10 +254,14 @@ IN_PARTS_MAX_WEIGHT_BYTES = 64 << 20   # q/k/v from 5 rows: a larger weight than
                                        # sizes' 6144 x 4096, 50 MB, stays: 3.89 against 3.93)
 
 
+FEW_ROWS_LIBRARY_MIN_K = 4097   # ... unless K is short enough for the blocks of the few-rows kernel to keep x in registers
+                                # (8 rows: 27904 x 2048 in 24 us against the library's 35, 55808 x 4096 in 82 against 95)
+
+
 def _few_rows_to_library(x: Tensor, weight: Tensor) -> bool:
     """A product that stores bfloat16 (q/k/v), 5 to 16 rows, a weight too large for the kernels of
     few rows to win: the matrix library."""
-    return (FEW_ROWS_IN_PARTS < x.shape[0] <= SKINNY_MAX_ROWS
+    return (FEW_ROWS_IN_PARTS < x.shape[0] <= SKINNY_MAX_ROWS and weight.shape[1] >= FEW_ROWS_LIBRARY_MIN_K
             and weight.shape[0] * weight.shape[1] * weight.element_size() > IN_PARTS_MAX_WEIGHT_BYTES)
 
 
@@ -1270,7 +1274,8 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
     shape) receives the values as stored, for layers that lean on this one's.  ``norm_weight_q`` / ``norm_weight_k``
     (float32 [head_dim], shared by the heads): the unit norm's result times a weight per dim, an RMS norm;
     ``norm_first``: the norm comes before the rotation instead of behind it.  ``q_temp`` (coef, every): queries at
-    position p are multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)`` last of all."""
+    position p are multiplied by ``1 + coef * ln(floor((p + 1) / every) + 1)`` last of all.  Pages whose rows are wider than
+    a head (``masked_attention`` says why): q_out has the key pages' row width, q and key rows are filled up with zeros."""
     channels = (q_heads + kv_heads) * head_dim + kv_heads * value_dim
     for name, w in (("norm_weight_q", norm_weight_q), ("norm_weight_k", norm_weight_k)):
         if w is not None:
@@ -1286,8 +1291,6 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
     if qkv.dim() != 2 or qkv.shape[1] < channels or qkv.stride(1) != 1:
         raise KernelError(f"qkv must be [T, >= {channels}] with unit inner stride")
     _gpu(q_out, "q_out", qkv.dtype)
-    if q_out.shape != (tokens, q_heads * head_dim):
-        raise KernelError(f"q_out must be [{tokens}, {q_heads * head_dim}]")
     if bias is not None:
         _gpu(bias, "bias", torch.float32)
         if bias.shape != (channels,):
@@ -1314,11 +1317,13 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
     _gpu(block_table, "block_table", torch.int32)
     _gpu(key_pages, "key_pages", qkv.dtype)
     _gpu(value_pages, "value_pages", qkv.dtype)
-    if key_pages.dim() != 4 or key_pages.shape[1] != kv_heads or key_pages.shape[3] != head_dim:
-        raise KernelError(f"key pages must be [blocks, {kv_heads}, block_size, {head_dim}], got {tuple(key_pages.shape)}")
-    num_blocks, _, block_size, _ = key_pages.shape
-    if value_pages.shape != (num_blocks, kv_heads, value_dim, block_size):
-        raise KernelError(f"value pages are transposed: [blocks, {kv_heads}, {value_dim}, block_size], got {tuple(value_pages.shape)}")
+    if key_pages.dim() != 4 or key_pages.shape[1] != kv_heads or key_pages.shape[3] < head_dim:
+        raise KernelError(f"key pages must be [blocks, {kv_heads}, block_size, >= {head_dim}], got {tuple(key_pages.shape)}")
+    num_blocks, _, block_size, key_row = key_pages.shape
+    if q_out.shape != (tokens, q_heads * key_row):
+        raise KernelError(f"q_out must be [{tokens}, {q_heads * key_row}]")
+    if value_pages.dim() != 4 or value_pages.shape != (num_blocks, kv_heads, value_pages.shape[2], block_size) or value_pages.shape[2] < value_dim:
+        raise KernelError(f"value pages are transposed: [blocks, {kv_heads}, >= {value_dim}, block_size], got {tuple(value_pages.shape)}")
     if block_table.dim() != 2 or block_table.stride(1) != 1 or block_table.shape[0] < num_seqs:
         raise KernelError("block_table must be [sequences, max_blocks] with unit inner stride")
     for name, dense in (("v_from", v_from), ("v_keep", v_keep)):
@@ -1335,7 +1340,8 @@ def conv_rope_norm_write(qkv: Tensor, bias: Tensor | None, conv_weight: Tensor |
           c_int(value_dim), c_int(rotary_dim), c_float(unit_norm_eps if unit_norm_eps is not None else 0.0),
           c_int(1 if unit_norm_eps is not None else 0), c_int(taps), c_int(block_size), c_int(num_blocks), c_int(slots),
           _ptr(v_from), c_float(v_mix), _ptr(v_keep), _ptr(norm_weight_q), _ptr(norm_weight_k), c_int(1 if norm_first else 0),
-          c_float(q_temp[0] if q_temp is not None else 0.0), c_double(q_temp[1] if q_temp is not None else 0.0), _stream())
+          c_float(q_temp[0] if q_temp is not None else 0.0), c_double(q_temp[1] if q_temp is not None else 0.0),
+          c_int(key_row), c_int(value_pages.shape[2]), _stream())
     if taps > 1:
         _call("conv_rope", "fe_conv_state_update", _ptr(qkv), c_int(_code(qkv.dtype)), c_longlong(stride), _ptr(bias), _ptr(conv_state),
               _ptr(cu_q), _ptr(state_slots), c_int(num_seqs), c_int(channels), c_int(taps), c_int(slots), c_int(tokens),
@@ -1357,7 +1363,8 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     of key j loses slopes[h] * (p - j); ``dist_bias`` (float32 [Hq, span]): head h's score of key j gains
     dist_bias[h, min(p - j, span - 1)] (after the scale, which does not multiply it); ``value_pages`` None: a key's
     first ``value_dim`` dims are its value (a cache of keys only).  out [T, Hq * Dv]; with a gate its rows may have any
-    stride, and ``factor`` multiplies the gated result.  Scores and softmax
+    stride, and ``factor`` multiplies the gated result.  Pages may be wider than the heads (keys and values, and q,
+    filled up to sizes that the matrix-core kernels take): with a gate alone, whose kernel then leaves the rest out.  Scores and softmax
     float32.  A bfloat16 cache with keys and values of 64 or 128 elements, groups up to 8 and pages of
     a power of two >= 16 goes to the matrix-core kernels of ``paged_attention`` (single tokens and
     portions each to its own), with the gate in a small kernel behind them; everything else, and
@@ -1370,8 +1377,20 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     _gpu(ctx_len, "ctx_len", torch.int32)
     _gpu(block_table, "block_table", torch.int32)
     tokens = q.shape[0]
-    q_stride = _strided_rows(q, "q", q_heads * head_dim)
     out_stride = _strided_rows(out, "out", q_heads * value_dim)
+    if key_pages.dim() == 4 and value_pages is not None and value_pages.dim() == 4 and (
+            key_pages.shape[3] > head_dim or value_pages.shape[2] > value_dim):
+        if gate is None or out.shape != (tokens, q_heads * value_dim) or key_pages.shape[3] < head_dim or value_pages.shape[2] < value_dim:
+            raise KernelError("pages wider than the heads come with a gate")
+        wide = value_pages.shape[2]
+        attended = torch.empty((tokens, q_heads * wide), dtype=q.dtype, device=q.device)
+        masked_attention(q, key_pages, value_pages, attended, cu_q, ctx_len, block_table, num_seqs=num_seqs, max_q_len=max_q_len,
+                         q_heads=q_heads, kv_heads=kv_heads, head_dim=key_pages.shape[3], value_dim=wide, scale=scale, window=window,
+                         chunk=chunk, sink=sink, num_decode=num_decode, max_ctx=max_ctx, softcap=softcap, slopes=slopes,
+                         dist_bias=dist_bias)
+        _sigmoid_gate(attended, gate, out, q_heads, value_dim, wide, head_gate, factor)
+        return out
+    q_stride = _strided_rows(q, "q", q_heads * head_dim)
     if out.shape != (tokens, q_heads * value_dim) or out.dtype != q.dtype:
         raise KernelError(f"out must be [{tokens}, {q_heads * value_dim}] in q's dtype, got {tuple(out.shape)}")
     if gate is None and (factor != 1.0 or not out.is_contiguous()):
@@ -1422,9 +1441,7 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
                         num_decode=num_decode, max_ctx=max_ctx, chunk=chunk, sink=sink, softcap=softcap, slopes=slopes,
                         dist_bias=dist_bias)
         if gate is not None:
-            _call("stream_ops", "fe_sigmoid_gate", _ptr(attended), _ptr(gate), c_longlong(gate_stride), _ptr(out), c_longlong(out_stride),
-                  c_int(_code(out.dtype)), c_int(tokens), c_int(q_heads * value_dim), c_int(value_dim if head_gate else 1),
-                  c_float(factor), _stream())
+            _sigmoid_gate(attended, gate, out, q_heads, value_dim, value_dim, head_gate, factor)
         return out
     _call("attention_masked", "fe_masked_attention", _ptr(q), c_int(_code(q.dtype)), c_longlong(q_stride), _ptr(key_pages),
           _ptr(value_pages), _ptr(out), c_longlong(out_stride), c_float(factor), _ptr(gate), c_longlong(gate_stride), _ptr(sink), _ptr(cu_q), _ptr(ctx_len),
@@ -1433,6 +1450,17 @@ def masked_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
           c_int(window or 0), c_int(chunk or 0), c_float(scale), c_float(softcap or 0.0), c_int(1 if head_gate else 0),
           c_int(tokens), _ptr(slopes), _ptr(dist_bias), c_int(span), _stream())
     return out
+
+
+def _sigmoid_gate(x: Tensor, gate: Tensor, out: Tensor, heads: int, dim: int, x_dim: int, per_head: bool, factor: float) -> None:
+    """out[t, h, :dim] = x[t, h, :dim] * sigmoid(gate) * factor: x [T, heads * x_dim] dense, gate [T, heads * dim] (or a
+    number a head) and out [T, heads * dim] rows of any stride."""
+    gate_stride = _strided_rows(gate, "gate", heads if per_head else heads * dim)
+    if gate.dtype != x.dtype or out.dtype != x.dtype or gate.shape[0] != x.shape[0]:
+        raise KernelError("gate and out must be in x's dtype with one row a token")
+    _call("stream_ops", "fe_sigmoid_gate", _ptr(x), _ptr(gate), c_longlong(gate_stride), _ptr(out),
+          c_longlong(_strided_rows(out, "out", heads * dim)), c_int(_code(out.dtype)), c_int(x.shape[0]), c_int(heads * dim),
+          c_int(dim if per_head else 1), c_float(factor), c_int(dim), c_int(x_dim), _stream())
 
 
 MASKED_MAX_KEY_DIM = 640        # what the vector-ALU attention kernel holds of a key tile in LDS
@@ -2148,16 +2176,23 @@ def rotary_table(positions: Tensor, inv_freq: Tensor) -> Tensor:
     return table
 
 
-HEAD_SEGMENT = 128              # tokens a segment when a step's sequences are cut up (a multiple of 32)
-HEAD_SEGMENT_MIN_TOKENS = 128   # ... which happens when a sequence of the step may be this much longer than one token
-HEAD_STEP_MAX_NORMED = 1024     # widest head whose norm and gate the kernel for single tokens takes along
+# A long sequence is walked in segments side by side: short ones fill the chip and cost states in memory, so as many
+# as make about this many blocks (us a launch of 2,048 tokens, 64 heads of 128 x 64: 362 in one walk, 194 / 153 / 132 /
+# 159 in segments of 64 / 128 / 256 / 512; 32 heads: 360, 114 / 89 / 94 / 153; 8,192 tokens, 64 heads: 1407, 777 / 537 /
+# 455 / 429).
+HEAD_SEGMENT_BLOCKS = 512
+HEAD_SEGMENT_TOKENS = (64, 512)      # the shortest and the longest segment
+HEAD_SEGMENT_MIN_TOKENS = 128        # a step is cut up when a sequence of it may be this much longer than one token
+HEAD_STEP_MAX_NORMED = 1024          # widest head whose norm and gate the kernel for single tokens takes along
 
 
-def head_recurrence_segment(tokens: int, num_seqs: int) -> int:
-    """Tokens a segment, or 0 for one walk a sequence."""
-    if HEAD_SEGMENT <= 0 or tokens - num_seqs < HEAD_SEGMENT_MIN_TOKENS:
+def head_recurrence_segment(tokens: int, num_seqs: int, heads: int, value_dim: int) -> int:
+    """Tokens a segment (a multiple of 32), or 0 for one walk a sequence."""
+    if tokens - num_seqs < HEAD_SEGMENT_MIN_TOKENS:
         return 0
-    return HEAD_SEGMENT
+    segments = max(1, HEAD_SEGMENT_BLOCKS // (heads * -(-value_dim // 64)))
+    shortest, longest = HEAD_SEGMENT_TOKENS
+    return max(shortest, min(longest, -(-tokens // segments // 32) * 32))
 
 
 def _head_recurrence_checked(q, k, v, state, cu_q, state_slots, *, num_seqs, heads, share, key_dim, value_dim, rate, table,
@@ -2220,7 +2255,7 @@ def head_recurrence(q: Tensor, k: Tensor, v: Tensor, state: Tensor, cu_q: Tensor
               c_int(value_dim), c_int(tokens), _stream())
         return out
     if segment is None:
-        segment = head_recurrence_segment(tokens, num_seqs)
+        segment = head_recurrence_segment(tokens, num_seqs, heads, value_dim)
     seg_state = seg_sum = None
     slots = 0
     if segment:

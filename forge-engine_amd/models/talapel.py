@@ -39,7 +39,8 @@ def _mixer(config: TalapelConfig, kind: str, sizes: dict, prefix: str) -> PartSp
     attention = PartSpec("gqa_attention", {
         "hidden_size": width, "num_heads": left["heads"], "num_kv_heads": left["kv_heads"], "head_dim": left["dim"],
         "value_dim": left["vdim"], "scale": left["scale"], "softcap": left.get("softcap"), "query_temperature": left.get("q_temp"),
-        "bias": True, "bias_init": "small", "output_bias_init": "small", "output_gate": True, "output_scale": sizes["left_scale"], "position": PartSpec("none"),
+        "bias": True, "bias_init": "small", "output_bias_init": "small", "output_gate": True, "output_scale": sizes["left_scale"], "fill_rows": True,
+        "position": PartSpec("none"),
         "names": ATTENTION_NAMES,
     }, f"{prefix}.left")
     recurrence = PartSpec("state_space_duality", {

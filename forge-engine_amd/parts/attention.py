@@ -36,7 +36,8 @@ once, when the table is loaded); ``qk_norm_eps`` on the general path (the weight
 and k head, before the rotation, in the kernel that writes the pages);
 ``query_temperature`` (``{"coef": c, "every": n}``: queries at position p times
 ``1 + c ln(floor((p + 1) / n) + 1)``); ``output_scale`` (a factor on the layer's output, its bias included; it comes
-with an output gate, whose kernel applies it in float32);
+with an output gate, whose kernel applies it in float32); ``fill_rows`` (bfloat16 with an output gate: heads and values
+of sizes that the matrix-core kernels do not take, up to 128, lie in rows of 64 or 128 that are filled up with zeros);
 ``force_general`` (take the general path whatever the options).  A position part may scale its
 cosines and sines (``magnitude``).  With any of them the step takes the general path:
 one product for q, k, v (and the gate), one kernel for convolution, rotation, norms and the
@@ -66,14 +67,14 @@ class GroupedQueryAttention(Mixer):
                  fixed_sink: float | None = None, distance_slope_bits: float | None = None,
                  value_mix: str | None = None, value_mix_key: str = "values", force_general: bool = False,
                  bias_init: str = "zeros", distance_bias: dict | None = None, query_temperature: dict | None = None,
-                 output_scale: float = 1.0, output_bias_init: str = "zeros") -> None:
+                 output_scale: float = 1.0, output_bias_init: str = "zeros", fill_rows: bool = False) -> None:
         super().__init__(ctx, prefix)
         self.output_bias_init = output_bias_init
         self.bias_init = bias_init      # how random models draw the biases of q, k and v ("small": so that they show)
         if num_heads % num_kv_heads:
             raise ValueError("query heads must be a multiple of kv heads")
-        if head_dim % 2 or not 2 <= head_dim <= 256:
-            raise ValueError(f"head size {head_dim} is not supported: even sizes from 2 to 256")
+        if not 1 <= head_dim <= 256:
+            raise ValueError(f"head size {head_dim} is not supported: sizes to 256")
         self.hidden_size = hidden_size
         self.num_heads = num_heads
         self.num_kv_heads = num_kv_heads
@@ -133,6 +134,13 @@ class GroupedQueryAttention(Mixer):
                             or distance_slope_bits is not None or value_mix is not None
                             or self.output_bias != bool(bias) or force_general or distance_bias is not None
                             or query_temperature is not None)
+        if head_dim % 2 and not (self.general and position.kind == "none"):
+            raise ValueError(f"head size {head_dim} is not supported: even sizes from 2 to 256")
+        # the widths of a cached key's and value's row
+        self.key_row, self.value_row = head_dim, self.value_dim
+        widest = max(head_dim, self.value_dim)
+        if fill_rows and self.output_gate and own_kv and whole_norm_eps is None and ctx.dtype == torch.bfloat16 and widest <= 128:
+            self.key_row = self.value_row = 64 if widest <= 64 else 128
         if (value_mix is not None or fixed_sink is not None or distance_slope_bits is not None) and whole_norm_eps is not None:
             raise ValueError("value mixing, fixed sinks and distance slopes are not combined with the whole-projection norm")
         if self.general and qk_norm_eps is not None and (whole_norm_eps is not None or unit_norm_eps is not None):
@@ -292,8 +300,8 @@ class GroupedQueryAttention(Mixer):
 
     # ------------------------------------------------------------ running
     def cache_needs(self) -> CacheNeeds:
-        paged = PagedKV(self.num_kv_heads, self.head_dim, self.window,
-                        None if self.value_dim == self.head_dim else self.value_dim, chunk=self.chunk)
+        paged = PagedKV(self.num_kv_heads, self.key_row, self.window,
+                        None if self.value_row == self.key_row else self.value_row, chunk=self.chunk)
         if self.conv_taps < 2:        # one tap looks at the token's own row only: nothing to keep
             return CacheNeeds(paged=paged)
         # the last taps - 1 projected rows (q, k and v channels), exact in float32
@@ -367,7 +375,7 @@ class GroupedQueryAttention(Mixer):
 
     def _attend(self, qkv: Tensor, attn: Tensor, batch, cache: CacheView, writes_cache: bool, inv_freq, rotary_dim: int) -> None:
         """From the projections to the gated heads, side by side."""
-        q = torch.empty((qkv.shape[0], self.q_size), dtype=qkv.dtype, device=qkv.device)
+        q = torch.empty((qkv.shape[0], self.num_heads * self.key_row), dtype=qkv.dtype, device=qkv.device)
         magnitude = self.position.magnitude()
         if self.whole_norm_eps is not None:
             ops.whole_norm_rope_write(

@@ -427,14 +427,15 @@ def conv_rope_norm_write(qkv, bias, conv_weight, conv_state, inv_freq, positions
     v = v.view(tokens, kv_heads, value_dim).to(qkv.dtype)
     if v_keep is not None:
         v_keep.copy_(v.reshape(tokens, v_size))
-    q_out.copy_(q.reshape(tokens, q_size).to(q_out.dtype))
+    key_row = key_pages.shape[3]         # rows wider than a head are filled up with zeros
+    q_out.view(tokens, q_heads, key_row).zero_()[..., :head_dim] = q.to(q_out.dtype)
     block_size = key_pages.shape[2]
     for t in range(tokens):
         pos = int(positions[t])
         page = int(block_table[int(token_seq[t]), pos // block_size])
         assert page >= 0, "token without a page"
-        key_pages[page, :, pos % block_size] = k[t]
-        value_pages[page, :, :, pos % block_size] = v[t]
+        key_pages[page, :, pos % block_size] = torch.nn.functional.pad(k[t], (0, key_row - head_dim))
+        value_pages[page, :, :value_dim, pos % block_size] = v[t]
 
 
 def masked_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table, *, num_seqs, max_q_len, q_heads, kv_heads,
@@ -442,16 +443,18 @@ def masked_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table,
                      softcap=None, head_gate=False, slopes=None, dist_bias=None, factor=1.0):
     block_size = key_pages.shape[2]
     groups = q_heads // kv_heads
+    if key_pages.shape[3] > head_dim:
+        q = q.reshape(q.shape[0], q_heads, -1)[..., :head_dim].reshape(q.shape[0], -1)
     for s in range(num_seqs):
         a, b = int(cu_q[s]), int(cu_q[s + 1])
         ctx = int(ctx_len[s])
         if b == a:
             continue
-        keys = gather_pages(key_pages, block_table[s], ctx, block_size)                         # [kv, ctx, D]
+        keys = gather_pages(key_pages, block_table[s], ctx, block_size)[..., :head_dim]         # [kv, ctx, D]
         if value_pages is None:      # a cache of keys only: a key's first dims are its value
             values = keys[..., :value_dim]
         else:
-            values = gather_pages(value_pages.transpose(2, 3), block_table[s], ctx, block_size)     # [kv, ctx, Dv]
+            values = gather_pages(value_pages.transpose(2, 3), block_table[s], ctx, block_size)[..., :value_dim]     # [kv, ctx, Dv]
         for i in range(b - a):
             p = ctx - (b - a) + i
             first = 0

@@ -264,11 +264,13 @@ ATTENTION = [(4, 2, 64, 64, 16), (8, 1, 128, 128, 32), (4, 2, 48, 96, 16), (3, 3
 
 
 @pytest.mark.parametrize("heads,kv_heads,dim,vdim,block", ATTENTION)
+@pytest.mark.parametrize("filled", [False, True])
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_queries_by_position_and_one_key_that_stands_out(heads, kv_heads, dim, vdim, block, dtype):
+def test_queries_by_position_and_one_key_that_stands_out(heads, kv_heads, dim, vdim, block, filled, dtype):
     """Biases and the query temperature on the way into the pages, then capped attention with a gate and a factor, into
     rows of another stride: a portion and single tokens at page borders, far behind and right behind the one key that
-    stands out; the temperature's runs begin in the middle of a portion."""
+    stands out; the temperature's runs begin in the middle of a portion.  ``filled``: pages whose rows are wider than the
+    heads, as the matrix-core kernels want them (what lies in the rest of a value may be anything)."""
     from forge_engine_amd.kernels import ops
     g = torch.Generator().manual_seed(dim + vdim)
     scale, cap, temp = dim ** -0.5, 6.0, (0.8, 37)
@@ -283,24 +285,27 @@ def test_queries_by_position_and_one_key_that_stands_out(heads, kv_heads, dim, v
     for s, n in enumerate(pages):
         table[s, :n] = torch.tensor([free.pop() for _ in range(n)], dtype=torch.int32)
     channels = (heads + kv_heads) * dim + kv_heads * vdim
+    row = (64 if max(dim, vdim) <= 64 else 128) if filled else 0
+    key_row, value_row = max(row, dim), max(row, vdim)
     for target in ("first", "border"):
-        key_pages = torch.randn(sum(pages), kv_heads, block, dim, generator=g).to(dtype)
-        value_pages = torch.randn(sum(pages), kv_heads, vdim, block, generator=g).to(dtype)
+        key_pages = torch.zeros(sum(pages), kv_heads, block, key_row, dtype=dtype)
+        key_pages[..., :dim] = torch.randn(sum(pages), kv_heads, block, dim, generator=g).to(dtype)
+        value_pages = torch.randn(sum(pages), kv_heads, value_row, block, generator=g).to(dtype)
         qkv = torch.randn(tokens, channels + heads * vdim, generator=g).to(dtype)
         bias = torch.randn(channels, generator=g)
-        q = torch.empty(tokens, heads * dim, dtype=dtype)
+        q = torch.empty(tokens, heads * key_row, dtype=dtype)
         for s, n in enumerate(pages):          # a key of every cached context that all queries of its sequence favour
             place = 0 if target == "first" else max(0, (before[s] // block) * block - 1)
             if place < before[s]:
-                row = qkv[int(cu_q[s + 1]) - 1, :heads * dim].float() + bias[:heads * dim]
+                favourite = qkv[int(cu_q[s + 1]) - 1, :heads * dim].float() + bias[:heads * dim]
                 for hk in range(kv_heads):
-                    head = row[hk * (heads // kv_heads) * dim:][:dim]
-                    key_pages[int(table[s, place // block]), hk, place % block] = (12.0 * head / head.norm()).to(dtype)
+                    head = favourite[hk * (heads // kv_heads) * dim:][:dim]
+                    key_pages[int(table[s, place // block]), hk, place % block, :dim] = (12.0 * head / head.norm()).to(dtype)
         got_pages = [key_pages.clone().to(DEV), value_pages.clone().to(DEV)]
         kw = dict(num_seqs=seqs, q_heads=heads, kv_heads=kv_heads, head_dim=dim, value_dim=vdim, rotary_dim=0, unit_norm_eps=None, taps=0, q_temp=temp)
         slots = torch.zeros(seqs, dtype=torch.int32)
         refs.conv_rope_norm_write(qkv, bias, None, None, None, positions, token_seq, cu_q, slots, table, key_pages, value_pages, q, **kw)
-        q_gpu = torch.empty(tokens, heads * dim, dtype=dtype, device=DEV)
+        q_gpu = torch.full((tokens, heads * key_row), 7.0, dtype=dtype, device=DEV)
         wide = qkv.to(DEV)
         ops.conv_rope_norm_write(wide, bias.to(DEV), None, None, None, *to_dev(positions, token_seq, cu_q, slots, table), *got_pages, q_gpu, **kw)
         close(q_gpu, q, dtype)
@@ -357,3 +362,123 @@ def test_traces_match_the_plain_implementation(name, mode, dtype, folders, plain
     requests, want = plain_of(name, dtype, 3, LENGTHS[name])
     got = ru.run_trace(folders(name, dtype), dtype, TRACES[mode](requests), tmp_path, block_size=BLOCKS[name])
     tu.compare(got, want, dtype, float32_factor=2.0)
+
+
+def sharpen(tensors):
+    """Queries and keys larger and decays near one: one key of hundreds, and the first token, reach the logits."""
+    tu.enlarge(tensors, 3.0)
+    for name in tensors:
+        if name.endswith((".left.q", ".left.k")):
+            tensors[name] = (tensors[name].float() * 2.0).to(tensors[name].dtype)
+        if name.endswith(".A_log"):
+            tensors[name] = torch.full_like(tensors[name], -4.0)
+        if name.endswith(".dt_bias"):
+            tensors[name] = torch.full_like(tensors[name], -2.0)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_requests_with_sharp_attention_and_a_long_memory(dtype, tmp_path):
+    """Prompts of several hundred tokens, so that recurrences are walked in segments: whole, then the last 40 tokens one
+    by one, then in portions, then three at once; and the control that the first token moves the last logits."""
+    raw = dict(tu.MEDIUM, layers=[dict(layer) for layer in tu.MEDIUM["layers"]])
+    raw["layers"][1] = tu.layer(tu.retention(4, 64, 128, 64, decay=[0.999, 0.9999, 0.99, 1.0]), raw["layers"][1]["mlp"])
+    folder = tu.write_model(raw, 32, tmp_path / "sharp", change=sharpen)
+    requests = ru.make_requests({"vocab_size": raw["vocab"]}, 9, (500, 333, 129))
+    want = tu.plain_logits(folder, requests)
+    cfg, weights = tu.folder_weights(folder)
+    changed = [(requests["r0"][0] + 1) % raw["vocab"]] + requests["r0"][1:]
+    last = want[("r0", 499)]
+    assert float((plain.forward(cfg, weights, changed)[-1] - last).abs().max()) > 20 * (1e-5 + 1e-4 * float(last.abs().max()))
+    for mode, trace in (("whole", ru.trace_whole(requests)), ("tail", ru.trace_tail(requests, 40)),
+                        ("portions", ru.trace_portions(requests, sizes=(64, 17, 2, 230, 3, 48, 16, 2, 33), want_all=False)),
+                        ("mixed", ru.trace_mixed(requests, 11, max_live=3))):
+        got = ru.run_trace(folder, dtype, trace, tmp_path / mode, block_size=16)
+        tu.compare(got, want, dtype, fraction=0.06, float32_factor=4.0)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_captured_steps_equal_eager_steps_and_long_decoding(dtype, folders, plain_of):
+    """A prompt and then 150 single tokens, two requests side by side: steps replayed from captured graphs against the
+    same steps run eagerly (states move on once a step either way), and both against the plain implementation; then
+    portions whose shape repeats, captured and replayed with other contents."""
+    from forge_engine_amd.engine import ModelRunner, StepEntry, load_model
+    _, model = load_model(folders("M", dtype), dtype=dtype, device=DEV)
+    requests, want = plain_of("M", dtype, 21, (160, 171))
+    results = {}
+    for graphs in (True, False):
+        runner = ModelRunner(model, block_size=16, block_capacity=40, num_state_slots=3, use_graphs=graphs, eager_sightings=1)
+        got = {}
+        for name in requests:
+            runner.begin(name)
+        at = {"r0": 10, "r1": 21}
+        logits = runner.step([StepEntry(n, requests[n][:at[n]], [at[n] - 1]) for n in requests])
+        for row, n in zip(logits, requests):
+            got[(n, at[n] - 1)] = row.cpu().clone()
+        for _ in range(150):
+            logits = runner.step([StepEntry(n, [requests[n][at[n]]], [0]) for n in requests])
+            for row, n in zip(logits, requests):
+                got[(n, at[n])] = row.cpu().clone()
+                at[n] += 1
+        assert runner.graph_replays >= (140 if graphs else 0) and (graphs or runner.graph_replays == 0)
+        for name in requests:
+            runner.end(name)
+            runner.begin(name)
+        replays = runner.portion_graph_replays
+        for start in range(0, 160, 40):          # the same shape four times: eager, captured, replayed
+            logits = runner.step([StepEntry(n, requests[n][start:start + 40], [39]) for n in requests])
+            for row, n in zip(logits, requests):
+                got[(n, start + 39, "portions")] = row.cpu().clone()
+        assert runner.portion_graph_replays - replays >= (2 if graphs else 0)
+        results[graphs] = got
+        tu.compare({key[:2]: row for key, row in got.items() if len(key) == 2}, want, dtype, float32_factor=2.0)
+        tu.compare({key[:2]: row for key, row in got.items() if len(key) == 3}, want, dtype, float32_factor=2.0)
+    for key, row in results[True].items():
+        torch.testing.assert_close(row, results[False][key], rtol=0, atol=1e-4 if dtype == "float32" else 3e-2)
+
+
+def test_first_tokens_and_slot_reuse(folders):
+    """A request that takes over the state slot of one that ended starts from empty states in every pass, whatever the
+    slot still holds; requests of one and two tokens."""
+    from forge_engine_amd.engine import ModelRunner, StepEntry, load_model
+    folder = folders("A", "float32")
+    _, model = load_model(folder, dtype="float32", device=DEV)
+    runner = ModelRunner(model, block_size=4, block_capacity=16, num_state_slots=1)
+    cfg, weights = tu.folder_weights(folder)
+    for tokens in ([5, 80, 17, 3], [44], [7, 7], [80, 5, 17, 3, 3, 3, 8, 1, 2]):
+        runner.begin("only")
+        rows = [runner.step([StepEntry("only", [token], [0])])[0].cpu().clone() for token in tokens]
+        runner.end("only")
+        for got, row in zip(rows, plain.forward(cfg, weights, tokens)):
+            assert float((got.double() - row).abs().max()) <= 2e-5 + 2e-4 * float(row.abs().max())
+
+
+def test_generation_through_the_entry_point_and_the_command_line(folders):
+    import os
+    import subprocess
+    import sys
+    from conftest import ROOT
+    from forge_engine_amd.config import SchedulerConfig
+    from forge_engine_amd.engine import engine_from_folder
+    from forge_engine_amd.sampling import SamplingParams
+
+    folder = folders("A", "float32")
+    cfg, weights = tu.folder_weights(folder)
+
+    def greedy(prompt, count):
+        tokens = list(prompt)
+        for _ in range(count):
+            tokens.append(int(plain.forward(cfg, weights, tokens)[-1].argmax()))
+        return tokens[len(prompt):]
+
+    prompts = list(ru.make_requests({"vocab_size": tu.SMALL_A["vocab"]}, 13, (11, 3, 25)).values())
+    want = [greedy(prompt, 8) for prompt in prompts]
+    engine = engine_from_folder(folder, scheduler_config=SchedulerConfig(block_size=4, block_capacity=128, token_budget=16),
+                                dtype="float32", eos_token_ids=[])
+    ids = [engine.submit(prompt, sampling_params=SamplingParams(max_new_tokens=8)) for prompt in prompts]
+    engine.run_until_idle()
+    assert [list(engine.request(i).output_token_ids) for i in ids] == want
+    command = [sys.executable, str(ROOT / "bin" / "forge-engine"), "generate", "--model", str(folder), "--dtype", "float32",
+               "--max-new-tokens", "8", "--block-size", "4", "--prompt-ids", ",".join(map(str, prompts[0]))]
+    done = subprocess.run(command, capture_output=True, text=True, timeout=300, env=dict(os.environ))
+    assert done.returncode == 0, done.stderr[-2000:]
+    assert ",".join(map(str, want[0])) in done.stdout.replace(" ", "")
