@@ -25,7 +25,7 @@ MIXER_TYPES = ("parallel", "retention")
 MLP_KINDS = ("dense", "moe")
 
 
-def _section(raw: dict, key: str, where: str) -> dict:
+def section(raw: dict, key: str, where: str) -> dict:
     value = raw.get(key)
     if not isinstance(value, dict):
         raise ConfigError(f"{where} needs an object '{key}'")
@@ -52,12 +52,12 @@ def _check_attention(raw: dict, where: str) -> None:
     if raw.get("softcap") is not None:
         read.number("softcap")
     if raw.get("q_temp") is not None:
-        temp = _section(raw, "q_temp", where)
+        temp = section(raw, "q_temp", where)
         _finite(temp, "coef", where)
         KeyReader(temp).number("every")
 
 
-def _check_state_space(raw: dict, where: str) -> None:
+def check_state_space(raw: dict, where: str) -> None:
     read = KeyReader(raw)
     heads, vdim, groups, parts = (read.integer(key) for key in ("heads", "vdim", "groups", "norm_groups"))
     if read.integer("state") > 256:
@@ -80,7 +80,7 @@ def _check_retention(raw: dict, where: str) -> None:
     if (not isinstance(decay, list) or len(decay) != heads
             or not all(isinstance(d, (int, float)) and not isinstance(d, bool) and 0.0 < d < float("inf") for d in decay)):
         raise ConfigError(f"{where}: 'decay' must list {heads} positive numbers, got {decay!r}")
-    rot = _section(raw, "rot", where)
+    rot = section(raw, "rot", where)
     dims = KeyReader(rot).integer("dims", minimum=2)
     KeyReader(rot).number("base")
     if dims % 2 or dims > dim:
@@ -95,8 +95,8 @@ def _check_mlp(mlp: Any, where: str) -> None:
     if mlp["kind"] == "dense":
         KeyReader(mlp).integer("ff")
         return
-    KeyReader(_section(mlp, "expert", where)).integer("ff")
-    router = KeyReader(_section(mlp, "router", where))
+    KeyReader(section(mlp, "expert", where)).integer("ff")
+    router = KeyReader(section(mlp, "router", where))
     experts, top = router.integer("experts"), router.integer("top")
     if top > experts:
         raise ConfigError(f"{where}: router.top ({top}) exceeds router.experts ({experts})")
@@ -110,18 +110,18 @@ def _check_layer(layer: Any, where: str) -> None:
     kind = layer.get("type")
     if kind not in MIXER_TYPES:
         raise ConfigError(f"{where}: unknown mixer type {kind!r} (known: {', '.join(MIXER_TYPES)})")
-    mixer = _section(layer, "mixer", where)
+    mixer = section(layer, "mixer", where)
     if kind == "retention":
         _check_retention(mixer, f"{where}.mixer")
     else:
-        _check_attention(_section(mixer, "left", where), f"{where}.mixer.left")
-        _check_state_space(_section(mixer, "right", where), f"{where}.mixer.right")
+        _check_attention(section(mixer, "left", where), f"{where}.mixer.left")
+        check_state_space(section(mixer, "right", where), f"{where}.mixer.right")
         for key in ("left_scale", "right_scale"):
             _finite(mixer, key, f"{where}.mixer")
     _check_mlp(layer.get("mlp"), f"{where}.mlp")
 
 
-def _loop(raw: Any, layers: int) -> tuple[int, int, int] | None:
+def read_loop(raw: Any, layers: int) -> tuple[int, int, int] | None:
     if raw is None:
         return None
     if not isinstance(raw, dict):
@@ -158,13 +158,13 @@ class TalapelConfig(ModelConfig):
         for index, layer in enumerate(layers):
             _check_layer(layer, f"layers[{index}]")
         embedding = raw.get("embedding")
-        scale = 1.0 if embedding is None else _finite(_section(raw, "embedding", "config.json"), "scale", "embedding")
+        scale = 1.0 if embedding is None else _finite(section(raw, "embedding", "config.json"), "scale", "embedding")
         eos = raw.get("eos_token_id")
         if eos is not None and (isinstance(eos, bool) or not isinstance(eos, int)):
             raise ConfigError(f"'eos_token_id' must be an integer, got {eos!r}")
         return cls(vocab=read.integer("vocab"), width=read.integer("width"),
-                   norm_eps=KeyReader(_section(raw, "norm", "config.json")).number("eps"),
-                   layers_json=json.dumps(layers, sort_keys=True), loop=_loop(raw.get("loop"), len(layers)),
+                   norm_eps=KeyReader(section(raw, "norm", "config.json")).number("eps"),
+                   layers_json=json.dumps(layers, sort_keys=True), loop=read_loop(raw.get("loop"), len(layers)),
                    embedding_scale=scale, eos_token_id=eos)
 
     def to_dict(self) -> dict[str, Any]:

@@ -22,6 +22,11 @@
 // rows and long contexts; each run leaves its unnormalised output, maximum and sum in float32, and a
 // second kernel merges them in order.  Slots beyond the context may hold anything: their values are
 // masked to zero in the operand.
+//
+// window > 0: the token at position p reads keys p - window + 1 .. p only; a block's walk begins at the tile of its first
+// row's first key, and the values of keys below that one (their pages may have been given back, or be missing)
+// are masked to zero like those beyond the context.  sink (float32 [heads]): exp(sink_h) joins head h's denominator
+// once, with no key and no value: the walk of the first run starts from maximum sink_h and sum 1.
 #include "common.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -103,7 +108,7 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
     const bf16_t* __restrict__ value_pages, bf16_t* __restrict__ out, float* __restrict__ part_o,
     float* __restrict__ part_ml, const int* __restrict__ cu_q, const int* __restrict__ ctx_len,
     const int* __restrict__ block_table, int table_stride, int heads, int block_shift, int num_blocks,
-    float scale_log2, int splits, int total_rows) {
+    float scale_log2, int splits, int total_rows, int window, const float* __restrict__ sink) {
   constexpr int KC = DK / 32, DT = DV / 16, CHUNKS = DK / 8;
   constexpr int K_UNITS = LA_KEYS * CHUNKS, V_UNITS = DV * 4;             // 16-byte units of a tile's keys and values
   constexpr int LOADS = (K_UNITS + V_UNITS) / 64;                         // load instructions a tile, 64 units each
@@ -134,9 +139,14 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
   const bool wave_ok = row0 + wave * 16 < rows_total;
   const int wave_pos_max = before + (min(rows_total, row0 + wave * 16 + 16) - 1) / heads;
   const int block_pos_max = before + (min(rows_total, row0 + LA_ROWS) - 1) / heads;
+  // the first keys that this lane's row, the wave's first row and the block's first row read
+  const int my_first = window > 0 ? max(0, pos - window + 1) : 0;
+  const int wave_first = window > 0 ? max(0, before + (row0 + wave * 16) / heads - window + 1) : 0;
+  const int block_first = window > 0 ? max(0, before + row0 / heads - window + 1) : 0;
+  const int tile0 = block_first / LA_KEYS;
   const int tiles = block_pos_max / LA_KEYS + 1;
-  const int run = (tiles + splits - 1) / splits;
-  const int t_lo = split * run, t_hi = min(tiles, t_lo + run);
+  const int run = (tiles - tile0 + splits - 1) / splits;
+  const int t_lo = tile0 + split * run, t_hi = min(tiles, t_lo + run);
 
   bf16x8 qb[KC];
   {
@@ -149,6 +159,10 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
 #pragma unroll
   for (int t = 0; t < DT; ++t) o[t] = floatx4{0.f, 0.f, 0.f, 0.f};
   float m_run = -INFINITY, l_run = 0.f;
+  if (sink && split == 0) {
+    m_run = sink[head] * 1.4426950408889634f;
+    l_run = 1.f;
+  }
   const int* table = block_table + (size_t)seq * table_stride;
   const int last_key = ctx - 1;
 
@@ -227,7 +241,7 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
       fetch(tile + 1, buffer ^ 1);
       page_ids(tile + 2);         // keys beyond the context read the last key's entry: always a valid index
     }
-    if (!wave_ok || kb > wave_pos_max) continue;            // the whole wave: no row, or no row that sees this tile
+    if (!wave_ok || kb > wave_pos_max || kb + LA_KEYS <= wave_first) continue;   // the whole wave: no row, or no row that sees this tile
     const unsigned int keys_at = lds_at + buffer * TILE_BYTES, values_at = keys_at + K_UNITS * 16;
 
     floatx4 st[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
@@ -247,7 +261,7 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int key = kb + 8 * lq + j;
-      s[j] = (row_ok && key <= pos) ? st[j >> 2][j & 3] * scale_log2 : -INFINITY;
+      s[j] = (row_ok && key <= pos && key >= my_first) ? st[j >> 2][j & 3] * scale_log2 : -INFINITY;
       mx = fmaxf(mx, s[j]);
     }
     mx = max_xor32(max_xor16(mx));
@@ -265,17 +279,18 @@ __global__ __launch_bounds__(256, (DK / 8 + DV / 4 > 160) ? 1 : 2) void latent_a
     m_run = m_new;
     const bf16x8 pb = __builtin_bit_cast(bf16x8, uintx4{pack_two(s[0], s[1]), pack_two(s[2], s[3]), pack_two(s[4], s[5]), pack_two(s[6], s[7])});
 
-    // O^T: this lane's eight keys of the value operand; in the tile that crosses the context's end those
-    // beyond it are cleared
+    // O^T: this lane's eight keys of the value operand; in a tile that crosses the context's end, or the first key
+    // that the block reads, those outside are cleared
     const bool rescale = __builtin_amdgcn_ballot_w64(corr != 1.f) != 0;      // the whole wave: once the maxima have settled, nothing to do
-    const bool crosses = kb + LA_KEYS > ctx;
+    const bool crosses = kb + LA_KEYS > ctx || kb < block_first;
     uintx4 v_mask = uintx4{~0u, ~0u, ~0u, ~0u};
     if (crosses) {
       const int vkey = kb + 8 * lq;
 #pragma unroll
       for (int w = 0; w < 4; ++w) {
-        const unsigned int lo = vkey + 2 * w < ctx ? 0x0000ffffu : 0u;
-        const unsigned int hi = vkey + 2 * w + 1 < ctx ? 0xffff0000u : 0u;
+        const int k0 = vkey + 2 * w, k1 = k0 + 1;
+        const unsigned int lo = k0 < ctx && k0 >= block_first ? 0x0000ffffu : 0u;
+        const unsigned int hi = k1 < ctx && k1 >= block_first ? 0xffff0000u : 0u;
         v_mask[w] = lo | hi;
       }
     }
@@ -369,7 +384,7 @@ template <int DK, int DV>
 static int launch_latent(const void* q, long long q_stride, const void* key_pages, const void* value_pages, void* out,
                          float* part_o, float* part_ml, const int* cu_q, const int* ctx_len, const int* block_table,
                          int table_stride, int num_seqs, int max_q_len, int heads, int block_size, int num_blocks,
-                         float scale, int splits, int tokens, hipStream_t stream) {
+                         float scale, int splits, int tokens, int window, const float* sink, hipStream_t stream) {
   const long long rows = (long long)max_q_len * heads;
   const dim3 grid((unsigned)((rows + LA_ROWS - 1) / LA_ROWS), splits, num_seqs);
   constexpr int lds = 2 * (LA_KEYS * DK + DV * 32) * 2;   // two buffers of a tile's keys and its transposed values
@@ -384,7 +399,7 @@ static int launch_latent(const void* q, long long q_stride, const void* key_page
   latent_attention_kernel<DK, DV><<<grid, 256, lds, stream>>>(
       (const bf16_t*)q, (size_t)q_stride, (const bf16_t*)key_pages, (const bf16_t*)value_pages, (bf16_t*)out, part_o,
       part_ml, cu_q, ctx_len, block_table, table_stride, heads, block_shift, num_blocks, scale * 1.4426950408889634f,
-      splits, tokens * heads);
+      splits, tokens * heads, window, sink);
   if (splits > 1) latent_merge_kernel<<<tokens * heads, 128, 0, stream>>>(part_o, part_ml, (bf16_t*)out, splits, tokens * heads, DV);
   return fe_check_launch();
 }
@@ -399,16 +414,16 @@ extern "C" int fe_latent_attention(const void* q, long long q_stride, const void
                                    float* part_o, float* part_ml, const int* cu_q, const int* ctx_len,
                                    const int* block_table, int table_stride, int num_seqs, int max_q_len, int heads,
                                    int row_dim, int value_dim, int block_size, int num_blocks, float scale, int splits,
-                                   int tokens, hipStream_t stream) {
+                                   int tokens, int window, const float* sink, hipStream_t stream) {
   if (tokens <= 0 || num_seqs <= 0) return FE_OK;
-  if (heads < 1 || max_q_len < 1 || block_size < 8 || (block_size & (block_size - 1)) || num_blocks < 1 || splits < 1 || splits > 64 ||
+  if (heads < 1 || max_q_len < 1 || block_size < 8 || (block_size & (block_size - 1)) || num_blocks < 1 || splits < 1 || splits > 64 || window < 0 ||
       num_seqs > 65535 || q_stride < (long long)heads * row_dim || q_stride % 8 || (splits > 1 && (!part_o || !part_ml)) ||
       (long long)tokens * heads > 0x7fffffffLL || !fe_latent_attention_supported(row_dim, value_dim))
     return FE_BAD_ARGUMENT;
 #define CASE(DK, DV)                                                                                                   \
   if (row_dim == DK && value_dim == DV)                                                                                \
     return launch_latent<DK, DV>(q, q_stride, key_pages, value_pages, out, part_o, part_ml, cu_q, ctx_len, block_table, \
-                                 table_stride, num_seqs, max_q_len, heads, block_size, num_blocks, scale, splits, tokens, stream)
+                                 table_stride, num_seqs, max_q_len, heads, block_size, num_blocks, scale, splits, tokens, window, sink, stream)
   CASE(576, 512);
   CASE(320, 256);
   CASE(192, 128);

@@ -18,8 +18,9 @@
 //   lane l supplies A[m = l % 16][k = 8*(l / 16) .. +8] and B[k = 8*(l / 16) .. +8][n = l % 16]
 //   and receives D[m = 4*(l / 16) + i][n = l % 16], i < 4.
 //
-// Epilogues: store float32, store bfloat16, or silu(gate) * up -> bfloat16.
+// Epilogues: store float32, store bfloat16, or act(gate) * up -> bfloat16 (gate_act.h).
 #include "common.h"
+#include "gate_act.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float floatx4;
@@ -32,7 +33,6 @@ typedef __attribute__((ext_vector_type(4))) unsigned int uintx4;
 #define EPI_BF16 1
 #define EPI_SWIGLU 2
 
-__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + __expf(-g)) * u; }
 
 template <int MT, int NW>
 struct StepRegs {
@@ -45,7 +45,7 @@ struct StepRegs {
 template <int MT, int NT, int EPI, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ out_base, int M, int N,
-    int K, long long ldw, long long ldo, int second_offset, int steps_per_split, long long part_stride) {
+    int K, long long ldw, long long ldo, int second_offset, int steps_per_split, long long part_stride, GateAct act) {
   constexpr int NW = EPI == EPI_SWIGLU ? 2 * NT : NT;   // weight tiles per wave
   // blockIdx.y: which part of K this block sums (float32 epilogue only); its sums go to a part of their own
   void* out = EPI == EPI_F32 ? (void*)((float*)out_base + (size_t)blockIdx.y * part_stride) : out_base;
@@ -157,7 +157,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(
           if (m < M && n < N) {
             if (EPI == EPI_SWIGLU) {
               if (half == 0) gate = v;
-              else ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(silu_mul(gate, v));
+              else ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(gate_times(gate, v, act));
             } else if (EPI == EPI_F32) {
               ((float*)out)[(size_t)m * ldo + n] = v;
             } else {
@@ -178,6 +178,7 @@ struct SkinnyCall {
   int second_offset;      // rows between a gate row and its up row
   int splits;             // parts of K, each summed by blocks of its own (float32 epilogue)
   long long part_stride;  // floats between the parts' outputs
+  GateAct act;
   hipStream_t stream;
 };
 
@@ -189,7 +190,7 @@ static int launch_skinny(const SkinnyCall& c) {
   const int per_split = (steps + splits - 1) / splits;
   gemm_skinny_kernel<MT, NT, EPI, WAVES><<<dim3(blocks, splits), WAVES * 64, 0, c.stream>>>(
       (const bf16_t*)c.x, (const bf16_t*)c.w, c.out, c.M, c.N, c.K, c.ldw, c.ldo, c.second_offset, per_split,
-      c.part_stride);
+      c.part_stride, c.act);
   return fe_check_launch();
 }
 
@@ -209,7 +210,7 @@ static int launch_skinny(const SkinnyCall& c) {
 template <int EPI, int XS, int WAVES>
 __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_resident_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ out, int M, int N,
-    int K, long long ldw, long long ldo, int second_offset, int tiles) {
+    int K, long long ldw, long long ldo, int second_offset, int tiles, GateAct act) {
   constexpr int HALVES = EPI == EPI_SWIGLU ? 2 : 1;
   __shared__ __attribute__((aligned(16))) float red[HALVES][WAVES][64][4];
 
@@ -278,7 +279,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_resident_kernel(
       const int m = (src_lane >> 4) * 4 + i;
       const int n = tile * ROWS + (src_lane & 15);
       if (m < M && n < N) {
-        if (EPI == EPI_SWIGLU) ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(silu_mul(v[0], v[HALVES - 1]));
+        if (EPI == EPI_SWIGLU) ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(gate_times(v[0], v[HALVES - 1], act));
         else if (EPI == EPI_F32) ((float*)out)[(size_t)m * ldo + n] = v[0];
         else ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(v[0]);
       }
@@ -293,7 +294,7 @@ static bool resident_fits(int M, int N, int K) {
 
 template <int EPI>
 static int launch_resident(const void* x, const void* w, void* out, int M, int N, int K, long long ldw,
-                           long long ldo, int second_offset, hipStream_t stream) {
+                           long long ldo, int second_offset, GateAct act, hipStream_t stream) {
   const int tiles = (N + ROWS - 1) / ROWS;
   const int steps = (K + KSTEP - 1) / KSTEP;
   const bool wide = steps > 4 * RESIDENT_WAVES;
@@ -303,7 +304,7 @@ static int launch_resident(const void* x, const void* w, void* out, int M, int N
   const int xs = (steps + waves - 1) / waves;
 #define FE_GO(XS, WV)                                                                               \
   gemm_skinny_resident_kernel<EPI, XS, WV><<<blocks, WV * 64, 0, stream>>>(                          \
-      (const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldw, ldo, second_offset, tiles)
+      (const bf16_t*)x, (const bf16_t*)w, out, M, N, K, ldw, ldo, second_offset, tiles, act)
   if (wide) FE_GO(3, RESIDENT_WAVES_WIDE);
   else if (xs <= 1) FE_GO(1, RESIDENT_WAVES);
   else if (xs == 2) FE_GO(2, RESIDENT_WAVES);
@@ -363,11 +364,13 @@ static int dispatch(int mt, int nt, int waves, const SkinnyCall& c) {
 // the resident variant (refused where it does not apply); 0 uses it wherever it applies.
 // splits > 1 (float32 epilogue, at most 16): K is cut into that many parts of whole 128-steps,
 // each summed by blocks of its own into out + part * part_stride; the caller adds the parts up
-// (in a fixed order, so the result stays deterministic).
+// (in a fixed order, so the result stays deterministic).  activation: the gated epilogue's (gate_act.h).
 extern "C" int fe_gemm_skinny(const void* x, const void* w, void* out, int M, int N, int K,
                               long long ldw, long long ldo, int epilogue, int tiles, int waves,
-                              int splits, long long part_stride, hipStream_t stream) {
+                              int splits, long long part_stride, int activation, hipStream_t stream) {
   if (M < 1) return FE_OK;
+  GateAct act;
+  if (!gate_act(activation, &act)) return FE_BAD_ARGUMENT;
   if (splits < 1 || splits > 16 || (splits > 1 && (epilogue != EPI_F32 || part_stride < (long long)M * ldo)))
     return FE_BAD_ARGUMENT;
   if (M > 64 || N < 1 || K < 8 || K % 8 || ldw < K || ldw % 8 || ldo < N) return FE_BAD_ARGUMENT;
@@ -378,9 +381,9 @@ extern "C" int fe_gemm_skinny(const void* x, const void* w, void* out, int M, in
   const int weight_rows = epilogue == EPI_SWIGLU ? 2 * N : N;
   if (tiles == -1 || (tiles == 0 && waves == 0 && splits == 1 && resident_fits(M, N, K))) {
     if (M > 16 || steps > RESIDENT_MAX_STEPS || splits != 1) return FE_BAD_ARGUMENT;
-    if (epilogue == EPI_SWIGLU) return launch_resident<EPI_SWIGLU>(x, w, out, M, N, K, ldw, ldo, N, stream);
-    if (epilogue == EPI_F32) return launch_resident<EPI_F32>(x, w, out, M, N, K, ldw, ldo, 0, stream);
-    return launch_resident<EPI_BF16>(x, w, out, M, N, K, ldw, ldo, 0, stream);
+    if (epilogue == EPI_SWIGLU) return launch_resident<EPI_SWIGLU>(x, w, out, M, N, K, ldw, ldo, N, act, stream);
+    if (epilogue == EPI_F32) return launch_resident<EPI_F32>(x, w, out, M, N, K, ldw, ldo, 0, act, stream);
+    return launch_resident<EPI_BF16>(x, w, out, M, N, K, ldw, ldo, 0, act, stream);
   }
   if (tiles == 0) {
     // measured on MI355X: up to 16 rows of x one tile per wave is fastest at every width; with more
@@ -396,7 +399,7 @@ extern "C" int fe_gemm_skinny(const void* x, const void* w, void* out, int M, in
   }
   if (waves != 4 && waves != 8 && waves != 16) return FE_BAD_ARGUMENT;
   if (waves == 16 && !shape_fits(mt, tiles * (epilogue == EPI_SWIGLU ? 2 : 1), 16)) waves = 8;
-  const SkinnyCall call = {x, w, out, M, N, K, ldw, ldo, epilogue == EPI_SWIGLU ? N : 0, splits, part_stride, stream};
+  const SkinnyCall call = {x, w, out, M, N, K, ldw, ldo, epilogue == EPI_SWIGLU ? N : 0, splits, part_stride, act, stream};
   if (epilogue == EPI_SWIGLU) return dispatch<EPI_SWIGLU>(mt, tiles, waves, call);
   if (epilogue == EPI_F32) return dispatch<EPI_F32>(mt, tiles, waves, call);
   return dispatch<EPI_BF16>(mt, tiles, waves, call);

@@ -1,13 +1,13 @@
 // bfloat16 matrix products for steps that hold dozens to thousands of rows (portions of prompts,
 // whole prompts, large decode batches), with the ending fused:
-//   gated:  out[M, I] = silu(x Wg^T) * (x Wu^T)   for a fused gate/up weight [2 I, K], gate rows first
+//   gated:  out[M, I] = act(x Wg^T) * (x Wu^T)   for a fused gate/up weight [2 I, K], gate rows first
 //
 // A block keeps a tile of rows of x, 64 elements of K at a time, in LDS, several steps deep; the
 // tile goes there by `global_load_lds_dwordx4` (no staging registers, no LDS stores) and is shared
 // by the block's waves.  The weight goes from memory straight into MFMA operand registers, several
 // steps ahead.  A wave owns 16 * MT rows of the tile and, of the output, 16 * NG columns: their
 // gate rows and their up rows, so that 16 * MT x 32 * NG accumulators stay in registers for the
-// whole of K and silu(gate) * up is formed from them lane by lane, without a trip through memory
+// whole of K and act(gate) * up is formed from them lane by lane, without a trip through memory
 // for the 2 I wide intermediate.  An A fragment read from LDS feeds 2 NG MFMAs, a B fragment from
 // memory MT of them.  The block is RW x CW waves: RW take different rows, CW different columns.
 //
@@ -26,6 +26,7 @@
 //   and receives D[m = 4*(l / 16) + i][n = l % 16]: four neighbouring output columns of one row
 //   of x, which leave as one 8-byte store.
 #include "common.h"
+#include "gate_act.h"
 #include <algorithm>
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
@@ -74,7 +75,6 @@ __device__ __forceinline__ void global_arrived(uintx4* v) {
                  : "n"(PENDING));
 }
 
-__device__ __forceinline__ float silu_times(float g, float u) { return g / (1.f + __expf(-g)) * u; }
 
 // LDS holds a step of x as [row][8 chunks of 16 bytes], chunk c of row r at position c ^ (r % 8):
 // the lanes that a 16-byte read serves in one cycle then hit different bank groups.  A wave's load
@@ -87,7 +87,7 @@ template <int MT, int NG, int RW, int CW, int STAGES, int R, int D>
 __device__ __forceinline__ void gated_tile(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf16_t* __restrict__ out, int M, int N,
     int K, long long ldw, long long ldo, long long up_offset, int block_id, int col_blocks, int row_tiles,
-    int first_col) {
+    int first_col, GateAct act) {
   constexpr int THREADS = 64 * RW * CW;
   constexpr int ROWS = MT * 16 * RW;                 // rows of x a block holds
   constexpr int NF = 2 * NG;                         // weight operands a wave holds: NG gate tiles, then their NG up tiles
@@ -266,7 +266,7 @@ __device__ __forceinline__ void gated_tile(
       if (m >= M) continue;
       bf16_t y[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) y[i] = float_to_bf16(silu_times(acc[g][mt][i], acc[NG + g][mt][i]));
+      for (int i = 0; i < 4; ++i) y[i] = float_to_bf16(gate_times(acc[g][mt][i], acc[NG + g][mt][i], act));
       bf16_t* to = out + (size_t)m * ldo + col;
       if (col + 3 < N && (ldo & 3) == 0 && ((uintptr_t)out & 7) == 0) {
         uint2 packed;
@@ -285,8 +285,8 @@ __device__ __forceinline__ void gated_tile(
 template <int MT, int NG, int RW, int CW, int STAGES, int R, int D>
 __global__ __launch_bounds__(64 * RW * CW, 1) void gemm_gated_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf16_t* __restrict__ out, int M, int N,
-    int K, long long ldw, long long ldo, long long up_offset, int col_blocks, int row_tiles) {
-  gated_tile<MT, NG, RW, CW, STAGES, R, D>(x, w, out, M, N, K, ldw, ldo, up_offset, blockIdx.x, col_blocks, row_tiles, 0);
+    int K, long long ldw, long long ldo, long long up_offset, int col_blocks, int row_tiles, GateAct act) {
+  gated_tile<MT, NG, RW, CW, STAGES, R, D>(x, w, out, M, N, K, ldw, ldo, up_offset, blockIdx.x, col_blocks, row_tiles, 0, act);
 }
 
 // Tiles of 256 x 128 for as many columns as fill whole rounds of one block a CU, tiles of 256 x 64 for
@@ -296,12 +296,12 @@ __global__ __launch_bounds__(64 * RW * CW, 1) void gemm_gated_kernel(
 __global__ __launch_bounds__(256, 1) void gemm_gated_mixed_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf16_t* __restrict__ out, int M, int N,
     int K, long long ldw, long long ldo, long long up_offset, int wide_blocks, int wide_col_blocks,
-    int narrow_col_blocks, int row_tiles) {
+    int narrow_col_blocks, int row_tiles, GateAct act) {
   if ((int)blockIdx.x < wide_blocks)
-    gated_tile<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, up_offset, blockIdx.x, wide_col_blocks, row_tiles, 0);
+    gated_tile<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, up_offset, blockIdx.x, wide_col_blocks, row_tiles, 0, act);
   else
     gated_tile<16, 1, 1, 4, 4, 4, 8>(x, w, out, M, N, K, ldw, ldo, up_offset, blockIdx.x - wide_blocks, narrow_col_blocks,
-                                     row_tiles, wide_col_blocks * 128);
+                                     row_tiles, wide_col_blocks * 128, act);
 }
 
 // The kernels' loads are waited for by hand, on registers that the compiler must leave alone
@@ -322,7 +322,7 @@ static int fit_to_launch(const void* kernel, size_t lds_bytes, int* checked) {
 
 template <int MT, int NG, int RW, int CW, int STAGES, int R, int D>
 static int launch_gated(const void* x, const void* w, void* out, int M, int N, int K, long long ldw, long long ldo,
-                        hipStream_t stream) {
+                        GateAct act, hipStream_t stream) {
   constexpr int rows = MT * 16 * RW;
   constexpr size_t lds_bytes = (size_t)STAGES * rows * 128;
   static_assert(lds_bytes <= 160 * 1024, "LDS of a CU");
@@ -335,7 +335,7 @@ static int launch_gated(const void* x, const void* w, void* out, int M, int N, i
   const long long blocks = (long long)((col_blocks + 7) / 8) * 8 * row_tiles;
   if (blocks > 0x7fffffffLL) return FE_BAD_ARGUMENT;
   kernel<<<(unsigned)blocks, 64 * RW * CW, lds_bytes, stream>>>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)out, M, N, K,
-                                                               ldw, ldo, (long long)N * ldw, col_blocks, row_tiles);
+                                                               ldw, ldo, (long long)N * ldw, col_blocks, row_tiles, act);
   return fe_check_launch();
 }
 
@@ -343,7 +343,7 @@ static int launch_gated(const void* x, const void* w, void* out, int M, int N, i
 // Wide tiles alone, or wide tiles for whole rounds and narrow ones for the rest, whichever takes fewer
 // rounds (a round of narrow tiles counted as two thirds of a round of wide ones: measured).
 static int launch_gated_rounds(const void* x, const void* w, void* out, int M, int N, int K, long long ldw, long long ldo,
-                               hipStream_t stream) {
+                               GateAct act, hipStream_t stream) {
   const int row_tiles = (M + 255) / 256;
   const int all_wide = (N + 127) / 128;
   const long long tiles = (long long)row_tiles * all_wide;
@@ -353,7 +353,7 @@ static int launch_gated_rounds(const void* x, const void* w, void* out, int M, i
   const double mixed = (double)(((long long)wide_cols * row_tiles + FE_CUS - 1) / FE_CUS) +
                        0.67 * (double)(((long long)narrow_cols * row_tiles + FE_CUS - 1) / FE_CUS);
   if (wide_cols == 0 || narrow_cols <= 0 || mixed >= plain)
-    return launch_gated<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, stream);
+    return launch_gated<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, act, stream);
   constexpr size_t lds_bytes = (size_t)4 * 256 * 128;
   static int checked = 0;
   const int fit = fit_to_launch((const void*)gemm_gated_mixed_kernel, lds_bytes, &checked);
@@ -363,12 +363,13 @@ static int launch_gated_rounds(const void* x, const void* w, void* out, int M, i
   if (wide_blocks + narrow_blocks > 0x7fffffffLL) return FE_BAD_ARGUMENT;
   gemm_gated_mixed_kernel<<<(unsigned)(wide_blocks + narrow_blocks), 256, lds_bytes, stream>>>(
       (const bf16_t*)x, (const bf16_t*)w, (bf16_t*)out, M, N, K, ldw, ldo, (long long)N * ldw, (int)wide_blocks, wide_cols,
-      narrow_cols, row_tiles);
+      narrow_cols, row_tiles, act);
   return fe_check_launch();
 }
 
 // x [M, K] bf16 contiguous, K a multiple of 64; w [2 N, K] bf16 with row stride ldw (a multiple of 8),
-// gate rows first; out [M, N] bf16 with row stride ldo: out = silu(x gate^T) * (x up^T), float32 sums.
+// gate rows first; out [M, N] bf16 with row stride ldo: out = act(x gate^T) * (x up^T), float32 sums, act by
+// `activation` (gate_act.h).
 // shape: which tile a block of four waves takes (rows of x x output columns):
 //   0: 256 x 64, waves of 256 rows x 16 columns     1: 256 x 128, waves of 256 rows x 32 columns
 //   2: 128 x 64, waves of 128 rows x 16 columns
@@ -377,16 +378,18 @@ static int launch_gated_rounds(const void* x, const void* w, void* out, int M, i
 // FE_BAD_ARGUMENT also if the library was built with registers spilled to scratch memory (see
 // launch_gated): the kernel then never runs.
 extern "C" int fe_gemm_gated(const void* x, const void* w, void* out, int M, int N, int K, long long ldw, long long ldo,
-                             int shape, hipStream_t stream) {
+                             int shape, int activation, hipStream_t stream) {
   if (M < 1) return FE_OK;
+  GateAct act;
+  if (!gate_act(activation, &act)) return FE_BAD_ARGUMENT;
   if (N < 1 || K < KSTEP || K % KSTEP || ldw < K || ldw % 8 || ldo < N) return FE_BAD_ARGUMENT;
   if ((((uintptr_t)x) & 15) || (((uintptr_t)w) & 15)) return FE_BAD_ARGUMENT;
   if ((long long)M * K >= (1LL << 32) || 2LL * N * ldw >= (1LL << 32)) return FE_BAD_ARGUMENT;   // 32-bit element offsets inside
   switch (shape) {
-    case 0: return launch_gated<16, 1, 1, 4, 4, 4, 8>(x, w, out, M, N, K, ldw, ldo, stream);
-    case 1: return launch_gated<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, stream);
-    case 2: return launch_gated<8, 1, 1, 4, 6, 4, 8>(x, w, out, M, N, K, ldw, ldo, stream);
-    case 3: return launch_gated_rounds(x, w, out, M, N, K, ldw, ldo, stream);
+    case 0: return launch_gated<16, 1, 1, 4, 4, 4, 8>(x, w, out, M, N, K, ldw, ldo, act, stream);
+    case 1: return launch_gated<16, 2, 1, 4, 4, 3, 4>(x, w, out, M, N, K, ldw, ldo, act, stream);
+    case 2: return launch_gated<8, 1, 1, 4, 6, 4, 8>(x, w, out, M, N, K, ldw, ldo, act, stream);
+    case 3: return launch_gated_rounds(x, w, out, M, N, K, ldw, ldo, act, stream);
   }
   return FE_BAD_ARGUMENT;
 }

@@ -2,7 +2,7 @@
 // one that holds a portion of a prompt):
 //   out[M, N] = x[M, K] * W[N, K]^T
 // with one of three endings: float32 partial sums over parts of K ([parts][M, N]; the consumer, the
-// next norm, adds them in order), bfloat16, or silu(gate) * up as bfloat16 for a fused gate/up
+// next norm, adds them in order), bfloat16, or act(gate) * up as bfloat16 for a fused gate/up
 // weight.  At these row counts the product is bound by the weight's bytes and by how the rows of x
 // reach the matrix cores, not by arithmetic: the matrix library, tuned for large products, takes
 // three to four times the time the bytes need.
@@ -23,6 +23,7 @@
 //   lane l supplies A[m = l % 16][k = 8*(l / 16) .. +8], B[k = 8*(l / 16) .. +8][n = l % 16]
 //   and receives D[m = 4*(l / 16) + i][n = l % 16].
 #include "common.h"
+#include "gate_act.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float floatx4;
@@ -35,7 +36,6 @@ typedef __attribute__((ext_vector_type(4))) unsigned int uintx4;
 #define EPI_SWIGLU 2
 #define EPI_SWIGLU_HALF 3     // a wave's 16 weight rows are 8 gate rows and the 8 up rows that belong to them
 
-__device__ __forceinline__ float silu_times(float g, float u) { return g / (1.f + __expf(-g)) * u; }
 
 // 16 bytes from LDS byte address `at` + 2048 * STEP (sixteen rows of a stage further); nothing waits for them here
 template <int STEP>
@@ -68,7 +68,7 @@ __device__ __forceinline__ void lds_arrived(uintx4& v) {
 template <int MT, int EPI, int R, int WPB>
 __global__ __launch_bounds__(64 * WPB, 2) void gemm_wide_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, void* __restrict__ out, int M, int N,
-    int K, long long ldw, long long ldo, int steps_per_part, long long part_stride, long long up_offset) {
+    int K, long long ldw, long long ldo, int steps_per_part, long long part_stride, long long up_offset, GateAct act) {
   constexpr int WF = EPI == EPI_SWIGLU ? 2 : 1;     // weight operands a wave holds: a gate tile and an up tile, or one
   constexpr int THREADS = 64 * WPB;
   constexpr int PIECES = MT * 128;                  // 16-byte pieces of a step of x
@@ -222,9 +222,9 @@ __global__ __launch_bounds__(64 * WPB, 2) void gemm_wide_kernel(
         else if (EPI == EPI_SWIGLU_HALF) {
           // the lane 8 further in its row of 16 holds the up projection of this lane's column (and the other way round)
           const float other = __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(acc[0][mt][i]), 0x128, 0xF, 0xF, true));
-          if (lr < 8 && m < M) ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(silu_times(acc[0][mt][i], other));
+          if (lr < 8 && m < M) ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(gate_times(acc[0][mt][i], other, act));
         }
-        else ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(silu_times(acc[0][mt][i], acc[WF - 1][mt][i]));
+        else ((bf16_t*)out)[(size_t)m * ldo + n] = float_to_bf16(gate_times(acc[0][mt][i], acc[WF - 1][mt][i], act));
       }
   }
 }
@@ -235,7 +235,7 @@ __global__ __launch_bounds__(64 * WPB, 2) void gemm_wide_kernel(
 //   has no steps), so the caller may add all of them up.
 // ending 1: out is bfloat16 [M, N] with row stride ldo; parts must be 1.
 // ending 2: w is a fused gate/up weight [2 N, K], gate rows first; out is bfloat16 [M, N] =
-//   silu(x gate^T) * (x up^T); parts must be 1.  A wave multiplies 16 gate rows and their 16 up rows.
+//   act(x gate^T) * (x up^T), act by `activation` (gate_act.h); parts must be 1.  A wave multiplies 16 gate rows and their 16 up rows.
 // ending 3: the same result with 8 gate rows and their 8 up rows a wave (one weight operand, the two halves
 //   of a result tile meet by a lane exchange), so that a block takes 8 columns a wave: block_rows = 32 to 64
 //   in steps of 8 (four to eight waves) is then the block's columns, chosen so that the blocks fill rounds of
@@ -247,8 +247,10 @@ __global__ __launch_bounds__(64 * WPB, 2) void gemm_wide_kernel(
 // waves, plain endings) halves how often x is read.
 extern "C" int fe_gemm_wide(const void* x, const void* w, void* out, int M, int N, int K, long long ldw,
                             long long ldo, int ending, int parts, long long part_stride, int row_tile,
-                            int block_rows, hipStream_t stream) {
+                            int block_rows, int activation, hipStream_t stream) {
   if (M < 1) return FE_OK;
+  GateAct act;
+  if (!gate_act(activation, &act)) return FE_BAD_ARGUMENT;
   if (N < 1 || K < WSTEP || K % WSTEP || ldw < K || ldw % 8 || ldo < N) return FE_BAD_ARGUMENT;
   if ((((uintptr_t)x) & 15) || (((uintptr_t)w) & 15)) return FE_BAD_ARGUMENT;
   if (ending < EPI_PARTS || ending > EPI_SWIGLU_HALF) return FE_BAD_ARGUMENT;
@@ -266,7 +268,7 @@ extern "C" int fe_gemm_wide(const void* x, const void* w, void* out, int M, int 
   const long long up_offset = (long long)N * ldw;
 #define FE_LAUNCH(MT, EPI, WPB)                                                                                  \
   gemm_wide_kernel<MT, EPI, 4, WPB><<<grid, 64 * WPB, 0, stream>>>((const bf16_t*)x, (const bf16_t*)w, out, M, N, K, \
-                                                                    ldw, ldo, per_part, part_stride, up_offset)
+                                                                    ldw, ldo, per_part, part_stride, up_offset, act)
 #define FE_GO(MT, EPI)                                  \
   do {                                                  \
     if (block_rows == 128) FE_LAUNCH(MT, EPI, 8);       \

@@ -10,7 +10,7 @@
 // serves chosen rows only.  Without `out` the kernel only applies the update.
 //
 // fe_embed_token_pairs: a token's row of the embedding table plus a row of a second table chosen
-// by the token and the one before it; fe_scale_rows: a factor on every element.
+// by the token and the one before it; fe_scale_rows: a factor on every element; fe_cap_rows: a soft cap on every element.
 #include "common.h"
 
 #define MAX_STREAMS 8
@@ -242,5 +242,18 @@ __global__ void scale_kernel(float* __restrict__ x, float factor, long long coun
 extern "C" int fe_scale_rows(float* x, float factor, long long count, hipStream_t stream) {
   if (count <= 0) return FE_OK;
   scale_kernel<<<(int)((count + 255) / 256), 256, 0, stream>>>(x, factor, count);
+  return fe_check_launch();
+}
+
+// x <- cap * tanh(x * factor / cap), in place
+__global__ __launch_bounds__(256) void cap_kernel(float* x, float factor, float cap, long long count) {
+  const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (i < count) x[i] = cap * tanhf(x[i] * factor / cap);
+}
+
+extern "C" int fe_cap_rows(float* x, float factor, float cap, long long count, hipStream_t stream) {
+  if (count <= 0) return FE_OK;
+  if (!(cap > 0.f)) return FE_BAD_ARGUMENT;
+  cap_kernel<<<(int)((count + 255) / 256), 256, 0, stream>>>(x, factor, cap, count);
   return fe_check_launch();
 }

@@ -2,6 +2,7 @@
 // The residual stream is float32 in every mode; activations handed to matrix
 // products are float32 or bfloat16.
 #include "common.h"
+#include "gate_act.h"
 
 // ---------------------------------------------------------------- embedding
 // out[t, :] = float(table[ids[t], :]) * scale.  One block per token.
@@ -33,12 +34,49 @@ extern "C" int fe_embed_rows(const int* ids, const void* table, int table_dtype,
   return fe_check_launch();
 }
 
+// The same with a norm behind it: e = float(table[ids[t], :]) * scale, out[t, :] = e * rsqrt(mean(e^2) + eps) * w.
+template <typename TW>
+__global__ __launch_bounds__(256) void embed_rows_norm_kernel(const int* __restrict__ ids, const TW* __restrict__ table,
+                                                              const float* __restrict__ w, float* __restrict__ out, int hidden,
+                                                              int vocab, float scale, float eps) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  const int id = ids[t];
+  float* dst = out + (size_t)t * hidden;
+  if (id < 0 || id >= vocab) {
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = __int_as_float(0x7fc00000);
+    return;
+  }
+  const TW* src = table + (size_t)id * hidden;
+  float sumsq = 0.f;
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+    const float v = load_as_float(src + i) * scale;
+    sumsq += v * v;
+  }
+  const float inv = rsqrtf(block_sum<true>(sumsq, scratch) / (float)hidden + eps);
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = load_as_float(src + i) * scale * inv * w[i];
+}
+
+extern "C" int fe_embed_rows_norm(const int* ids, const void* table, int table_dtype, const float* w, float* out, int tokens,
+                                  int hidden, int vocab, float scale, float eps, hipStream_t stream) {
+  if (tokens <= 0) return FE_OK;
+  if (hidden <= 0 || vocab <= 0 || !w || !(eps > 0.f)) return FE_BAD_ARGUMENT;
+  if (table_dtype == FE_F32)
+    embed_rows_norm_kernel<float><<<tokens, 256, 0, stream>>>(ids, (const float*)table, w, out, hidden, vocab, scale, eps);
+  else if (table_dtype == FE_BF16)
+    embed_rows_norm_kernel<bf16_t><<<tokens, 256, 0, stream>>>(ids, (const bf16_t*)table, w, out, hidden, vocab, scale, eps);
+  else
+    return FE_BAD_ARGUMENT;
+  return fe_check_launch();
+}
+
 // ------------------------------------------------------- add + RMSNorm
 // For output row r (source row s = rows ? rows[r] : r):
-//   sum = h[s] + delta[s]          (float32; written back to h[s] if store_sum)
+//   sum = h[s] + delta[s] + other[s] + shift     (float32; written back to h[s] if store_sum)
 //   out[r] = sum * rsqrt(mean(sum^2) + eps) * w
 // delta may come in `parts` pieces `part_stride` elements apart (the partial sums of a product
-// whose K was split over blocks); they are added in order before anything else.
+// whose K was split over blocks); they are added in order before anything else.  other (float32, laid
+// out like h) and shift (float32, one number a channel) come on top; any of the three may be null.
 // Statistics, scaling and the weight product are float32; one rounding at the
 // store.  One block per row; the row is re-read from h/delta in the second
 // pass (it is cache-resident), so any width works.
@@ -50,8 +88,8 @@ __device__ __forceinline__ float delta_sum(const TD* p, int parts, size_t part_s
 }
 
 template <typename TD, typename TO>
-__global__ void add_rmsnorm_kernel(float* __restrict__ h, const TD* __restrict__ delta,
-                                   const float* __restrict__ w, TO* __restrict__ out,
+__global__ void add_rmsnorm_kernel(float* __restrict__ h, const TD* __restrict__ delta, const float* __restrict__ other,
+                                   const float* __restrict__ shift, const float* __restrict__ w, TO* __restrict__ out,
                                    const int* __restrict__ rows, int hidden, float eps,
                                    int store_sum, int parts, size_t part_stride) {
   __shared__ float scratch[16];
@@ -59,21 +97,25 @@ __global__ void add_rmsnorm_kernel(float* __restrict__ h, const TD* __restrict__
   const int s = rows ? rows[r] : r;
   float* hrow = h + (size_t)s * hidden;
   const TD* drow = delta ? delta + (size_t)s * hidden : nullptr;
+  const float* xrow = other ? other + (size_t)s * hidden : nullptr;
+  auto summed = [&](int i) {
+    float v = hrow[i];
+    if (drow) v += delta_sum(drow + i, parts, part_stride);
+    if (xrow) v += xrow[i];
+    if (shift) v += shift[i];
+    return v;
+  };
   float sumsq = 0.f;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-    float v = hrow[i];
-    if (drow) {
-      v += delta_sum(drow + i, parts, part_stride);
-      if (store_sum) hrow[i] = v;
-    }
+    const float v = summed(i);
+    if (store_sum) hrow[i] = v;
     sumsq += v * v;
   }
   const float total = block_sum<true>(sumsq, scratch);
   const float inv = rsqrtf(total / (float)hidden + eps);
   TO* orow = out + (size_t)r * hidden;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
-    float v = hrow[i];
-    if (drow && !store_sum) v += delta_sum(drow + i, parts, part_stride);
+    const float v = store_sum ? hrow[i] : summed(i);
     store_from_float(orow + i, v * inv * w[i]);
   }
 }
@@ -96,7 +138,8 @@ __device__ __forceinline__ void store4_from_float(bf16_t* p, float4 v) {
 
 template <typename TD, typename TO, int VEC, int THREADS>
 __global__ __launch_bounds__(THREADS) void add_rmsnorm_regs_kernel(
-    float* __restrict__ h, const TD* __restrict__ delta, const float* __restrict__ w,
+    float* __restrict__ h, const TD* __restrict__ delta, const float* __restrict__ other, const float* __restrict__ shift,
+    const float* __restrict__ w,
     TO* __restrict__ out, const int* __restrict__ rows, int hidden, float eps, int store_sum,
     int parts, size_t part_stride) {
   __shared__ float scratch[16];
@@ -126,8 +169,16 @@ __global__ __launch_bounds__(THREADS) void add_rmsnorm_regs_kernel(
             if (k + u < parts) { d.x += e[u].x; d.y += e[u].y; d.z += e[u].z; d.w += e[u].w; }
         }
         v[j].x += d.x; v[j].y += d.y; v[j].z += d.z; v[j].w += d.w;
-        if (store_sum) *(float4*)(hrow + i) = v[j];
       }
+      if (other) {
+        const float4 d = *(const float4*)(other + (size_t)s * hidden + i);
+        v[j].x += d.x; v[j].y += d.y; v[j].z += d.z; v[j].w += d.w;
+      }
+      if (shift) {
+        const float4 d = *(const float4*)(shift + i);
+        v[j].x += d.x; v[j].y += d.y; v[j].z += d.z; v[j].w += d.w;
+      }
+      if (store_sum) *(float4*)(hrow + i) = v[j];
       sumsq += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
     }
   }
@@ -144,100 +195,105 @@ __global__ __launch_bounds__(THREADS) void add_rmsnorm_regs_kernel(
 }
 
 template <typename TD, typename TO>
-static void launch_add_rmsnorm_typed(float* h, const TD* delta, const float* w, TO* out, const int* rows,
+static void launch_add_rmsnorm_typed(float* h, const TD* delta, const float* other, const float* shift, const float* w, TO* out, const int* rows,
                                      int n_rows, int hidden, float eps, int store_sum, int parts,
                                      size_t part_stride, hipStream_t stream) {
-  const bool aligned = hidden % 4 == 0 && part_stride % 4 == 0 && (((uintptr_t)h | (uintptr_t)delta | (uintptr_t)w | (uintptr_t)out) & 15) == 0;
+  const bool aligned = hidden % 4 == 0 && part_stride % 4 == 0 && (((uintptr_t)h | (uintptr_t)delta | (uintptr_t)other | (uintptr_t)shift | (uintptr_t)w | (uintptr_t)out) & 15) == 0;
   if (aligned && n_rows <= 512 && hidden > 1024 && hidden <= 4096)   // up to a few hundred rows: a whole row in flight at once
-    add_rmsnorm_regs_kernel<TD, TO, 1, 1024><<<n_rows, 1024, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_regs_kernel<TD, TO, 1, 1024><<<n_rows, 1024, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   else if (aligned && n_rows <= 512 && hidden > 4096 && hidden <= 8192)
-    add_rmsnorm_regs_kernel<TD, TO, 2, 1024><<<n_rows, 1024, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_regs_kernel<TD, TO, 2, 1024><<<n_rows, 1024, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   else if (aligned && hidden <= 1024)
-    add_rmsnorm_regs_kernel<TD, TO, 1, 256><<<n_rows, 256, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_regs_kernel<TD, TO, 1, 256><<<n_rows, 256, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   else if (aligned && hidden <= 4096)
-    add_rmsnorm_regs_kernel<TD, TO, 4, 256><<<n_rows, 256, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_regs_kernel<TD, TO, 4, 256><<<n_rows, 256, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   else if (aligned && hidden <= 8192)
-    add_rmsnorm_regs_kernel<TD, TO, 8, 256><<<n_rows, 256, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_regs_kernel<TD, TO, 8, 256><<<n_rows, 256, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   else {
     const int threads = hidden >= 2048 ? 512 : (hidden >= 512 ? 256 : 64);
-    add_rmsnorm_kernel<TD, TO><<<n_rows, threads, 0, stream>>>(h, delta, w, out, rows, hidden, eps, store_sum, parts, part_stride);
+    add_rmsnorm_kernel<TD, TO><<<n_rows, threads, 0, stream>>>(h, delta, other, shift, w, out, rows, hidden, eps, store_sum, parts, part_stride);
   }
 }
 
 template <typename TD>
-static int launch_add_rmsnorm(float* h, const TD* delta, const float* w, void* out, int out_dtype,
+static int launch_add_rmsnorm(float* h, const TD* delta, const float* other, const float* shift, const float* w, void* out, int out_dtype,
                               const int* rows, int n_rows, int hidden, float eps, int store_sum,
                               int parts, size_t part_stride, hipStream_t stream) {
   if (out_dtype == FE_F32)
-    launch_add_rmsnorm_typed<TD, float>(h, delta, w, (float*)out, rows, n_rows, hidden, eps, store_sum, parts, part_stride, stream);
+    launch_add_rmsnorm_typed<TD, float>(h, delta, other, shift, w, (float*)out, rows, n_rows, hidden, eps, store_sum, parts, part_stride, stream);
   else if (out_dtype == FE_BF16)
-    launch_add_rmsnorm_typed<TD, bf16_t>(h, delta, w, (bf16_t*)out, rows, n_rows, hidden, eps, store_sum, parts, part_stride, stream);
+    launch_add_rmsnorm_typed<TD, bf16_t>(h, delta, other, shift, w, (bf16_t*)out, rows, n_rows, hidden, eps, store_sum, parts, part_stride, stream);
   else
     return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }
 
-// delta may be null (plain RMSNorm).  rows may be null (all n_rows rows in order).
+// delta, other and shift may be null (all three: plain RMSNorm).  rows may be null (all n_rows rows in order).
 // With rows given, store_sum must be 0 unless the rows are distinct.  delta_parts >= 1 pieces of
 // delta lie part_stride elements apart.
-extern "C" int fe_add_rmsnorm(float* h, const void* delta, int delta_dtype, const float* w,
+extern "C" int fe_add_rmsnorm(float* h, const void* delta, int delta_dtype, const float* other, const float* shift, const float* w,
                               void* out, int out_dtype, const int* rows, int n_rows, int hidden,
                               float eps, int store_sum, int delta_parts, long long part_stride,
                               hipStream_t stream) {
   if (n_rows <= 0) return FE_OK;
   if (hidden <= 0 || !(eps > 0.f) || delta_parts < 1 || delta_parts > 64 || part_stride < 0) return FE_BAD_ARGUMENT;
   if (delta == nullptr || delta_dtype == FE_F32)
-    return launch_add_rmsnorm<float>(h, (const float*)delta, w, out, out_dtype, rows, n_rows, hidden, eps, store_sum, delta_parts, (size_t)part_stride, stream);
+    return launch_add_rmsnorm<float>(h, (const float*)delta, other, shift, w, out, out_dtype, rows, n_rows, hidden, eps, store_sum, delta_parts, (size_t)part_stride, stream);
   if (delta_dtype == FE_BF16)
-    return launch_add_rmsnorm<bf16_t>(h, (const bf16_t*)delta, w, out, out_dtype, rows, n_rows, hidden, eps, store_sum, delta_parts, (size_t)part_stride, stream);
+    return launch_add_rmsnorm<bf16_t>(h, (const bf16_t*)delta, other, shift, w, out, out_dtype, rows, n_rows, hidden, eps, store_sum, delta_parts, (size_t)part_stride, stream);
   return FE_BAD_ARGUMENT;
 }
 
-// h[t] += delta[t] for all rows (flushes a pending update without a norm); delta in `parts`
-// pieces `part_stride` elements apart, added in order.
+// h[t] += delta[t] + other[t] + shift for all rows (flushes what is pending without a norm; any of the three
+// may be null); delta in `parts` pieces `part_stride` elements apart, added in order.
 template <typename TD>
-__global__ void add_rows_kernel(float* __restrict__ h, const TD* __restrict__ delta, size_t count, int parts,
-                                size_t part_stride) {
-  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x)
-    h[i] += delta_sum(delta + i, parts, part_stride);
+__global__ void add_rows_kernel(float* __restrict__ h, const TD* __restrict__ delta, const float* __restrict__ other,
+                                const float* __restrict__ shift, size_t count, int hidden, int parts, size_t part_stride) {
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x) {
+    float v = h[i];
+    if (delta) v += delta_sum(delta + i, parts, part_stride);
+    if (other) v += other[i];
+    if (shift) v += shift[i % hidden];
+    h[i] = v;
+  }
 }
 
-extern "C" int fe_add_rows(float* h, const void* delta, int delta_dtype, long long count, int delta_parts,
-                           long long part_stride, hipStream_t stream) {
+extern "C" int fe_add_rows(float* h, const void* delta, int delta_dtype, const float* other, const float* shift, long long count,
+                           int hidden, int delta_parts, long long part_stride, hipStream_t stream) {
   if (count <= 0) return FE_OK;
-  if (delta_parts < 1 || delta_parts > 64 || part_stride < 0) return FE_BAD_ARGUMENT;
+  if (hidden <= 0 || delta_parts < 1 || delta_parts > 64 || part_stride < 0) return FE_BAD_ARGUMENT;
   const int threads = 256;
   long long want = (count + threads - 1) / threads;
   const int blocks = (int)(want < 4096 ? want : 4096);
   if (delta_dtype == FE_F32)
-    add_rows_kernel<float><<<blocks, threads, 0, stream>>>(h, (const float*)delta, (size_t)count, delta_parts, (size_t)part_stride);
+    add_rows_kernel<float><<<blocks, threads, 0, stream>>>(h, (const float*)delta, other, shift, (size_t)count, hidden, delta_parts, (size_t)part_stride);
   else if (delta_dtype == FE_BF16)
-    add_rows_kernel<bf16_t><<<blocks, threads, 0, stream>>>(h, (const bf16_t*)delta, (size_t)count, delta_parts, (size_t)part_stride);
+    add_rows_kernel<bf16_t><<<blocks, threads, 0, stream>>>(h, (const bf16_t*)delta, other, shift, (size_t)count, hidden, delta_parts, (size_t)part_stride);
   else
     return FE_BAD_ARGUMENT;
   return fe_check_launch();
 }
 
-// ---------------------------------------------------------------- SwiGLU
+// ---------------------------------------------------------------- gated activations (SwiGLU and its like)
 // gate_up is [T, 2*inter] with gate in the first half of each row:
-//   out[t, i] = silu(gate[t, i]) * up[t, i],  silu(z) = z / (1 + exp(-z)),  in float32.
+//   out[t, i] = act(gate[t, i]) * up[t, i],  act by gate_act.h (silu(z) = z / (1 + exp(-z)), or gelu's tanh form),  in float32.
 template <typename T>
 __global__ void swiglu_kernel(const T* __restrict__ gate_up, size_t in_stride, T* __restrict__ out, size_t out_stride, int inter,
-                              size_t total) {
+                              size_t total, GateAct act) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / inter;
     const int c = (int)(i - t * inter);
     const T* row = gate_up + t * in_stride;
     const float g = load_as_float(row + c);
     const float u = load_as_float(row + inter + c);
-    store_from_float(out + t * out_stride + c, g / (1.f + expf(-g)) * u);
+    store_from_float(out + t * out_stride + c, gate_times_exact(g, u, act));
   }
 }
 
 // bfloat16 rows whose width is a multiple of 8: eight elements (16 bytes) of gate and of up per thread.
 __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __restrict__ gate_up, size_t in_stride8,
                                                             bf16_t* __restrict__ out, size_t out_stride8, int inter8,
-                                                            size_t total8) {
+                                                            size_t total8, GateAct act) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total8; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / inter8;
     const int c = (int)(i - t * inter8);
@@ -250,8 +306,8 @@ __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __rest
     for (int k = 0; k < 4; ++k) {
       const float g0 = __uint_as_float(gw[k] << 16), g1 = __uint_as_float(gw[k] & 0xffff0000u);
       const float u0 = __uint_as_float(uw[k] << 16), u1 = __uint_as_float(uw[k] & 0xffff0000u);
-      ow[k] = (uint32_t)float_to_bf16(g0 / (1.f + expf(-g0)) * u0) |
-              ((uint32_t)float_to_bf16(g1 / (1.f + expf(-g1)) * u1) << 16);
+      ow[k] = (uint32_t)float_to_bf16(gate_times_exact(g0, u0, act)) |
+              ((uint32_t)float_to_bf16(gate_times_exact(g1, u1, act)) << 16);
     }
     ((uint4*)out)[t * out_stride8 + c] = make_uint4(ow[0], ow[1], ow[2], ow[3]);
   }
@@ -259,8 +315,10 @@ __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __rest
 
 // rows of gate_up (gate, then up) lie in_stride elements apart, rows of out out_stride
 extern "C" int fe_swiglu(const void* gate_up, long long in_stride, void* out, long long out_stride, int dtype, int tokens,
-                         int inter, hipStream_t stream) {
+                         int inter, int activation, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
+  GateAct act;
+  if (!gate_act(activation, &act)) return FE_BAD_ARGUMENT;
   if (inter <= 0 || in_stride < 2LL * inter || out_stride < inter) return FE_BAD_ARGUMENT;
   const size_t total = (size_t)tokens * inter;
   const int threads = 256;
@@ -269,15 +327,15 @@ extern "C" int fe_swiglu(const void* gate_up, long long in_stride, void* out, lo
     const size_t total8 = total / 8;
     const size_t want8 = (total8 + threads - 1) / threads;
     swiglu_bf16x8_kernel<<<(int)(want8 < 16384 ? want8 : 16384), threads, 0, stream>>>(
-        (const bf16_t*)gate_up, (size_t)in_stride / 8, (bf16_t*)out, (size_t)out_stride / 8, inter / 8, total8);
+        (const bf16_t*)gate_up, (size_t)in_stride / 8, (bf16_t*)out, (size_t)out_stride / 8, inter / 8, total8, act);
     return fe_check_launch();
   }
   size_t want = (total + threads - 1) / threads;
   const int blocks = (int)(want < 8192 ? want : 8192);
   if (dtype == FE_F32)
-    swiglu_kernel<float><<<blocks, threads, 0, stream>>>((const float*)gate_up, (size_t)in_stride, (float*)out, (size_t)out_stride, inter, total);
+    swiglu_kernel<float><<<blocks, threads, 0, stream>>>((const float*)gate_up, (size_t)in_stride, (float*)out, (size_t)out_stride, inter, total, act);
   else if (dtype == FE_BF16)
-    swiglu_kernel<bf16_t><<<blocks, threads, 0, stream>>>((const bf16_t*)gate_up, (size_t)in_stride, (bf16_t*)out, (size_t)out_stride, inter, total);
+    swiglu_kernel<bf16_t><<<blocks, threads, 0, stream>>>((const bf16_t*)gate_up, (size_t)in_stride, (bf16_t*)out, (size_t)out_stride, inter, total, act);
   else
     return FE_BAD_ARGUMENT;
   return fe_check_launch();

@@ -68,8 +68,10 @@ def _call(lib_name: str, fn_name: str, *args) -> None:
 
 # ------------------------------------------------------------------ row-wise
 
-def embed_rows(ids: Tensor, table: Tensor, out: Tensor, scale: float = 1.0) -> Tensor:
-    """out[t] = float32(table[ids[t]]) * scale; ids int32 [T], table [V, H], out float32 [T, H]."""
+def embed_rows(ids: Tensor, table: Tensor, out: Tensor, scale: float = 1.0, norm_weight: Tensor | None = None,
+               eps: float = 0.0) -> Tensor:
+    """out[t] = e = float32(table[ids[t]]) * scale; ids int32 [T], table [V, H], out float32 [T, H].  With ``norm_weight``
+    (float32 [H]): out[t] = e * rsqrt(mean(e^2) + eps) * norm_weight."""
     _gpu(ids, "ids", torch.int32)
     _gpu(table, "table")
     _gpu(out, "out", torch.float32)
@@ -77,16 +79,25 @@ def embed_rows(ids: Tensor, table: Tensor, out: Tensor, scale: float = 1.0) -> T
     vocab, hidden = table.shape
     if out.shape != (tokens, hidden):
         raise KernelError(f"out must be [{tokens}, {hidden}], got {tuple(out.shape)}")
+    if norm_weight is not None:
+        _gpu(norm_weight, "norm_weight", torch.float32)
+        if norm_weight.shape != (hidden,) or not eps > 0.0:
+            raise KernelError(f"norm_weight must be [{hidden}] and come with a positive eps")
+        _call("rowwise", "fe_embed_rows_norm", _ptr(ids), _ptr(table), c_int(_code(table.dtype)), _ptr(norm_weight), _ptr(out),
+              c_int(tokens), c_int(hidden), c_int(vocab), c_float(scale), c_float(eps), _stream())
+        return out
     _call("rowwise", "fe_embed_rows", _ptr(ids), _ptr(table), c_int(_code(table.dtype)), _ptr(out),
           c_int(tokens), c_int(hidden), c_int(vocab), c_float(scale), _stream())
     return out
 
 
 def add_rmsnorm(h: Tensor, delta: Tensor | None, weight: Tensor, eps: float, out: Tensor,
-                rows: Tensor | None = None, store_sum: bool = True) -> Tensor:
-    """sum = h[s] + delta[s] (float32, written back to h if store_sum);
+                rows: Tensor | None = None, store_sum: bool = True, other: Tensor | None = None,
+                shift: Tensor | None = None) -> Tensor:
+    """sum = h[s] + delta[s] + other[s] + shift (float32, written back to h if store_sum);
     out[r] = sum * rsqrt(mean(sum^2) + eps) * weight, s = rows[r] or r.
-    delta may be [parts, rows, hidden]: the parts are added up in order first."""
+    delta may be [parts, rows, hidden]: the parts are added up in order first.  other: float32 like h, shift: float32
+    [hidden]; any of the three may be None."""
     _gpu(h, "h", torch.float32)
     _gpu(weight, "weight", torch.float32)
     _gpu(out, "out")
@@ -101,17 +112,31 @@ def add_rmsnorm(h: Tensor, delta: Tensor | None, weight: Tensor, eps: float, out
     if rows is not None:
         _gpu(rows, "rows", torch.int32)
         n_rows = rows.numel()
-        if store_sum and delta is not None:
+        if store_sum and not (delta is None and other is None and shift is None):
             raise KernelError("store_sum with a row list is not allowed (rows may repeat)")
+    _stream_extras(h, other, shift)
     if out.shape != (n_rows, hidden):
         raise KernelError(f"out must be [{n_rows}, {hidden}], got {tuple(out.shape)}")
     if not eps > 0.0:
         raise KernelError("eps must be positive")
     _call("rowwise", "fe_add_rmsnorm", _ptr(h), _ptr(delta),
-          c_int(_code(delta.dtype) if delta is not None else FE_F32), _ptr(weight), _ptr(out),
+          c_int(_code(delta.dtype) if delta is not None else FE_F32), _ptr(other), _ptr(shift), _ptr(weight), _ptr(out),
           c_int(_code(out.dtype)), _ptr(rows), c_int(n_rows), c_int(hidden), c_float(eps),
-          c_int(1 if (store_sum and delta is not None) else 0), c_int(parts), c_longlong(h.numel()), _stream())
+          c_int(1 if store_sum and not (delta is None and other is None and shift is None) else 0), c_int(parts),
+          c_longlong(h.numel()), _stream())
     return out
+
+
+def _stream_extras(h: Tensor, other: Tensor | None, shift: Tensor | None) -> None:
+    """What may be added to the stream beside an update: another float32 tensor like it, and a number a channel."""
+    if other is not None:
+        _gpu(other, "other", torch.float32)
+        if other.shape != h.shape or other.data_ptr() == h.data_ptr():
+            raise KernelError(f"other must be a {tuple(h.shape)} tensor apart from the stream")
+    if shift is not None:
+        _gpu(shift, "shift", torch.float32)
+        if shift.shape != (h.shape[1],):
+            raise KernelError(f"shift must be [{h.shape[1]}]")
 
 
 def _delta_parts(h: Tensor, delta: Tensor) -> int:
@@ -122,25 +147,39 @@ def _delta_parts(h: Tensor, delta: Tensor) -> int:
     raise KernelError(f"delta must be {tuple(h.shape)} or [parts <= 64, {h.shape[0]}, {h.shape[1]}], got {tuple(delta.shape)}")
 
 
-def add_rows(h: Tensor, delta: Tensor) -> Tensor:
-    """h += delta, in float32; delta may be [parts, rows, hidden] (added up in order)."""
+def add_rows(h: Tensor, delta: Tensor | None, other: Tensor | None = None, shift: Tensor | None = None) -> Tensor:
+    """h += delta + other + shift, in float32; delta may be [parts, rows, hidden] (added up in order), other is like h,
+    shift [hidden]; any of the three may be None."""
     _gpu(h, "h", torch.float32)
-    _gpu(delta, "delta")
-    parts = _delta_parts(h, delta)
-    _call("rowwise", "fe_add_rows", _ptr(h), _ptr(delta), c_int(_code(delta.dtype)),
-          c_longlong(h.numel()), c_int(parts), c_longlong(h.numel()), _stream())
+    parts = 1
+    if delta is not None:
+        _gpu(delta, "delta")
+        parts = _delta_parts(h, delta)
+    _stream_extras(h, other, shift)
+    _call("rowwise", "fe_add_rows", _ptr(h), _ptr(delta), c_int(_code(delta.dtype) if delta is not None else FE_F32), _ptr(other),
+          _ptr(shift), c_longlong(h.numel()), c_int(h.shape[-1]), c_int(parts), c_longlong(h.numel()), _stream())
     return h
 
 
-def swiglu(gate_up: Tensor, out: Tensor) -> Tensor:
-    """out[t, i] = silu(gate_up[t, i]) * gate_up[t, I + i]; rows of any stride."""
+GATE_ACTS = {"silu": 0, "gelu_tanh": 1}     # FE_GATE_* of csrc/gate_act.h
+
+
+def _gate_act(act: str) -> c_int:
+    if act not in GATE_ACTS:
+        raise KernelError(f"unknown activation of a gate '{act}' (known: {', '.join(GATE_ACTS)})")
+    return c_int(GATE_ACTS[act])
+
+
+def swiglu(gate_up: Tensor, out: Tensor, act: str = "silu") -> Tensor:
+    """out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; rows of any stride.  ``act``: ``silu`` or ``gelu_tanh``
+    (0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))))."""
     tokens, two_inter = gate_up.shape
     in_stride = _strided_rows(gate_up, "gate_up", two_inter)
     if two_inter % 2 or out.shape != (tokens, two_inter // 2) or out.dtype != gate_up.dtype:
         raise KernelError(f"out must be [{tokens}, {two_inter // 2}] in gate_up's dtype, got {tuple(out.shape)}")
     out_stride = _strided_rows(out, "out", two_inter // 2)
     _call("rowwise", "fe_swiglu", _ptr(gate_up), c_longlong(in_stride), _ptr(out), c_longlong(out_stride), c_int(_code(out.dtype)),
-          c_int(tokens), c_int(two_inter // 2), _stream())
+          c_int(tokens), c_int(two_inter // 2), _gate_act(act), _stream())
     return out
 
 
@@ -198,11 +237,11 @@ def _skinny_fits(x: Tensor, weight: Tensor, rows: int = SKINNY_MAX_ROWS) -> bool
 
 
 def gemm_skinny(x: Tensor, weight: Tensor, epilogue: str = "bf16", tiles: int = 0, waves: int = 0,
-                splits: int = 1) -> Tensor:
+                splits: int = 1, act: str = "silu") -> Tensor:
     """y = x @ weight^T for up to 64 rows of bfloat16 x, float32 accumulation.
 
     epilogue ``f32``/``bf16``: y [M, N] in that dtype; ``swiglu``: weight is
-    [2I, K] with the gate rows first and y = silu(x Wg^T) * (x Wu^T) in bfloat16.
+    [2I, K] with the gate rows first and y = act(x Wg^T) * (x Wu^T) in bfloat16 (``act`` as in ``swiglu``).
     ``splits`` > 1 (``f32`` only): K is summed in that many parts by blocks of their own
     and the result is the parts [splits, M, N], to be added up by the consumer."""
     _gpu(x, "x", torch.bfloat16)
@@ -223,7 +262,7 @@ def gemm_skinny(x: Tensor, weight: Tensor, epilogue: str = "bf16", tiles: int = 
     out = torch.empty(shape, dtype=torch.float32 if code == _EPI_F32 else torch.bfloat16, device=x.device)
     _call("gemm_skinny", "fe_gemm_skinny", _ptr(x), _ptr(weight), _ptr(out), c_int(m), c_int(n), c_int(k),
           c_longlong(weight.stride(0)), c_longlong(n), c_int(code), c_int(tiles), c_int(waves), c_int(splits),
-          c_longlong(m * n), _stream())
+          c_longlong(m * n), _gate_act(act), _stream())
     return out
 
 
@@ -384,10 +423,10 @@ def _wide_fits(x: Tensor, weight: Tensor, most_rows: int, least_rows: int = MID_
 
 
 def gemm_wide(x: Tensor, weight: Tensor, ending: str = "bf16", parts: int = 1, row_tile: int = 0,
-              block_rows: int = 64) -> Tensor:
+              block_rows: int = 64, act: str = "silu") -> Tensor:
     """x @ weight^T for a few dozen to a few hundred bfloat16 rows: ``"parts"`` float32 partial sums
-    [parts, M, N] over runs of whole 64-steps of K, ``"bf16"`` [M, N], or ``"swiglu"``: silu(gate) * up
-    [M, N / 2] for a fused gate/up weight (gate rows first)."""
+    [parts, M, N] over runs of whole 64-steps of K, ``"bf16"`` [M, N], or ``"swiglu"``: act(gate) * up
+    [M, N / 2] for a fused gate/up weight (gate rows first; ``act`` as in ``swiglu``)."""
     _gpu(x, "x", torch.bfloat16)
     _gpu(weight, "weight", torch.bfloat16, contiguous=False)
     m, k = x.shape
@@ -405,7 +444,7 @@ def gemm_wide(x: Tensor, weight: Tensor, ending: str = "bf16", parts: int = 1, r
         raise KernelError(f"no ending {ending!r} with {parts} parts")
     _call("gemm_wide", "fe_gemm_wide", _ptr(x), _ptr(weight), _ptr(out), c_int(m), c_int(cols), c_int(k),
           c_longlong(weight.stride(0)), c_longlong(cols), c_int(code), c_int(parts), c_longlong(m * cols),
-          c_int(row_tile or (16 if m <= 16 else 64 if m <= 64 else 128)), c_int(block_rows), _stream())
+          c_int(row_tile or (16 if m <= 16 else 64 if m <= 64 else 128)), c_int(block_rows), _gate_act(act), _stream())
     return out
 
 
@@ -503,8 +542,8 @@ def linear_in_parts(x: Tensor, weight: Tensor) -> Tensor | None:
     return None
 
 
-def gemm_gated(x: Tensor, gate_up_weight: Tensor, shape: int = 0) -> Tensor:
-    """silu(x Wg^T) * (x Wu^T) for the fused weight [2I, K] (gate rows first) and any number of
+def gemm_gated(x: Tensor, gate_up_weight: Tensor, shape: int = 0, act: str = "silu") -> Tensor:
+    """act(x Wg^T) * (x Wu^T) (``act`` as in ``swiglu``) for the fused weight [2I, K] (gate rows first) and any number of
     bfloat16 rows: blocks keep a tile of rows of x in LDS and their accumulators in registers over
     the whole of K; the intermediate [M, 2I] never exists.  ``shape``: the block's tile, see
     ``fe_gemm_gated``."""
@@ -517,7 +556,7 @@ def gemm_gated(x: Tensor, gate_up_weight: Tensor, shape: int = 0) -> Tensor:
         raise KernelError("the gated product takes contiguous bfloat16 rows, K a multiple of 64, an even number of weight rows")
     out = torch.empty((m, rows // 2), dtype=torch.bfloat16, device=x.device)
     _call("gemm_tile", "fe_gemm_gated", _ptr(x), _ptr(gate_up_weight), _ptr(out), c_int(m), c_int(rows // 2), c_int(k),
-          c_longlong(gate_up_weight.stride(0)), c_longlong(rows // 2), c_int(shape), _stream())
+          c_longlong(gate_up_weight.stride(0)), c_longlong(rows // 2), c_int(shape), _gate_act(act), _stream())
     return out
 
 
@@ -541,8 +580,8 @@ GATED_TILE_MAX_ROWS = 4096
 GATED_TILE_MAX_K = 3072
 
 
-def linear_swiglu(x: Tensor, gate_up_weight: Tensor) -> Tensor:
-    """silu(x Wg^T) * (x Wu^T) for the fused weight [2I, K] (gate rows first)."""
+def linear_swiglu(x: Tensor, gate_up_weight: Tensor, act: str = "silu") -> Tensor:
+    """act(x Wg^T) * (x Wu^T) for the fused weight [2I, K] (gate rows first); ``act`` as in ``swiglu``."""
     _gpu(x, "x")
     _gpu(gate_up_weight, "gate_up_weight")
     rows = x.shape[0]
@@ -551,7 +590,7 @@ def linear_swiglu(x: Tensor, gate_up_weight: Tensor) -> Tensor:
             and gate_up_weight.dim() == 2 and gate_up_weight.stride(1) == 1 and gate_up_weight.stride(0) % 8 == 0
             and x.data_ptr() % 16 == 0 and gate_up_weight.data_ptr() % 16 == 0
             and gate_up_weight.shape[0] * gate_up_weight.stride(0) < 2 ** 32 and rows * x.shape[1] < 2 ** 32):
-        return gemm_gated(x, gate_up_weight, shape=3)
+        return gemm_gated(x, gate_up_weight, shape=3, act=act)
     to_library = (2 <= rows <= SKINNY_MAX_ROWS and gate_up_weight.shape[0] > GATE_LIBRARY_WEIGHT_ROWS
                   and x.dtype == torch.bfloat16 and gate_up_weight.dtype == torch.bfloat16)
     paired_fits = (rows <= MID_ROWS and x.dtype == torch.bfloat16 and gate_up_weight.dtype == torch.bfloat16
@@ -563,12 +602,12 @@ def linear_swiglu(x: Tensor, gate_up_weight: Tensor) -> Tensor:
         # matrix library with the gate kernel behind it: 24 against 28 us at 9728 columns of K = 2560, 46 against 50 at
         # 12288 of K = 4096; at K = 5120 the library wins (17408 columns: 85 against 82 us, 25600 columns: 111 against
         # 96), and from 96 rows on at every size.  Up to 16 rows: see FEW_ROWS above.
-        return gemm_wide(x, gate_up_weight, "swiglu_half", block_rows=_gate_block_columns(gate_up_weight.shape[0] // 2))
+        return gemm_wide(x, gate_up_weight, "swiglu_half", block_rows=_gate_block_columns(gate_up_weight.shape[0] // 2), act=act)
     if _skinny_fits(x, gate_up_weight) and not to_library:
-        return gemm_skinny(x, gate_up_weight, "swiglu")
+        return gemm_skinny(x, gate_up_weight, "swiglu", act=act)
     gate_up = torch.matmul(x, gate_up_weight.t()) if to_library else linear(x, gate_up_weight)
     out = torch.empty((x.shape[0], gate_up_weight.shape[0] // 2), dtype=gate_up.dtype, device=x.device)
-    return swiglu(gate_up, out)
+    return swiglu(gate_up, out, act)
 
 
 # ------------------------------------------------------------------ attention
@@ -1469,74 +1508,83 @@ MASKED_MAX_VALUE_DIM = 512
 
 # ------------------------------------------------- attention through a latent
 
-def latent_norm_rope_write(x: Tensor, q_weight: Tensor, kv_weight: Tensor | None, inv_freq: Tensor | None, positions: Tensor,
+def latent_norm_rope_write(x: Tensor, q_weight: Tensor | None, kv_weight: Tensor | None, inv_freq: Tensor | None, positions: Tensor,
                            token_seq: Tensor, block_table: Tensor | None, key_pages: Tensor | None, value_pages: Tensor | None,
-                           cq_out: Tensor, *, q_rank: int, kv_rank: int, rot_dim: int, rotary_dim: int, eps: float,
-                           write_kv: bool) -> Tensor:
-    """From a token's fused down-projections x = [a | b | r] (float32 [T, >= q_rank (+ kv_rank + rot_dim)], any
-    row stride): ``cq_out`` [T, q_rank] = a / rms(a) * q_weight, and with ``write_kv`` the token's cache row
-    [b / rms(b) * kv_weight | rotate(r)] into ``key_pages`` [blocks, 1, block_size, kv_rank + rot_dim] and, if the
-    cache keeps values (``value_pages`` [blocks, 1, kv_rank, block_size], transposed), its first kv_rank numbers
-    there as well.  The rotation turns the first ``rotary_dim`` dims of r, dim i with dim i + rotary_dim / 2, by
-    position * inv_freq[i].  Norms and angles float32 (epsilon inside the root), one rounding at the stores."""
-    _gpu(x, "x", torch.float32, contiguous=False)
-    _gpu(q_weight, "q_weight", torch.float32)
-    _gpu(cq_out, "cq_out")
+                           cq_out: Tensor | None, *, q_rank: int, kv_rank: int, rot_dim: int, rotary_dim: int, eps: float,
+                           write_kv: bool, interleaved: bool = False, magnitude: float = 1.0, latent_row: int | None = None) -> Tensor | None:
+    """From a token's fused down-projections x = [a | b | r] (float32 or the cache's dtype, [T, >= q_rank (+ kv_rank +
+    rot_dim)], any row stride): ``cq_out`` [T, q_rank] = a / rms(a) * q_weight (q_rank 0, no ``cq_out``: x is [b | r]), and
+    with ``write_kv`` the token's cache row [b / rms(b) * kv_weight | rotate(r)] into ``key_pages`` [blocks, 1, block_size,
+    row] and, if the cache keeps values (``value_pages`` [blocks, 1, latent_row, block_size], transposed), its first kv_rank
+    numbers there as well.  ``latent_row`` (default kv_rank): the latent part's width in a row, the rest being the rotated
+    part's; both are filled up with zeros.  The rotation turns the first ``rotary_dim`` dims of r by position *
+    inv_freq[i], cosines and sines times ``magnitude``: dim i with dim i + rotary_dim / 2, or (``interleaved``) dim 2i with
+    dim 2i + 1.  Norms and angles float32 (epsilon inside the root), one rounding at the stores."""
+    _gpu(x, "x", contiguous=False)
+    dtype = cq_out.dtype if cq_out is not None else (key_pages.dtype if key_pages is not None else x.dtype)
     tokens = x.shape[0]
     need = q_rank + (kv_rank + rot_dim if write_kv else 0)
-    if x.dim() != 2 or x.shape[1] < need or (x.shape[1] > 1 and x.stride(1) != 1):
-        raise KernelError(f"x must be [T, >= {need}] with unit inner stride, got {tuple(x.shape)}")
-    if q_weight.shape != (q_rank,) or cq_out.shape != (tokens, q_rank) or not eps > 0.0:
-        raise KernelError(f"q_weight must be [{q_rank}], cq_out [{tokens}, {q_rank}] and eps positive")
+    if x.dim() != 2 or x.shape[1] < need or (x.shape[1] > 1 and x.stride(1) != 1) or x.dtype not in (torch.float32, dtype):
+        raise KernelError(f"x must be [T, >= {need}] with unit inner stride, in float32 or {dtype}, got {tuple(x.shape)} {x.dtype}")
+    if not eps > 0.0 or (q_rank == 0) != (cq_out is None) or (q_rank == 0 and not write_kv):
+        raise KernelError("eps must be positive, and cq_out comes with a query bottleneck")
+    if q_rank:
+        _gpu(q_weight, "q_weight", torch.float32)
+        _gpu(cq_out, "cq_out")
+        if q_weight.shape != (q_rank,) or cq_out.shape != (tokens, q_rank):
+            raise KernelError(f"q_weight must be [{q_rank}] and cq_out [{tokens}, {q_rank}]")
     if rotary_dim % 2 or not 0 <= rotary_dim <= rot_dim:
         raise KernelError("rotary_dim must be even and at most rot_dim")
-    block_size = num_blocks = table_stride = 0
+    latent_row = kv_rank if latent_row is None else int(latent_row)
+    block_size = num_blocks = table_stride = row = 0
     if write_kv:
         _gpu(kv_weight, "kv_weight", torch.float32)
-        _gpu(key_pages, "key_pages", cq_out.dtype)
+        _gpu(key_pages, "key_pages", dtype)
         _gpu(block_table, "block_table", torch.int32)
         _gpu(positions, "positions", torch.int32)
         _gpu(token_seq, "token_seq", torch.int32)
         if kv_weight.shape != (kv_rank,) or positions.numel() != tokens or token_seq.numel() != tokens:
             raise KernelError(f"kv_weight must be [{kv_rank}], positions and token_seq hold one entry per token")
-        if key_pages.dim() != 4 or key_pages.shape[1] != 1 or key_pages.shape[3] != kv_rank + rot_dim:
-            raise KernelError(f"key pages must be [blocks, 1, block_size, {kv_rank + rot_dim}], got {tuple(key_pages.shape)}")
+        if key_pages.dim() != 4 or key_pages.shape[1] != 1 or latent_row < kv_rank or key_pages.shape[3] < latent_row + rot_dim:
+            raise KernelError(f"key pages must be [blocks, 1, block_size, >= {latent_row} + {rot_dim}], got {tuple(key_pages.shape)}")
         if block_table.dim() != 2 or block_table.stride(1) != 1:
             raise KernelError("block_table must be [sequences, max_blocks] with unit inner stride")
         if rotary_dim:
             _gpu(inv_freq, "inv_freq", torch.float32)
             if inv_freq.shape != (rotary_dim // 2,):
                 raise KernelError(f"inv_freq must be [{rotary_dim // 2}]")
-        num_blocks, _, block_size, _ = key_pages.shape
+        num_blocks, _, block_size, row = key_pages.shape
         table_stride = block_table.stride(0)
         if value_pages is not None:
-            _gpu(value_pages, "value_pages", cq_out.dtype)
-            if value_pages.shape != (num_blocks, 1, kv_rank, block_size):
-                raise KernelError(f"value pages are transposed: [blocks, 1, {kv_rank}, block_size], got {tuple(value_pages.shape)}")
+            _gpu(value_pages, "value_pages", dtype)
+            if value_pages.shape != (num_blocks, 1, latent_row, block_size):
+                raise KernelError(f"value pages are transposed: [blocks, 1, {latent_row}, block_size], got {tuple(value_pages.shape)}")
     stride = x.stride(0) if tokens > 1 else max(x.stride(0), x.shape[1])
-    _call("latent", "fe_latent_norm_rope_write", _ptr(x), c_longlong(stride), c_int(q_rank), c_int(kv_rank), c_int(rot_dim),
-          c_int(rotary_dim), _ptr(q_weight), _ptr(kv_weight if write_kv else None), _ptr(inv_freq if write_kv and rotary_dim else None),
-          _ptr(positions if write_kv else None), _ptr(token_seq if write_kv else None), _ptr(block_table if write_kv else None),
-          c_int(table_stride), _ptr(key_pages if write_kv else None), _ptr(value_pages if write_kv else None), _ptr(cq_out),
-          c_int(_code(cq_out.dtype)), c_float(eps),
-          c_int(tokens), c_int(block_size), c_int(num_blocks), c_int(1 if write_kv else 0), _stream())
+    _call("latent", "fe_latent_norm_rope_write", _ptr(x), c_int(_code(x.dtype)), c_longlong(stride), c_int(q_rank), c_int(kv_rank),
+          c_int(rot_dim), c_int(rotary_dim), _ptr(q_weight if q_rank else None), _ptr(kv_weight if write_kv else None),
+          _ptr(inv_freq if write_kv and rotary_dim else None), _ptr(positions if write_kv else None), _ptr(token_seq if write_kv else None),
+          _ptr(block_table if write_kv else None), c_int(table_stride), _ptr(key_pages if write_kv else None),
+          _ptr(value_pages if write_kv else None), _ptr(cq_out), c_int(_code(dtype)), c_float(eps), c_int(tokens), c_int(block_size),
+          c_int(num_blocks), c_int(1 if write_kv else 0), c_int(row), c_int(latent_row), c_int(1 if interleaved else 0),
+          c_float(magnitude), _stream())
     return cq_out
 
 
 def latent_query_pack(q: Tensor, qa: Tensor, inv_freq: Tensor | None, positions: Tensor, out: Tensor, *, heads: int, dim: int,
-                      rot_dim: int, rotary_dim: int, kv_rank: int) -> Tensor:
-    """The attention's query rows ``out`` [T, heads, kv_rank + rot_dim]: head h's first kv_rank dims are
-    ``qa[h, t]`` (qa [heads, T, kv_rank]: the queries taken through the keys' up-projection), the rest the
-    last rot_dim dims of head h of ``q`` [T, heads * (dim + rot_dim)], their first ``rotary_dim`` rotated
-    (dim i with dim i + rotary_dim / 2, angle position * inv_freq[i], float32)."""
+                      rot_dim: int, rotary_dim: int, kv_rank: int, interleaved: bool = False, magnitude: float = 1.0) -> Tensor:
+    """The attention's query rows ``out`` [T, heads, row >= kv_rank + rot_dim], laid out like a cache row: head h's first
+    kv_rank dims are ``qa[h, t]`` (qa [heads, T, kv_rank]: the queries taken through the keys' up-projection; ``kv_rank`` here
+    is the latent part's width in a row, whatever it is filled up with), then the last rot_dim dims of head h of ``q``
+    [T, heads * (dim + rot_dim)], their first ``rotary_dim`` rotated as in ``latent_norm_rope_write``, then zeros."""
     _gpu(q, "q", contiguous=False)
     _gpu(qa, "qa", q.dtype)
     _gpu(out, "out", q.dtype)
     _gpu(positions, "positions", torch.int32)
     tokens = q.shape[0]
     q_stride = _strided_rows(q, "q", heads * (dim + rot_dim))
-    if qa.shape != (heads, tokens, kv_rank) or out.shape != (tokens, heads, kv_rank + rot_dim) or positions.numel() != tokens:
-        raise KernelError(f"qa must be [{heads}, {tokens}, {kv_rank}] and out [{tokens}, {heads}, {kv_rank + rot_dim}]")
+    if (qa.shape != (heads, tokens, kv_rank) or out.dim() != 3 or out.shape[:2] != (tokens, heads)
+            or out.shape[2] < kv_rank + rot_dim or positions.numel() != tokens):
+        raise KernelError(f"qa must be [{heads}, {tokens}, {kv_rank}] and out [{tokens}, {heads}, >= {kv_rank + rot_dim}]")
     if rotary_dim % 2 or not 0 <= rotary_dim <= rot_dim:
         raise KernelError("rotary_dim must be even and at most rot_dim")
     if rotary_dim:
@@ -1545,7 +1593,27 @@ def latent_query_pack(q: Tensor, qa: Tensor, inv_freq: Tensor | None, positions:
             raise KernelError(f"inv_freq must be [{rotary_dim // 2}]")
     _call("latent", "fe_latent_query_pack", _ptr(q), c_longlong(q_stride), _ptr(qa), _ptr(inv_freq if rotary_dim else None),
           _ptr(positions), _ptr(out), c_int(_code(q.dtype)), c_int(tokens), c_int(heads), c_int(dim), c_int(rot_dim),
-          c_int(rotary_dim), c_int(kv_rank), _stream())
+          c_int(rotary_dim), c_int(out.shape[2]), c_int(kv_rank), c_int(1 if interleaved else 0), c_float(magnitude), _stream())
+    return out
+
+
+def gate_heads(x: Tensor, gate: Tensor | None, out: Tensor) -> Tensor:
+    """``out[t, h * D + d] = x[h, t, d] * sigmoid(gate[t, h * D + d])`` (without a gate: the heads side by side): x [heads, T,
+    D], gate [T, heads * D] rows of any stride, out [T, heads * D], all in one dtype."""
+    _gpu(x, "x")
+    _gpu(out, "out", x.dtype)
+    if x.dim() != 3:
+        raise KernelError(f"x must be [heads, T, D], got {tuple(x.shape)}")
+    heads, tokens, dim = x.shape
+    if out.shape != (tokens, heads * dim):
+        raise KernelError(f"out must be [{tokens}, {heads * dim}], got {tuple(out.shape)}")
+    gate_stride = 0
+    if gate is not None:
+        gate_stride = _strided_rows(gate, "gate", heads * dim)
+        if gate.dtype != x.dtype or gate.shape[0] != tokens:
+            raise KernelError("gate must be in x's dtype with one row a token")
+    _call("latent", "fe_latent_gate_heads", _ptr(x), _ptr(gate), c_longlong(gate_stride), _ptr(out), c_int(_code(x.dtype)), c_int(tokens),
+          c_int(heads), c_int(dim), _stream())
     return out
 
 
@@ -1564,6 +1632,19 @@ def latent_splits(num_seqs: int, max_q_len: int, heads: int, max_ctx: int | None
     return max(1, min(-(-LATENT_TARGET_BLOCKS // blocks), max_ctx // (32 * LATENT_MIN_TILES), 32))
 
 
+LATENT_ROWS = ((96, 64), (160, 128), (192, 128), (320, 256), (576, 512))   # (row, latent part) the matrix-core kernel is compiled for
+
+
+def latent_row_sizes(dtype, kv_rank: int, rot_dim: int) -> tuple[int, int]:
+    """(width of a cache row, width of the latent part in it): the smallest sizes of the matrix-core kernel that a latent of
+    kv_rank and a rotated part of rot_dim fit into, filled up with zeros; where there are none, and in float32, their own."""
+    if dtype == torch.bfloat16:
+        for row, latent in LATENT_ROWS:
+            if kv_rank <= latent and rot_dim <= row - latent:
+                return row, latent
+    return kv_rank + rot_dim, kv_rank
+
+
 def latent_attention_supported(dtype, row_dim: int, value_dim: int, block_size: int) -> bool:
     """Whether the matrix-core kernel takes these sizes (else the vector-ALU kernel does)."""
     if dtype != torch.bfloat16 or block_size < 8 or block_size & (block_size - 1):      # pages of a power of two, eight slots or more
@@ -1575,11 +1656,13 @@ def latent_attention_supported(dtype, row_dim: int, value_dim: int, block_size: 
 
 def latent_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, out: Tensor, cu_q: Tensor, ctx_len: Tensor,
                      block_table: Tensor, *, num_seqs: int, max_q_len: int, heads: int, row_dim: int, value_dim: int,
-                     scale: float, num_decode: int | None = None, max_ctx: int | None = None, splits: int | None = None) -> Tensor:
+                     scale: float, num_decode: int | None = None, max_ctx: int | None = None, splits: int | None = None,
+                     window: int | None = None, sink: Tensor | None = None) -> Tensor:
     """Causal attention of ``heads`` query heads over one shared cache of rows, ``key_pages`` [blocks, 1,
     block_size, row_dim]: a row is the key of every head and its first ``value_dim`` dims are the value, which
     ``value_pages`` [blocks, 1, value_dim, block_size] holds a second time, transposed (None: a cache of keys
-    only, read by the vector-ALU kernel).  q [T, heads * row_dim], out [T, heads * value_dim]; scores and
+    only, read by the vector-ALU kernel).  ``window``: the token at position p reads keys j > p - window only; ``sink``
+    (float32 [heads]): exp(sink_h) joins head h's softmax denominator.  q [T, heads * row_dim], out [T, heads * value_dim]; scores and
     softmax float32.  bfloat16 at the sizes the matrix-core kernel is compiled for goes there (``splits``: its
     key runs, chosen here if None); everything else, and the float32 mode, to the vector-ALU kernel."""
     _gpu(q, "q")
@@ -1588,7 +1671,7 @@ def latent_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     if value_pages is None or not latent_attention_supported(q.dtype, row_dim, value_dim, block_size) or q.data_ptr() % 16:
         return masked_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table, num_seqs=num_seqs, max_q_len=max_q_len,
                                 q_heads=heads, kv_heads=1, head_dim=row_dim, value_dim=value_dim, scale=scale,
-                                num_decode=num_decode, max_ctx=max_ctx)
+                                num_decode=num_decode, max_ctx=max_ctx, window=window, sink=sink)
     _gpu(value_pages, "value_pages", q.dtype)
     _gpu(out, "out", q.dtype)
     _gpu(cu_q, "cu_q", torch.int32)
@@ -1606,7 +1689,14 @@ def latent_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
             or block_table.stride(1) != 1 or max_q_len < 1:
         raise KernelError("cu_q, ctx_len and block_table do not match the number of sequences")
     if splits is None:
-        splits = latent_splits(num_seqs, max_q_len, heads, max_ctx)
+        reach = max_ctx if max_ctx is None or window is None else min(max_ctx, window - 1 + max_q_len)
+        splits = latent_splits(num_seqs, max_q_len, heads, reach)
+    if window is not None and window < 1:
+        raise KernelError("window must be positive")
+    if sink is not None:
+        _gpu(sink, "sink", torch.float32)
+        if sink.shape != (heads,):
+            raise KernelError(f"sink must be [{heads}]")
     if not 1 <= splits <= 64:
         raise KernelError("between 1 and 64 key runs")
     part_o = part_ml = None
@@ -1616,7 +1706,7 @@ def latent_attention(q: Tensor, key_pages: Tensor, value_pages: Tensor | None, o
     _call("attention_latent", "fe_latent_attention", _ptr(q), c_longlong(q.stride(0)), _ptr(key_pages), _ptr(value_pages), _ptr(out),
           _ptr(part_o), _ptr(part_ml), _ptr(cu_q), _ptr(ctx_len), _ptr(block_table), c_int(block_table.stride(0)), c_int(num_seqs),
           c_int(max_q_len), c_int(heads), c_int(row_dim), c_int(value_dim), c_int(block_size), c_int(num_blocks), c_float(scale),
-          c_int(splits), c_int(tokens), _stream())
+          c_int(splits), c_int(tokens), c_int(window or 0), _ptr(sink), _stream())
     return out
 
 
@@ -1797,17 +1887,28 @@ def scale_rows(x: Tensor, factor: float) -> Tensor:
     return x
 
 
+def cap_rows(x: Tensor, cap: float, factor: float = 1.0) -> Tensor:
+    """x <- cap * tanh(x * factor / cap), in place (float32)."""
+    _gpu(x, "x", torch.float32)
+    if not cap > 0.0:
+        raise KernelError("a soft cap is positive")
+    _call("hyper", "fe_cap_rows", _ptr(x), c_float(factor), c_float(cap), c_longlong(x.numel()), _stream())
+    return x
+
+
 # ------------------------------------------------- a norm over the whole projection, rotation, page write
 
 def whole_norm_rope_write(qkv: Tensor, q_weight: Tensor, k_weight: Tensor | None, inv_freq: Tensor | None, positions: Tensor,
                           token_seq: Tensor, block_table: Tensor, key_pages: Tensor, value_pages: Tensor, q_out: Tensor, *,
                           q_heads: int, kv_heads: int, head_dim: int, value_dim: int, rotary_dim: int, eps: float,
-                          magnitude: float = 1.0, write_kv: bool = True) -> None:
+                          magnitude: float = 1.0, write_kv: bool = True, bias: Tensor | None = None) -> None:
     """q (and k) divided by the root mean square over the whole projection (all heads at once, epsilon
     inside the root) times a weight of that length; then the first ``rotary_dim`` dims of every head turn
     (dim i pairs with i + rotary_dim / 2, cosines and sines times ``magnitude``); q into ``q_out``
     [T, Hq * D], k and v into their pages (values transposed).  qkv [T, >= q | k | v] with any row stride;
-    with ``write_kv`` False it holds q alone and the pages are left as they are.  float32 inside."""
+    with ``write_kv`` False it holds q alone and the pages are left as they are.  ``bias`` (float32, over all of [q | k
+    | v]) is added to the projection first.  Pages whose rows are wider than a head: q_out has the key pages' row width, q
+    and key rows are filled up with zeros, the rest of a value's dims is left alone.  float32 inside."""
     q_size, kv_size, v_size = q_heads * head_dim, kv_heads * head_dim, kv_heads * value_dim
     need = q_size + (kv_size + v_size if write_kv else 0)
     _gpu(qkv, "qkv", contiguous=False)
@@ -1815,8 +1916,17 @@ def whole_norm_rope_write(qkv: Tensor, q_weight: Tensor, k_weight: Tensor | None
     if qkv.dim() != 2 or qkv.shape[1] < need or qkv.stride(1) != 1:
         raise KernelError(f"qkv must be [T, >= {need}] with unit inner stride")
     _gpu(q_out, "q_out", qkv.dtype)
-    if q_out.shape != (tokens, q_size):
-        raise KernelError(f"q_out must be [{tokens}, {q_size}]")
+    if bias is not None:
+        _gpu(bias, "bias", torch.float32)
+        if bias.shape != (need,):
+            raise KernelError(f"bias must be [{need}]")
+    key_row, value_row = head_dim, value_dim
+    if write_kv and key_pages.dim() == 4 and value_pages.dim() == 4:
+        key_row, value_row = key_pages.shape[3], value_pages.shape[2]
+    elif not write_kv and q_out.dim() == 2 and q_out.shape[1] % q_heads == 0:
+        key_row = q_out.shape[1] // q_heads
+    if q_out.shape != (tokens, q_heads * key_row) or key_row < head_dim:
+        raise KernelError(f"q_out must be [{tokens}, {q_heads * key_row}]")
     _gpu(q_weight, "q_weight", torch.float32)
     if q_weight.shape != (q_size,):
         raise KernelError(f"q_weight must be [{q_size}]")
@@ -1836,23 +1946,23 @@ def whole_norm_rope_write(qkv: Tensor, q_weight: Tensor, k_weight: Tensor | None
         _gpu(block_table, "block_table", torch.int32)
         _gpu(key_pages, "key_pages", qkv.dtype)
         _gpu(value_pages, "value_pages", qkv.dtype)
-        if key_pages.dim() != 4 or key_pages.shape[1] != kv_heads or key_pages.shape[3] != head_dim:
-            raise KernelError(f"key pages must be [blocks, {kv_heads}, block_size, {head_dim}], got {tuple(key_pages.shape)}")
+        if key_pages.dim() != 4 or key_pages.shape[1] != kv_heads or key_pages.shape[3] < head_dim:
+            raise KernelError(f"key pages must be [blocks, {kv_heads}, block_size, >= {head_dim}], got {tuple(key_pages.shape)}")
         num_blocks, _, block_size, _ = key_pages.shape
-        if value_pages.shape != (num_blocks, kv_heads, value_dim, block_size):
-            raise KernelError(f"value pages are transposed: [blocks, {kv_heads}, {value_dim}, block_size], got {tuple(value_pages.shape)}")
+        if value_pages.shape != (num_blocks, kv_heads, value_row, block_size) or value_row < value_dim:
+            raise KernelError(f"value pages are transposed: [blocks, {kv_heads}, >= {value_dim}, block_size], got {tuple(value_pages.shape)}")
         if block_table.dim() != 2 or block_table.stride(1) != 1:
             raise KernelError("block_table must be [sequences, max_blocks] with unit inner stride")
         table_stride = block_table.stride(0)
     if not eps > 0.0:
         raise KernelError("eps must be positive")
     stride = qkv.stride(0) if tokens > 1 else max(qkv.stride(0), qkv.shape[1])
-    _call("whole_norm_rope", "fe_whole_norm_rope_write", _ptr(qkv), c_int(_code(qkv.dtype)), c_longlong(stride), _ptr(q_weight),
+    _call("whole_norm_rope", "fe_whole_norm_rope_write", _ptr(qkv), c_int(_code(qkv.dtype)), c_longlong(stride), _ptr(bias), _ptr(q_weight),
           _ptr(k_weight if write_kv else None), _ptr(inv_freq if rotary_dim else None), _ptr(positions), _ptr(token_seq),
           _ptr(block_table if write_kv else None), c_int(table_stride), _ptr(key_pages if write_kv else None),
           _ptr(value_pages if write_kv else None), _ptr(q_out), c_int(tokens), c_int(q_heads), c_int(kv_heads), c_int(head_dim),
           c_int(value_dim), c_int(rotary_dim), c_float(eps), c_float(magnitude), c_int(1 if write_kv else 0), c_int(block_size),
-          c_int(num_blocks), _stream())
+          c_int(num_blocks), c_int(key_row), c_int(value_row), _stream())
 
 
 # ------------------------------------------------- a mixture of experts

@@ -113,9 +113,11 @@ class DecoderModel:
         residual = self.embedding.forward(batch) if embedding_view is None else self.embedding.forward(batch, embedding_view)
         if self.entry is not None:
             self.entry.begin(residual, batch)
+        passes = 0
         for index, call in enumerate(self.schedule):
             if call.enters:
-                self.entry.forward(residual, batch)
+                self.entry.forward(residual, batch, passes)
+                passes += 1
             self.layers[call.layer].forward(residual, batch, cache_views[index], call.writes_cache)
         if batch.num_wanted == 0:
             residual.flush()

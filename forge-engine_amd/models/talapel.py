@@ -64,11 +64,11 @@ def _feed_forward(config: TalapelConfig, mlp: dict | None, prefix: str) -> PartS
     }, prefix)
 
 
-def _schedule(config: TalapelConfig) -> tuple[LayerCall, ...]:
-    count = len(config.layers)
-    if config.loop is None:
+def run_order(count: int, loop: tuple[int, int, int] | None) -> tuple[LayerCall, ...]:
+    """The calls of ``count`` layers of which the run ``loop`` (start, stop, times) is passed through several times."""
+    if loop is None:
         return tuple(LayerCall(index) for index in range(count))
-    start, stop, times = config.loop
+    start, stop, times = loop
     calls = [LayerCall(index) for index in range(start)]
     for _ in range(times):
         calls += [LayerCall(index, enters=index == start) for index in range(start, stop)]
@@ -91,7 +91,7 @@ def talapel_plan(config: TalapelConfig) -> ModelPlan:
         vocab_size=config.vocab,
         embedding=PartSpec("token_embedding", dict(sizes, scale=config.embedding_scale), "embed"),
         layers=layers,
-        schedule=_schedule(config),
+        schedule=run_order(len(layers), config.loop),
         final_norm=norm("final.norm"),
         head=PartSpec("lm_head", dict(sizes), "head"),
         entry=None if config.loop is None else PartSpec("concat_projection", {"hidden_size": width, "leaf": ""}, "loop.in"),

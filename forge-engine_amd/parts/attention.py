@@ -37,7 +37,8 @@ and k head, before the rotation, in the kernel that writes the pages);
 ``query_temperature`` (``{"coef": c, "every": n}``: queries at position p times
 ``1 + c ln(floor((p + 1) / n) + 1)``); ``output_scale`` (a factor on the layer's output, its bias included; it comes
 with an output gate, whose kernel applies it in float32); ``fill_rows`` (bfloat16 with an output gate: heads and values
-of sizes that the matrix-core kernels do not take, up to 128, lie in rows of 64 or 128 that are filled up with zeros);
+of sizes that the matrix-core kernels do not take, up to 128, lie in rows of 64 or 128 that are filled up with zeros;
+without a gate likewise, and the output projection's columns with them);
 ``force_general`` (take the general path whatever the options).  A position part may scale its
 cosines and sines (``magnitude``).  With any of them the step takes the general path:
 one product for q, k, v (and the gate), one kernel for convolution, rotation, norms and the
@@ -119,8 +120,10 @@ class GroupedQueryAttention(Mixer):
         self.bias_table: Tensor | None = None       # as loaded [rows, heads]; by distance [heads, span] after finalize
         self.mix_weight: float | None = None
         self.slopes: Tensor | None = None
-        if whole_norm_eps is not None and (self.conv_taps or unit_norm_eps is not None or bias):
-            raise ValueError("a norm over the whole projection is not combined with convolutions, unit norms or biases")
+        if whole_norm_eps is not None and (self.conv_taps or unit_norm_eps is not None):
+            raise ValueError("a norm over the whole projection is not combined with convolutions or unit norms")
+        if bias and not own_kv:
+            raise ValueError("a layer without keys and values of its own has no biases")
         if not own_kv and whole_norm_eps is None:
             raise ValueError("a layer without keys and values of its own takes the path of the whole-projection norm")
         if self.conv_taps < 0:
@@ -139,7 +142,7 @@ class GroupedQueryAttention(Mixer):
         # the widths of a cached key's and value's row
         self.key_row, self.value_row = head_dim, self.value_dim
         widest = max(head_dim, self.value_dim)
-        if fill_rows and self.output_gate and own_kv and whole_norm_eps is None and ctx.dtype == torch.bfloat16 and widest <= 128:
+        if fill_rows and self.general and own_kv and ctx.dtype == torch.bfloat16 and widest <= 128:
             self.key_row = self.value_row = 64 if widest <= 64 else 128
         if (value_mix is not None or fixed_sink is not None or distance_slope_bits is not None) and whole_norm_eps is not None:
             raise ValueError("value mixing, fixed sinks and distance slopes are not combined with the whole-projection norm")
@@ -153,6 +156,8 @@ class GroupedQueryAttention(Mixer):
         self.window = window
         self.scale = head_dim ** -0.5 if scale is None else float(scale)
         self.position = build_part("position", position, ctx)
+        if self.position.interleaved:
+            raise ValueError("this attention turns dims half a rotation apart")
         self.conv_channels = self.q_size + self.kv_size + self.v_size
         if not own_kv:
             self.conv_channels = self.q_size
@@ -273,6 +278,10 @@ class GroupedQueryAttention(Mixer):
             self.qkv_bias = self.qkv_bias.to(self.qkv_weight.dtype)
         if self.o_bias is not None and self.o_weight.dtype != torch.float32:
             self.o_bias = self.o_bias.to(self.o_weight.dtype)
+        if not self.output_gate and self.value_row > self.value_dim:      # columns of zeros for what fills the heads' results up
+            wide = torch.zeros((self.hidden_size, self.num_heads, self.value_row), dtype=self.o_weight.dtype, device=device)
+            wide[:, :, :self.value_dim] = self.o_weight.view(self.hidden_size, self.num_heads, self.value_dim)
+            self.o_weight = wide.view(self.hidden_size, -1)
 
     def _bias_by_distance(self, table: Tensor) -> Tensor:
         """The loaded table [rows, heads] laid out by distance, float32 [heads, span]: entry n is the row of
@@ -355,10 +364,12 @@ class GroupedQueryAttention(Mixer):
             raise ValueError("the general attention path writes its own keys and values, except for a layer that "
                              "has none and reads another call's")
         qkv = ops.linear(x, self.qkv_weight)        # [T, q | k | v (| gate)]; the bias is added by the kernel below
-        attn = torch.empty((x.shape[0], self.out_size), dtype=x.dtype, device=x.device)
+        out_size = self.out_size if self.output_gate else self.num_heads * self.value_row
+        attn = torch.empty((x.shape[0], out_size), dtype=x.dtype, device=x.device)
         self._attend(qkv, attn, batch, cache, writes_cache, inv_freq, rotary_dim)
-        update = ops.linear_update(attn, self.o_weight)
-        return update if self.o_bias_f32 is None else ops.add_bias(update, self.o_bias_f32)
+        if self.o_bias_f32 is None:
+            return ops.linear_update(attn, self.o_weight, stream=stream)
+        return ops.add_bias(ops.linear_update(attn, self.o_weight), self.o_bias_f32)
 
     def joint_ends(self) -> JointEnds | None:
         if not (self.general and self.own_kv and self.output_gate):
@@ -382,15 +393,17 @@ class GroupedQueryAttention(Mixer):
                 qkv, self.q_norm, self.k_norm, inv_freq, batch.positions, batch.token_seq, cache.block_table,
                 cache.key_pages, cache.value_pages, q, q_heads=self.num_heads, kv_heads=self.num_kv_heads,
                 head_dim=self.head_dim, value_dim=self.value_dim, rotary_dim=rotary_dim, eps=self.whole_norm_eps,
-                magnitude=magnitude, write_kv=writes_cache)
+                magnitude=magnitude, write_kv=writes_cache, bias=self.conv_bias)
         elif magnitude != 1.0:
             raise ValueError("scaled cosines and sines come with the whole-projection norm's kernel only")
         else:
             self._conv_rope(qkv, q, batch, cache, inv_freq, rotary_dim)
+        whole_rows = not self.output_gate       # a gate's kernel takes the heads out of rows that are wider
         ops.masked_attention(
             q, cache.key_pages, cache.value_pages, attn, batch.cu_q, batch.ctx_len, cache.block_table,
             num_seqs=batch.num_seqs, max_q_len=batch.max_q_len, q_heads=self.num_heads,
-            kv_heads=self.num_kv_heads, head_dim=self.head_dim, value_dim=self.value_dim, scale=self.scale,
+            kv_heads=self.num_kv_heads, head_dim=self.key_row if whole_rows else self.head_dim,
+            value_dim=self.value_row if whole_rows else self.value_dim, scale=self.scale,
             window=self.window, chunk=self.chunk, sink=self.sink_weight, slopes=self.slopes, dist_bias=self.bias_table,
             gate=qkv[:, self.conv_channels:] if self.output_gate else None, num_decode=batch.num_decode,
             max_ctx=batch.max_ctx, softcap=self.softcap, head_gate=self.head_gate, factor=self.output_scale)

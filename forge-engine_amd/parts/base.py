@@ -69,6 +69,7 @@ class Residual:
         self.streams: Tensor | None = None
         self.pending_mix: tuple[Tensor, Tensor] | None = None    # (mix [S, S] indexed [from, to], share [S])
         self.pending_bias: Tensor | None = None                   # float32 [W]: added with the pending update, or alone
+        self.pending_other: Tensor | None = None                  # float32 like h, somebody else's: added with what is pending, or alone
         self.pending_norm: tuple[Tensor, float] | None = None    # (weight, eps): the update is RMS-normed before it is added
         self.in_compute_dtype: Tensor | None = None               # the stream as a norm of updates last stored it beside h (the same values)
 
@@ -79,8 +80,26 @@ class Residual:
         self.in_compute_dtype = None
         self.pending, self.pending_bias = update, bias
 
+    def join(self, other: Tensor | None, shift: Tensor | None) -> None:
+        """Leave ``h += other + shift`` pending on top of the update that is pending already (``other`` float32 like h,
+        which stays as it is; ``shift`` one number a channel): the next norm adds all of it in one pass."""
+        if self.streams is not None:
+            raise ValueError("additions to the stream itself need a model with one stream")
+        if not (self.pending_norm is None and self.pending_bias is None and self.pending_other is None):
+            self.flush()
+        self.in_compute_dtype = None
+        self.pending_other, self.pending_bias = other, shift
+
+    def take_joined(self) -> tuple[Tensor | None, Tensor | None, Tensor | None]:
+        """(update, other, shift) of what is pending, which the caller now applies itself."""
+        update, other, shift = self.pending, self.pending_other, self.pending_bias
+        self.pending = self.pending_other = self.pending_bias = None
+        return update, other, shift
+
     def take_biased(self) -> tuple[Tensor | None, Tensor | None]:
         """(update, bias) of what is pending, which the caller now applies itself."""
+        if self.pending_other is not None:
+            self.flush()
         update, bias = self.pending, self.pending_bias
         self.pending = self.pending_bias = None
         return update, bias
@@ -89,7 +108,7 @@ class Residual:
         """The stream is another tensor from here on (nothing of the old one, or pending on it, counts any more)."""
         self.h = h
         self.in_compute_dtype = None
-        self.pending, self.pending_bias = update, None
+        self.pending, self.pending_bias, self.pending_other = update, None, None
 
     def add_normed(self, update: Tensor, weight: Tensor, eps: float) -> None:
         """Leave ``h += update * rsqrt(mean(update^2) + eps) * weight`` pending (a norm behind a
@@ -141,11 +160,10 @@ class Residual:
         return out
 
     def flush(self) -> Tensor:
-        if self.pending_bias is not None:
+        if self.pending_bias is not None or self.pending_other is not None:
             if self.streams is not None:
                 raise ValueError("a bias on an update needs a model with one residual stream")
-            update, bias = self.take_biased()
-            ops.hyper_norm(self.h.unsqueeze(0), update, None, None, None, None, None, 0.0, None, shift=bias)
+            ops.add_rows(self.h, *self.take_joined())
         elif self.pending is not None:
             if self.streams is not None:
                 update, mix, share = self.take_pending()
@@ -229,6 +247,11 @@ class PositionEncoding(Part):
         q and k, or None."""
         return None
 
+    @property
+    def interleaved(self) -> bool:
+        """Whether dim 2i is paired with dim 2i + 1 (else dim i with i + rotary_dim / 2)."""
+        return False
+
     def magnitude(self) -> float:
         """A factor on every cosine and sine of the rotation (1: a plain rotation)."""
         return 1.0
@@ -307,8 +330,8 @@ class StreamEntry(Part):
     def begin(self, residual: Residual, batch) -> None:
         """Once a step, right behind the embedding: keep what the passes need of it (in ``batch.carry``)."""
 
-    def forward(self, residual: Residual, batch) -> None:
-        """Ahead of the first layer of a pass: replace the stream."""
+    def forward(self, residual: Residual, batch, number: int = 0) -> None:
+        """Ahead of the first layer of pass ``number`` (counted from 0 in every step): change the stream."""
         raise NotImplementedError
 
 

@@ -19,26 +19,38 @@ from .base import BuildContext, Embedding, Head, ParamSpec, Residual
 
 class TokenEmbedding(Embedding):
     def __init__(self, ctx: BuildContext, prefix: str, *, vocab_size: int, hidden_size: int,
-                 leaf: str = "weight", scale: float = 1.0) -> None:
-        """``scale``: a factor on every row as it enters the float32 stream."""
+                 leaf: str = "weight", scale: float = 1.0, norm_leaf: str | None = None, norm_eps: float = 1e-6) -> None:
+        """``scale``: a factor on every row as it enters the float32 stream.  ``norm_leaf``: the name, behind the prefix, of
+        the weight of an RMS norm of the row (None: no norm), which the same kernel applies."""
         super().__init__(ctx, prefix)
         self.vocab_size = vocab_size
         self.hidden_size = hidden_size
         self.leaf = leaf        # the table's name behind the prefix ("": the prefix itself)
         self.scale = float(scale)
+        self.norm_leaf, self.norm_eps = norm_leaf, float(norm_eps)
         self.weight: Tensor | None = None
+        self.norm_weight: Tensor | None = None
 
     def param_specs(self):
-        return {self.name(self.leaf): ParamSpec((self.vocab_size, self.hidden_size))}
+        specs = {self.name(self.leaf): ParamSpec((self.vocab_size, self.hidden_size))}
+        if self.norm_leaf is not None:
+            specs[self.name(self.norm_leaf)] = ParamSpec((self.hidden_size,), kind="vector", init="norm")
+        return specs
 
     def set_param(self, name: str, tensor: Tensor) -> None:
-        if name != self.name(self.leaf):
+        if name == self.name(self.leaf):
+            self.weight = tensor
+        elif self.norm_leaf is not None and name == self.name(self.norm_leaf):
+            self.norm_weight = tensor
+        else:
             raise KeyError(name)
-        self.weight = tensor
 
     def forward(self, batch) -> Residual:
         h = torch.empty((batch.num_tokens, self.hidden_size), dtype=torch.float32, device=self.weight.device)
-        ops.embed_rows(batch.token_ids, self.weight, h, self.scale)
+        if self.norm_weight is not None:
+            ops.embed_rows(batch.token_ids, self.weight, h, self.scale, self.norm_weight, self.norm_eps)
+        else:
+            ops.embed_rows(batch.token_ids, self.weight, h, self.scale)
         return Residual(h)
 
     def kernel_libraries(self):
@@ -86,10 +98,11 @@ class TokenPairEmbedding(TokenEmbedding):
 
 class LMHead(Head):
     def __init__(self, ctx: BuildContext, prefix: str, *, vocab_size: int, hidden_size: int,
-                 tied: bool = False, leaf: str = "weight", scale: float = 1.0) -> None:
-        """``scale``: a factor on the logits."""
+                 tied: bool = False, leaf: str = "weight", scale: float = 1.0, softcap: float | None = None) -> None:
+        """``scale``: a factor on the logits; ``softcap``: they then become ``cap * tanh(logit / cap)``."""
         super().__init__(ctx, prefix)
         self.scale = float(scale)
+        self.softcap = None if softcap is None else float(softcap)
         self.vocab_size = vocab_size
         self.hidden_size = hidden_size
         self.tied = tied
@@ -116,10 +129,12 @@ class LMHead(Head):
     def forward(self, z: Tensor) -> Tensor:
         # float32 accumulation and float32 logits in both modes (no rounding of the logits)
         logits = ops.linear(z, self.matrix(), out_dtype=torch.float32)
+        if self.softcap is not None:
+            return ops.cap_rows(logits, self.softcap, self.scale)
         return logits if self.scale == 1.0 else ops.scale_rows(logits, self.scale)
 
     def kernel_libraries(self):
-        return {"gemm_f32", "gemm_skinny"} | ({"hyper"} if self.scale != 1.0 else set())
+        return {"gemm_f32", "gemm_skinny"} | ({"hyper"} if self.scale != 1.0 or self.softcap is not None else set())
 
 
 register_part("embedding", "token_embedding", TokenEmbedding)

@@ -4,6 +4,9 @@
 every pass, what the pass before made of the stream blended with where it came from.  The stream, with what is
 pending on it, and x0 lie side by side in the compute dtype (x0 is put there once a step); the product's float32 result
 is the new stream (its first part, with the other parts pending, where it comes in partial sums over K).
+
+``pass_vectors``: ``x <- x + x0 + s_t`` ahead of pass t (in the first pass without x0), s_t a learned vector of the
+pass.  Both are left pending on the stream, beside the update of the layer before, for the kernel of the next norm.
 """
 
 from __future__ import annotations
@@ -39,7 +42,7 @@ class ConcatProjection(StreamEntry):
         batch.carry[self.CARRY] = pair
         ops.stream_sum_cast(h, None, None, pair[:, self.hidden_size:])
 
-    def forward(self, residual: Residual, batch) -> None:
+    def forward(self, residual: Residual, batch, number: int = 0) -> None:
         if residual.streams is not None or residual.pending_norm is not None:
             residual.flush()
         pair = batch.carry[self.CARRY]
@@ -55,4 +58,36 @@ class ConcatProjection(StreamEntry):
         return {"stream_ops", "gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide"}
 
 
+class PassVectors(StreamEntry):
+    CARRY = "stream entry"
+
+    def __init__(self, ctx: BuildContext, prefix: str, *, hidden_size: int, passes: int, leaf: str = "step") -> None:
+        super().__init__(ctx, prefix)
+        self.hidden_size, self.passes, self.leaf = hidden_size, passes, leaf
+        self.steps: Tensor | None = None       # [passes, hidden]
+
+    def param_specs(self):
+        return {self.name(self.leaf): ParamSpec((self.passes, self.hidden_size), kind="vector", init="unit")}
+
+    def set_param(self, name: str, tensor: Tensor) -> None:
+        if name != self.name(self.leaf):
+            raise KeyError(name)
+        self.steps = tensor.contiguous()
+
+    def begin(self, residual: Residual, batch) -> None:
+        if self.passes < 2:
+            return
+        h = residual.flush()
+        batch.carry[self.CARRY] = ops.stream_sum_cast(h, None, None, torch.empty_like(h))     # the stream itself changes in place
+
+    def forward(self, residual: Residual, batch, number: int = 0) -> None:
+        if not 0 <= number < self.passes:
+            raise ValueError(f"{self.prefix}: pass {number} of {self.passes}")
+        residual.join(batch.carry[self.CARRY] if number else None, self.steps[number])
+
+    def kernel_libraries(self):
+        return {"stream_ops", "rowwise"}
+
+
 register_part("entry", "concat_projection", ConcatProjection)
+register_part("entry", "pass_vectors", PassVectors)

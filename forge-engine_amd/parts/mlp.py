@@ -1,6 +1,6 @@
-"""Gated SiLU feed-forward: ``down(silu(gate(x)) * up(x))``, no biases
-(reference: src/forge_engine/qwen3.py:210-227).  gate and up share one fused
-matrix [2I, H] so that a step makes one product for both."""
+"""Gated feed-forward: ``down(act(gate(x)) * up(x))``, no biases, the activation SiLU
+(reference: src/forge_engine/qwen3.py:210-227) or, by ``activation``, the tanh form of gelu.  gate and up share
+one fused matrix [2I, H] so that a step makes one product for both."""
 
 from __future__ import annotations
 
@@ -16,8 +16,11 @@ class SwiGLU(FeedForward):
     DEFAULT_NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
     def __init__(self, ctx: BuildContext, prefix: str, *, hidden_size: int, intermediate_size: int,
-                 names: dict[str, str] | None = None) -> None:
+                 activation: str = "silu", names: dict[str, str] | None = None) -> None:
         super().__init__(ctx, prefix)
+        if activation not in ops.GATE_ACTS:
+            raise ValueError(f"unknown activation '{activation}' (known: {', '.join(ops.GATE_ACTS)})")
+        self.activation = activation
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
         self.names = dict(self.DEFAULT_NAMES, **(names or {}))
@@ -50,7 +53,7 @@ class SwiGLU(FeedForward):
     takes_stream = True
 
     def forward(self, x: Tensor, batch=None, stream: Tensor | None = None) -> Tensor | None:
-        act = ops.linear_swiglu(x, self.gate_up_weight)
+        act = ops.linear_swiglu(x, self.gate_up_weight, self.activation)
         return ops.linear_update(act, self.down_weight, stream=stream)   # the update stays float32 for the residual sum
 
     def joint_ends(self) -> JointEnds:
@@ -60,7 +63,7 @@ class SwiGLU(FeedForward):
         self.gate_up_weight = self.down_weight = None
 
     def forward_joint(self, z: Tensor, out: Tensor, batch=None) -> None:
-        ops.swiglu(z, out)
+        ops.swiglu(z, out, self.activation)
 
     def kernel_libraries(self):
         return {"rowwise", "gemm_f32", "gemm_skinny", "gemm_mid", "gemm_wide", "gemm_tile"}

@@ -38,8 +38,6 @@ class RMSNorm(Norm):
         self.weight = tensor + self.offset if self.offset else tensor
 
     def forward(self, residual: Residual, rows: Tensor | None = None) -> Tensor:
-        if residual.pending_bias is not None:    # this kernel knows no bias on the update
-            residual.flush()
         if residual.pending_norm is not None:    # a norm behind the sublayer before: both norms in one pass over the row
             if rows is not None:                 # the chosen rows alone; stream and pending update are left as they are
                 update, (weight, eps) = residual.pending, residual.pending_norm
@@ -51,10 +49,11 @@ class RMSNorm(Norm):
         if rows is not None:    # the chosen rows of stream + pending update; both are left as they are
             h = residual.h
             out = torch.empty((rows.numel(), self.size), dtype=self.ctx.dtype, device=h.device)
-            return ops.add_rmsnorm(h, residual.pending, self.weight, self.eps, out, rows=rows, store_sum=False)
-        update, residual.pending = residual.pending, None
+            return ops.add_rmsnorm(h, residual.pending, self.weight, self.eps, out, rows=rows, store_sum=False,
+                                   other=residual.pending_other, shift=residual.pending_bias)
+        update, other, shift = residual.take_joined()
         out = torch.empty((residual.h.shape[0], self.size), dtype=self.ctx.dtype, device=residual.h.device)
-        return ops.add_rmsnorm(residual.h, update, self.weight, self.eps, out)
+        return ops.add_rmsnorm(residual.h, update, self.weight, self.eps, out, other=other, shift=shift)
 
     def kernel_libraries(self):
         return {"rowwise", "stream_ops"}
@@ -114,6 +113,8 @@ class LayerNorm(Norm):
             raise KeyError(name)
 
     def forward(self, residual: Residual, rows: Tensor | None = None, read: Tensor | None = None) -> Tensor:
+        if residual.pending_other is not None:    # this kernel knows an update and a bias only
+            residual.flush()
         streams = residual.streams if residual.streams is not None else residual.h.unsqueeze(0)
         count = streams.shape[1] if rows is None else rows.numel()
         out = torch.empty((count, self.size), dtype=self.ctx.dtype, device=streams.device)

@@ -5,7 +5,8 @@ rotates q and k with.
 same expression as the reference (src/forge_engine/qwen3.py:352-360) so that the
 angles ``float(position) * inv_freq[j]`` are bit-equal to its own.  R is the
 number of rotated dims (the whole head unless ``rotary_dim`` says less); the
-partner of dim j is j + R/2 (rotate-half pairing, qwen3.py:366-381).
+partner of dim j is j + R/2 (rotate-half pairing, qwen3.py:366-381), unless ``interleaved``
+makes pairs of neighbours.
 """
 
 from __future__ import annotations
@@ -21,10 +22,11 @@ from .base import BuildContext, PositionEncoding
 
 class RotaryPosition(PositionEncoding):
     def __init__(self, ctx: BuildContext, prefix: str = "", *, head_dim: int, theta: float,
-                 rotary_dim: int | None = None, precise: bool = False) -> None:
+                 rotary_dim: int | None = None, precise: bool = False, interleaved: bool = False) -> None:
         """``precise``: the table is computed in 64-bit and rounded once, instead of with the
-        reference's float32 expression."""
+        reference's float32 expression.  ``interleaved``: neighbouring dims form the pairs (2i with 2i + 1)."""
         super().__init__(ctx, prefix)
+        self._interleaved = bool(interleaved)
         self.theta = float(theta)
         self.rotary_dim = head_dim if rotary_dim is None else rotary_dim
         if self.rotary_dim % 2 or not 0 < self.rotary_dim <= head_dim:
@@ -38,8 +40,14 @@ class RotaryPosition(PositionEncoding):
     def rotary(self):
         return self.inv_freq, self.rotary_dim
 
+    @property
+    def interleaved(self) -> bool:
+        return self._interleaved
+
     def table(self, batch):
         """Formed once a step for all parts that turn alike."""
+        if self.interleaved:
+            raise ValueError("the table serves pairs of dims half a rotation apart")
         key = ("rotary", type(self), self.theta, self.rotary_dim)
         if key not in batch.carry:
             batch.carry[key] = ops.rotary_table(batch.positions, self.inv_freq)
@@ -56,8 +64,8 @@ class YarnRotaryPosition(RotaryPosition):
     (``magnitude``)."""
 
     def __init__(self, ctx: BuildContext, prefix: str = "", *, head_dim: int, theta: float, factor: float,
-                 original: float, fast: float, slow: float, rotary_dim: int | None = None) -> None:
-        super().__init__(ctx, prefix, head_dim=head_dim, theta=theta, rotary_dim=rotary_dim)
+                 original: float, fast: float, slow: float, rotary_dim: int | None = None, interleaved: bool = False) -> None:
+        super().__init__(ctx, prefix, head_dim=head_dim, theta=theta, rotary_dim=rotary_dim, interleaved=interleaved)
         dims, half = self.rotary_dim, self.rotary_dim // 2
 
         def turning(turns: float) -> float:

@@ -81,10 +81,12 @@ class StateSpaceMixer(Mixer):
             states[self.CONV_STATE] = FixedState((self.conv_taps - 1, self.channels), torch.float32)
         return CacheNeeds(state=states)
 
-    def forward(self, x: Tensor, batch, cache: CacheView, writes_cache: bool = True) -> Tensor:
+    takes_stream = True
+
+    def forward(self, x: Tensor, batch, cache: CacheView, writes_cache: bool = True, stream: Tensor | None = None) -> Tensor | None:
         out = torch.empty((x.shape[0], self.inner), dtype=x.dtype, device=x.device)
         self.forward_joint(ops.linear(x, self.tensors["in"]), out, batch, cache, writes_cache)
-        return ops.linear_update(out, self.tensors["o"])
+        return ops.linear_update(out, self.tensors["o"], stream=stream)
 
     def joint_ends(self) -> JointEnds:
         return JointEnds(self.tensors["in"], self.tensors["o"])

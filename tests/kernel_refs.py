@@ -13,12 +13,16 @@ from __future__ import annotations
 import torch
 
 
-def embed_rows(ids, table, out, scale=1.0):
-    out.copy_(table[ids.long()].float() * scale)
+def embed_rows(ids, table, out, scale=1.0, norm_weight=None, eps=0.0):
+    rows = table[ids.long()].float() * scale
+    out.copy_(rows if norm_weight is None else _unit(rows, eps) * norm_weight)
     return out
 
 
-def add_rmsnorm(h, delta, weight, eps, out, rows=None, store_sum=True):
+def add_rmsnorm(h, delta, weight, eps, out, rows=None, store_sum=True, other=None, shift=None):
+    if other is not None or shift is not None:
+        extra = sum(t for t in (other, None if shift is None else shift.expand_as(h)) if t is not None)
+        delta = extra if delta is None else extra + (delta.float().sum(0) if delta.dim() == 3 else delta.float())
     if delta is not None and delta.dim() == 3:
         delta = delta.float().sum(0)
     if rows is not None:
@@ -34,16 +38,27 @@ def add_rmsnorm(h, delta, weight, eps, out, rows=None, store_sum=True):
     return out
 
 
-def add_rows(h, delta):
-    h += delta.float().sum(0) if delta.dim() == 3 else delta.float()
+def add_rows(h, delta, other=None, shift=None):
+    if delta is not None:
+        h += delta.float().sum(0) if delta.dim() == 3 else delta.float()
+    for t in (other, shift):
+        if t is not None:
+            h += t
     return h
 
 
-def swiglu(gate_up, out):
+def _gate(g, act):
+    if act == "gelu_tanh":
+        return torch.nn.functional.gelu(g, approximate="tanh")
+    assert act == "silu"
+    return g / (1.0 + torch.exp(-g))
+
+
+def swiglu(gate_up, out, act="silu"):
     inter = gate_up.shape[1] // 2
     g = gate_up[:, :inter].float()
     u = gate_up[:, inter:].float()
-    out.copy_((g / (1.0 + torch.exp(-g)) * u).to(out.dtype))
+    out.copy_((_gate(g, act) * u).to(out.dtype))
     return out
 
 
@@ -65,20 +80,20 @@ def linear(x, weight, bias=None, out_dtype=None):
     return y.to(x.dtype if out_dtype is None else out_dtype)
 
 
-def linear_swiglu(x, gate_up_weight):
+def linear_swiglu(x, gate_up_weight, act="silu"):
     inter = gate_up_weight.shape[0] // 2
     y = x.float() @ gate_up_weight.float().T
     g, u = y[:, :inter], y[:, inter:]
-    return (g / (1.0 + torch.exp(-g)) * u).to(x.dtype)
+    return (_gate(g, act) * u).to(x.dtype)
 
 
 def linear_update(x, weight, bias=None, stream=None):
     return linear(x, weight, bias, out_dtype=torch.float32)    # the stream is left to the caller's add
 
 
-def gemm_skinny(x, weight, epilogue="bf16", tiles=0, waves=0, splits=1):
+def gemm_skinny(x, weight, epilogue="bf16", tiles=0, waves=0, splits=1, act="silu"):
     if epilogue == "swiglu":
-        return linear_swiglu(x, weight)
+        return linear_swiglu(x, weight, act)
     return linear(x, weight, out_dtype=torch.float32 if epilogue == "f32" else torch.bfloat16)
 
 
@@ -591,9 +606,16 @@ def scale_rows(x, factor):
     return x.mul_(factor)
 
 
+def cap_rows(x, cap, factor=1.0):
+    return x.copy_(cap * torch.tanh(x * factor / cap))
+
+
 def whole_norm_rope_write(qkv, q_weight, k_weight, inv_freq, positions, token_seq, block_table, key_pages, value_pages, q_out, *,
-                          q_heads, kv_heads, head_dim, value_dim, rotary_dim, eps, magnitude=1.0, write_kv=True):
+                          q_heads, kv_heads, head_dim, value_dim, rotary_dim, eps, magnitude=1.0, write_kv=True, bias=None):
     tokens = qkv.shape[0]
+    stored = qkv.dtype
+    if bias is not None:
+        qkv = qkv[:, :bias.numel()].float() + bias
     q_size, k_size, v_size = q_heads * head_dim, kv_heads * head_dim, kv_heads * value_dim
 
     def prepare(x, weight, heads):
@@ -607,18 +629,19 @@ def whole_norm_rope_write(qkv, q_weight, k_weight, inv_freq, positions, token_se
             x = torch.cat((lo * cos - hi * sin, hi * cos + lo * sin, x[..., rotary_dim:]), dim=-1)
         return x
 
-    q_out.copy_(prepare(qkv[:, :q_size], q_weight, q_heads).reshape(tokens, q_size).to(q_out.dtype))
+    key_row = q_out.shape[1] // q_heads         # rows wider than a head are filled up with zeros
+    q_out.view(tokens, q_heads, key_row).zero_()[..., :head_dim] = prepare(qkv[:, :q_size], q_weight, q_heads).to(q_out.dtype)
     if not write_kv:
         return
-    k = prepare(qkv[:, q_size:q_size + k_size], k_weight, kv_heads).to(qkv.dtype)
-    v = qkv[:, q_size + k_size:q_size + k_size + v_size].view(tokens, kv_heads, value_dim)
+    k = torch.nn.functional.pad(prepare(qkv[:, q_size:q_size + k_size], k_weight, kv_heads).to(stored), (0, key_row - head_dim))
+    v = qkv[:, q_size + k_size:q_size + k_size + v_size].reshape(tokens, kv_heads, value_dim).to(stored)
     block_size = key_pages.shape[2]
     for t in range(tokens):
         pos = int(positions[t])
         page = int(block_table[int(token_seq[t]), pos // block_size])
         assert page >= 0, "token without a page"
         key_pages[page, :, pos % block_size] = k[t]
-        value_pages[page, :, :, pos % block_size] = v[t]
+        value_pages[page, :, :value_dim, pos % block_size] = v[t]
 
 
 def moe_route(x, router_weight, router_bias, top, scoring="softmax"):
@@ -806,26 +829,31 @@ def gate_rows(update, logits, column):
     return update
 
 
-def _turn(r, positions, inv_freq, rotary_dim):
-    """r [T, ..., n]: its first rotary_dim dims rotated, dim i with dim i + rotary_dim / 2."""
+def _turn(r, positions, inv_freq, rotary_dim, interleaved=False, magnitude=1.0):
     if not rotary_dim:
         return r
     half = rotary_dim // 2
-    angle = positions.float().view(-1, *([1] * (r.dim() - 2)), 1) * inv_freq.view(*([1] * (r.dim() - 1)), half)
-    cos, sin = angle.cos(), angle.sin()
-    lo, hi = r[..., :half], r[..., half:rotary_dim]
-    return torch.cat((lo * cos - hi * sin, hi * cos + lo * sin, r[..., rotary_dim:]), dim=-1)
+    angle = positions.float().view(-1, *([1] * (r.dim() - 1))) * inv_freq
+    cos, sin = angle.cos() * magnitude, angle.sin() * magnitude
+    first, second = (slice(0, rotary_dim, 2), slice(1, rotary_dim, 2)) if interleaved else (slice(0, half), slice(half, rotary_dim))
+    out = r.clone()
+    out[..., first] = r[..., first] * cos - r[..., second] * sin
+    out[..., second] = r[..., second] * cos + r[..., first] * sin
+    return out
 
 
 def latent_norm_rope_write(x, q_weight, kv_weight, inv_freq, positions, token_seq, block_table, key_pages, value_pages, cq_out, *,
-                           q_rank, kv_rank, rot_dim, rotary_dim, eps, write_kv):
+                           q_rank, kv_rank, rot_dim, rotary_dim, eps, write_kv, interleaved=False, magnitude=1.0, latent_row=None):
     x = x.float()
-    cq_out.copy_((_unit(x[:, :q_rank], eps) * q_weight).to(cq_out.dtype))
+    latent_row = kv_rank if latent_row is None else latent_row
+    if q_rank:
+        cq_out.copy_((_unit(x[:, :q_rank], eps) * q_weight).to(cq_out.dtype))
     if not write_kv:
         return cq_out
     latent = _unit(x[:, q_rank:q_rank + kv_rank], eps) * kv_weight
-    turned = _turn(x[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim], positions, inv_freq, rotary_dim)
-    rows = torch.cat((latent, turned), dim=-1).to(key_pages.dtype)
+    turned = _turn(x[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim], positions, inv_freq, rotary_dim, interleaved, magnitude)
+    rows = torch.zeros((x.shape[0], key_pages.shape[3]), dtype=key_pages.dtype)
+    rows[:, :kv_rank], rows[:, latent_row:latent_row + rot_dim] = latent.to(rows.dtype), turned.to(rows.dtype)
     block_size = key_pages.shape[2]
     for t in range(x.shape[0]):
         pos = int(positions[t])
@@ -833,20 +861,32 @@ def latent_norm_rope_write(x, q_weight, kv_weight, inv_freq, positions, token_se
         assert page >= 0, "token without a page"
         key_pages[page, 0, pos % block_size] = rows[t]
         if value_pages is not None:
-            value_pages[page, 0, :, pos % block_size] = rows[t, :kv_rank]
+            value_pages[page, 0, :kv_rank, pos % block_size] = rows[t, :kv_rank]
     return cq_out
 
 
-def latent_query_pack(q, qa, inv_freq, positions, out, *, heads, dim, rot_dim, rotary_dim, kv_rank):
+def latent_query_pack(q, qa, inv_freq, positions, out, *, heads, dim, rot_dim, rotary_dim, kv_rank, interleaved=False, magnitude=1.0):
     tokens = q.shape[0]
-    turned = _turn(q.view(tokens, heads, dim + rot_dim)[:, :, dim:].float(), positions, inv_freq, rotary_dim)
+    turned = _turn(q.reshape(tokens, heads, dim + rot_dim)[:, :, dim:].float(), positions, inv_freq, rotary_dim, interleaved, magnitude)
+    out.zero_()
     out[:, :, :kv_rank] = qa.transpose(0, 1)
-    out[:, :, kv_rank:] = turned.to(out.dtype)
+    out[:, :, kv_rank:kv_rank + rot_dim] = turned.to(out.dtype)
     return out
 
 
+def gate_heads(x, gate, out):
+    y = x.transpose(0, 1).reshape(out.shape).float()
+    out.copy_((y if gate is None else y * torch.sigmoid(gate.float())).to(out.dtype))
+    return out
+
+
+def latent_row_sizes(dtype, kv_rank, rot_dim):
+    """A filled-up row in bfloat16, as the kernels would have it, in sizes of its own."""
+    return (kv_rank + rot_dim, kv_rank) if dtype == torch.float32 else (kv_rank + 3 + rot_dim + 2, kv_rank + 3)
+
+
 def latent_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table, *, num_seqs, max_q_len, heads, row_dim, value_dim,
-                     scale, num_decode=None, max_ctx=None, splits=None):
+                     scale, num_decode=None, max_ctx=None, splits=None, window=None, sink=None):
     block_size = key_pages.shape[2]
     for s in range(num_seqs):
         a, b = int(cu_q[s]), int(cu_q[s + 1])
@@ -857,9 +897,13 @@ def latent_attention(q, key_pages, value_pages, out, cu_q, ctx_len, block_table,
         values = rows[:, :value_dim] if value_pages is None else gather_pages(value_pages.transpose(2, 3), block_table[s], ctx, block_size)[0]
         for i in range(b - a):
             p = ctx - (b - a) + i
+            first = 0 if window is None else max(0, p - window + 1)
             queries = q[a + i].float().view(heads, row_dim)
-            weights = torch.softmax(queries @ rows[:p + 1].T * scale, dim=-1)         # [heads, p + 1]
-            out[a + i] = (weights @ values[:p + 1]).reshape(-1).to(out.dtype)
+            scores = queries @ rows[first:p + 1].T * scale
+            if sink is not None:
+                scores = torch.cat((scores, sink.view(heads, 1)), dim=-1)
+            weights = torch.softmax(scores, dim=-1)[:, :p + 1 - first]                # [heads, keys]
+            out[a + i] = (weights @ values[first:p + 1]).reshape(-1).to(out.dtype)
     return out
 
 
@@ -895,7 +939,7 @@ def linear_in_parts(x, weight):
 DECODE_SPLITS_TESTED = tuple(range(1, 65))
 
 
-NAMES = ("decode_prepare_supported", "linear_in_parts", "embed_rows", "add_rmsnorm", "add_rows", "swiglu", "gemm_nt_f32", "linear", "linear_update", "linear_swiglu", "gemm_skinny",
+NAMES = ("cap_rows", "gate_heads", "latent_row_sizes", "decode_prepare_supported", "linear_in_parts", "embed_rows", "add_rmsnorm", "add_rows", "swiglu", "gemm_nt_f32", "linear", "linear_update", "linear_swiglu", "gemm_skinny",
          "qk_norm_rope_write", "paged_attention", "argmax_rows", "sample_filtered_rows",
          "cast_rows", "add_bias", "token_shift", "rmsnorm_update", "rmsnorm_mean", "polynorm", "tanh_rows", "head_norm_gate",
          "conv_rope_norm_write", "masked_attention", "linear_recurrence", "mlstm_gate_scan",
