@@ -112,7 +112,7 @@ def parse_args():
     parser.add_argument("--points", default=None, help="other decode batch sizes to report")
     parser.add_argument("--widths", default="1024,2048,4096",
                         help="--phase design: model widths at which Mazanex and Qwen3 are measured side by side")
-    parser.add_argument("--design", choices=("mazanex", "rekezen", "malusun", "dubizen", "talapel"), default="mazanex",
+    parser.add_argument("--design", choices=("mazanex", "rekezen", "malusun", "dubizen", "talapel", "budanex"), default="mazanex",
                         help="--phase design: which design is measured beside Qwen3")
     parser.add_argument("--only", default="", help="--phase design: measure this model of the comparison alone")
     parser.add_argument("--phase", choices=("all", "decode", "prefill", "micro", "check", "design"), default="all",
@@ -405,12 +405,35 @@ def talapel_configs(width: int, layers: int) -> dict:
     return {"Talapel": talapel, "Mazanex": others["Mazanex"], "Malusun": others["Malusun"], "Qwen3": others["Qwen3"]}
 
 
+def budanex_configs(width: int, layers: int) -> dict:
+    """Budanex beside Dubizen (attention through a latent), Talapel (passes, the state-space recurrence, capped attention),
+    Rekezen (norms over whole projections) and Qwen3, at one width: heads of 128, the same vocabulary, as many layer runs
+    as the others have layers.  Budanex passes twice through half as many layers: softcapped attention in groups of four
+    with half of every head turned, a state-space recurrence (twice the width inside, heads of 64, 128 states, eight
+    groups), attention through a latent (a cached row of 512 + 64 numbers a token) over a window of 1,024; every layer
+    with the gated feed-forward of three widths."""
+    heads = max(4, width // 128)
+    attention = {"heads": heads, "kv_heads": heads // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+                 "rot": {"dims": 64, "base": 10000.0}}
+    recurrence = {"heads": width // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "mask": {"size": 1024},
+              "rot": {"dims": 64, "base": 100000.0, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    kinds = [("attention", attention), ("mamba2", recurrence), ("latent_attention", latent)]
+    own = max(1, layers // 2)
+    budanex = {"architecture": "Budanex", "vocab": 32000, "width": width, "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+               "loop": {"start": 0, "stop": own, "times": 2},
+               "layers": [{"type": kinds[i % 3][0], "mixer": kinds[i % 3][1], "mlp": {"kind": "dense", "ff": 3 * width}} for i in range(own)]}
+    others = dubizen_configs(width, layers)
+    return {"Budanex": budanex, "Dubizen": others["Dubizen"], "Talapel": talapel_configs(width, layers)["Talapel"],
+            "Rekezen": others["Rekezen"], "Qwen3": others["Qwen3"]}
+
+
 DESIGN_CONFIGS = {"mazanex": design_configs, "rekezen": rekezen_configs, "malusun": malusun_configs, "dubizen": dubizen_configs,
-                  "talapel": talapel_configs}
+                  "talapel": talapel_configs, "budanex": budanex_configs}
 
 
 def design_comparison(args) -> int:
-    """Prefill and decode throughput of Mazanex (or, with ``--design``, Rekezen, Malusun, Dubizen or Talapel) beside the closest existing models at equal
+    """Prefill and decode throughput of Mazanex (or, with ``--design``, Rekezen, Malusun, Dubizen, Talapel or Budanex) beside the closest existing models at equal
     width, layer count, feed-forward size and vocabulary; random weights, one JSON line a model and width."""
     import torch
 

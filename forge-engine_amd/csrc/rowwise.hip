@@ -57,10 +57,82 @@ __global__ __launch_bounds__(256) void embed_rows_norm_kernel(const int* __restr
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = load_as_float(src + i) * scale * inv * w[i];
 }
 
+// Rows of up to 2048 * VEC elements, a multiple of eight: the row stays in registers between the two passes.
+__device__ __forceinline__ void load8_as_float(const float* p, float v[8]) {
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const float4 a = ((const float4*)p)[k];
+    v[4 * k] = a.x; v[4 * k + 1] = a.y; v[4 * k + 2] = a.z; v[4 * k + 3] = a.w;
+  }
+}
+__device__ __forceinline__ void load8_as_float(const bf16_t* p, float v[8]) {
+  const uint4 a = *(const uint4*)p;
+  const uint32_t u[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    v[2 * k] = __uint_as_float(u[k] << 16);
+    v[2 * k + 1] = __uint_as_float(u[k] & 0xffff0000u);
+  }
+}
+
+template <typename TW, int VEC>
+__global__ __launch_bounds__(256) void embed_rows_norm_regs_kernel(const int* __restrict__ ids, const TW* __restrict__ table,
+                                                                   const float* __restrict__ w, float* __restrict__ out, int hidden,
+                                                                   int vocab, float scale, float eps) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x;
+  const int id = ids[t];
+  const bool known = id >= 0 && id < vocab;
+  const TW* src = table + (size_t)(known ? id : 0) * hidden;
+  float v[VEC][8], g[VEC][8];
+  float sumsq = 0.f;
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) {
+    const int i = (threadIdx.x + j * 256) * 8;
+    if (i < hidden) {
+      load8_as_float(src + i, v[j]);
+      load8_as_float(w + i, g[j]);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        v[j][k] *= scale;
+        sumsq += v[j][k] * v[j][k];
+      }
+    }
+  }
+  const float inv = known ? rsqrtf(block_sum<true>(sumsq, scratch) / (float)hidden + eps) : __int_as_float(0x7fc00000);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) {
+    const int i = (threadIdx.x + j * 256) * 8;
+    if (i < hidden) {
+      float4* dst = (float4*)(out + (size_t)t * hidden + i);
+#pragma unroll
+      for (int k = 0; k < 2; ++k)
+        dst[k] = make_float4(v[j][4 * k] * inv * g[j][4 * k], v[j][4 * k + 1] * inv * g[j][4 * k + 1],
+                             v[j][4 * k + 2] * inv * g[j][4 * k + 2], v[j][4 * k + 3] * inv * g[j][4 * k + 3]);
+    }
+  }
+}
+
 extern "C" int fe_embed_rows_norm(const int* ids, const void* table, int table_dtype, const float* w, float* out, int tokens,
                                   int hidden, int vocab, float scale, float eps, hipStream_t stream) {
   if (tokens <= 0) return FE_OK;
   if (hidden <= 0 || vocab <= 0 || !w || !(eps > 0.f)) return FE_BAD_ARGUMENT;
+  if (hidden % 8 == 0 && hidden <= 8192 && (((uintptr_t)table | (uintptr_t)w | (uintptr_t)out) & 15) == 0) {
+#define LAUNCH(TW, VEC) \
+  embed_rows_norm_regs_kernel<TW, VEC><<<tokens, 256, 0, stream>>>(ids, (const TW*)table, w, out, hidden, vocab, scale, eps)
+#define PICK(TW)                           \
+  do {                                     \
+    if (hidden <= 2048) LAUNCH(TW, 1);     \
+    else if (hidden <= 4096) LAUNCH(TW, 2); \
+    else LAUNCH(TW, 4);                    \
+  } while (0)
+    if (table_dtype == FE_F32) PICK(float);
+    else if (table_dtype == FE_BF16) PICK(bf16_t);
+    else return FE_BAD_ARGUMENT;
+#undef PICK
+#undef LAUNCH
+    return fe_check_launch();
+  }
   if (table_dtype == FE_F32)
     embed_rows_norm_kernel<float><<<tokens, 256, 0, stream>>>(ids, (const float*)table, w, out, hidden, vocab, scale, eps);
   else if (table_dtype == FE_BF16)

@@ -1,0 +1,454 @@
+"""Budanex on the GPU: its kernels alone against their plain references (tests/kernel_refs.py), and
+the model against the plain implementation (tests/plain_budanex.py) in float32 and bfloat16 over
+traces that cut the same requests in different ways."""
+
+from __future__ import annotations
+
+import pytest
+import torch
+
+import budanex_util as bu
+import kernel_refs as refs
+import replay_util as ru
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+plain = bu.plain
+DTYPES = [torch.float32, torch.bfloat16]
+
+CONFIGS = dict(bu.CONFIGS, M=bu.MEDIUM)
+LENGTHS = {"A": (5, 1, 14, 27, 90), "B": (2, 9, 21, 33, 64), "C": (7, 18, 3, 1, 40), "D": (12, 1, 25, 6, 50), "M": (4, 45, 170, 83, 1)}
+BLOCKS = dict(bu.BLOCK_SIZE, M=16)
+
+
+def close(got, want, dtype, loose=1.0):
+    tolerance = (2e-5 if dtype == torch.float32 else 2e-2) * loose
+    torch.testing.assert_close(got.float().cpu(), want.float(), rtol=tolerance, atol=tolerance)
+
+
+def to_dev(*tensors):
+    return [None if t is None else t.to(DEV) for t in tensors]
+
+
+# ------------------------------------------------------------------ rows
+
+@pytest.mark.parametrize("tokens,hidden", [(1, 40), (7, 2048), (300, 1000), (5, 4096), (3, 8000), (4, 33), (2, 9000)])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_embedding_rows_with_a_norm(tokens, hidden, dtype):
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(hidden)
+    table, weight = torch.randn(50, hidden, generator=g).to(dtype), torch.randn(hidden, generator=g)
+    ids = torch.randint(0, 50, (tokens,), generator=g, dtype=torch.int32)
+    want = refs.embed_rows(ids, table, torch.empty(tokens, hidden), 0.7, weight, 1e-2)
+    close(ops.embed_rows(ids.to(DEV), table.to(DEV), torch.empty(tokens, hidden, device=DEV), 0.7, weight.to(DEV), 1e-2), want, torch.float32)
+
+
+@pytest.mark.parametrize("rows,width,parts", [(1, 24, 0), (5, 40, 1), (3, 1536, 4), (7, 6000, 2), (600, 2048, 1), (4, 33, 3), (9, 9000, 1)])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_norm_and_sum_with_another_stream_and_a_vector(rows, width, parts, dtype):
+    """Update, another stream and a number a channel, in every combination: normed with the sum written back, normed for
+    chosen rows, and added up alone."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(width)
+    h, weight = torch.randn(rows, width, generator=g), torch.randn(width, generator=g)
+    updates = [None] if parts == 0 else [None, torch.randn(*((parts,) if parts > 1 else ()), rows, width, generator=g)]
+    for update in updates:
+        for other in (None, torch.randn(rows, width, generator=g)):
+            for shift in (None, torch.randn(width, generator=g)):
+                moved = dict(zip(("other", "shift"), to_dev(other, shift)))
+                ref, gpu = h.clone(), h.clone().to(DEV)
+                want = refs.add_rmsnorm(ref, update, weight, 1e-3, torch.empty(rows, width, dtype=dtype), other=other, shift=shift)
+                got = ops.add_rmsnorm(gpu, *to_dev(update), weight.to(DEV), 1e-3, torch.empty(rows, width, dtype=dtype, device=DEV), **moved)
+                close(got, want, dtype)
+                close(gpu, ref, torch.float32)
+                chosen = torch.tensor([rows - 1, 0, rows - 1], dtype=torch.int32)
+                want = refs.add_rmsnorm(h.clone(), update, weight, 1e-3, torch.empty(3, width, dtype=dtype), rows=chosen, store_sum=False,
+                                        other=other, shift=shift)
+                gpu = h.clone().to(DEV)
+                got = ops.add_rmsnorm(gpu, *to_dev(update), weight.to(DEV), 1e-3, torch.empty(3, width, dtype=dtype, device=DEV),
+                                      rows=chosen.to(DEV), store_sum=False, **moved)
+                close(got, want, dtype)
+                assert torch.equal(gpu.cpu(), h)
+                close(ops.add_rows(gpu, *to_dev(update), **moved), refs.add_rows(h.clone(), update, other, shift), torch.float32)
+
+
+def test_soft_cap_on_logits():
+    from forge_engine_amd.kernels import ops
+    x = torch.randn(5, 1003, generator=torch.Generator().manual_seed(1)) * 20.0
+    for cap, factor in ((15.0, 1.0), (3.0, -0.4)):
+        close(ops.cap_rows(x.clone().to(DEV), cap, factor), refs.cap_rows(x.clone(), cap, factor), torch.float32)
+
+
+@pytest.mark.parametrize("rows,inter,k", [(1, 40, 40), (3, 96, 256), (8, 9000, 512), (16, 8224, 4160), (17, 320, 320), (40, 512, 128), (64, 96, 4608),
+                                          (90, 200, 72), (2048, 256, 128), (3000, 320, 64)])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_gelu_in_gated_products(rows, inter, k, dtype):
+    """Every kernel that ends in a gate: few rows (with and without x kept in registers), gate and up rows paired, tiles of
+    whole prompts, the library with the activation behind it."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(rows + inter)
+    x, w = torch.randn(rows, k, generator=g).to(dtype), (torch.randn(2 * inter, k, generator=g) * 2.0 * k ** -0.5).to(dtype)
+    want = refs.linear_swiglu(x, w, "gelu_tanh")
+    assert float((want.float() - refs.linear_swiglu(x, w).float()).abs().max()) > 0.05        # not silu
+    close(ops.linear_swiglu(x.to(DEV), w.to(DEV), "gelu_tanh"), want, dtype)
+    if dtype == torch.bfloat16:
+        xg, wg = x.to(DEV), w.to(DEV)
+        if rows <= 64:
+            close(ops.gemm_skinny(xg, wg, "swiglu", act="gelu_tanh"), want, dtype)
+        if k % 64 == 0:
+            close(ops.gemm_wide(xg, wg, "swiglu", row_tile=64, act="gelu_tanh"), want, dtype)
+            close(ops.gemm_wide(xg, wg, "swiglu_half", row_tile=16, act="gelu_tanh"), want, dtype)
+            for shape in range(4):
+                close(ops.gemm_gated(xg, wg, shape, act="gelu_tanh"), want, dtype)
+        with pytest.raises(ops.KernelError):
+            ops.linear_swiglu(xg, wg, "relu")
+    z = torch.tensor([[0.0, -0.0, 1e-8, -3.0, 3.0, -12.0, 12.0, -200.0, 200.0, 0.5]]).to(dtype)
+    both = torch.cat([z, torch.ones_like(z)], dim=1)
+    close(ops.swiglu(both.to(DEV), torch.empty(1, 10, dtype=dtype, device=DEV), "gelu_tanh"), refs.swiglu(both, torch.empty(1, 10, dtype=dtype), "gelu_tanh"), dtype)
+
+
+# ------------------------------------------------------------------ attention's kernels
+
+def paged(lengths, block, generator, extra=2):
+    """A block table over shuffled pages and their count."""
+    pages = [-(-n // block) for n in lengths]
+    free = torch.randperm(sum(pages) + extra, generator=generator).tolist()
+    table = torch.full((len(lengths), max(pages)), -1, dtype=torch.int32)
+    for s, n in enumerate(pages):
+        table[s, :n] = torch.tensor([free.pop() for _ in range(n)], dtype=torch.int32)
+    return table, sum(pages) + extra
+
+
+def layout(q_lens, before):
+    cu = [0]
+    for n in q_lens:
+        cu.append(cu[-1] + n)
+    ints = lambda values: torch.tensor(values, dtype=torch.int32)      # noqa: E731
+    return (ints(cu), ints([s for s, n in enumerate(q_lens) for _ in range(n)]), ints([b + i for n, b in zip(q_lens, before) for i in range(n)]),
+            ints([n + b for n, b in zip(q_lens, before)]))
+
+
+WHOLE = [(4, 2, 12, 10, 6, 12, 10), (4, 2, 64, 64, 32, 64, 64), (8, 2, 128, 128, 128, 128, 128), (3, 3, 48, 40, 16, 64, 64), (6, 1, 96, 48, 96, 128, 128),
+         (5, 1, 24, 9, 16, 24, 9), (2, 1, 256, 16, 64, 256, 16), (64, 8, 128, 128, 64, 128, 128)]
+
+
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,rot,key_row,value_row", WHOLE)
+@pytest.mark.parametrize("block", [4, 16])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_norm_over_the_whole_projection_with_biases(heads, kv_heads, dim, vdim, rot, key_row, value_row, block, dtype):
+    """A step of a few tokens (heads over blocks) and one of many; portions that begin at a multiple of eight and beside
+    it, so that values leave in runs of eight and one by one; a page that is missing; rows filled up."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(dim + block)
+    q_size, k_size, v_size = heads * dim, kv_heads * dim, kv_heads * vdim
+    for q_lens, before in (([1, 1, 3], [0, 17, 8]), ([40, 1, 29, 33], [0, 100, 5, 16])):
+        cu_q, token_seq, positions, ctx = layout(q_lens, before)
+        table, pages = paged(ctx.tolist(), block, g)
+        tokens = sum(q_lens)
+        qkv = torch.randn(tokens, q_size + k_size + v_size + 16, generator=g).to(dtype)
+        for bias in (torch.randn(q_size + k_size + v_size, generator=g), None):
+            wq, wk = torch.randn(q_size, generator=g), torch.randn(k_size, generator=g)
+            inv_freq = torch.rand(rot // 2, generator=g)
+            start = [torch.randn(pages, kv_heads, block, key_row, generator=g).to(dtype), torch.randn(pages, kv_heads, value_row, block, generator=g).to(dtype)]
+            kw = dict(q_heads=heads, kv_heads=kv_heads, head_dim=dim, value_dim=vdim, rotary_dim=rot, eps=1e-3, magnitude=1.2)
+            want, got = [t.clone() for t in start], [t.clone().to(DEV) for t in start]
+            q = torch.empty(tokens, heads * key_row, dtype=dtype)
+            refs.whole_norm_rope_write(qkv, wq, wk, inv_freq, positions, token_seq, table, *want, q, bias=bias, **kw)
+            hole = table.clone()
+            if len(q_lens) == 4:        # one page of the last sequence is not there: its tokens are not written, and nothing else is
+                gone = int(table[3, 16 // block])
+                hole[3, 16 // block] = -1
+                want[0][gone], want[1][gone] = start[0][gone], start[1][gone]
+            q_gpu = torch.full((tokens, heads * key_row), 7.0, dtype=dtype, device=DEV)
+            ops.whole_norm_rope_write(*to_dev(qkv, wq, wk, inv_freq, positions, token_seq, hole), *got, q_gpu, bias=None if bias is None else bias.to(DEV), **kw)
+            close(q_gpu, q, dtype)
+            for a, b in zip(got, want):
+                close(a, b, dtype)
+    if key_row == dim and vdim == value_row:
+        q_gpu = torch.empty(tokens, q_size, dtype=dtype, device=DEV)
+        ops.whole_norm_rope_write(qkv[:, :q_size].to(DEV), *to_dev(wq, None, inv_freq, positions, token_seq), None, None, None, q_gpu, write_kv=False, **kw)
+        refs.whole_norm_rope_write(qkv, wq, None, inv_freq, positions, token_seq, None, None, None, q, write_kv=False, **kw)
+        close(q_gpu, q, dtype)
+
+
+@pytest.mark.parametrize("heads,dim,rank,rot,turned,row,latent_row", [(3, 10, 14, 6, 6, 20, 14), (4, 48, 100, 32, 32, 160, 128), (2, 1, 7, 8, 6, 23, 12), (8, 128, 512, 64, 64, 576, 512),
+                                                                      (1, 5, 33, 0, 0, 33, 33), (2, 16, 64, 16, 8, 96, 64)])
+@pytest.mark.parametrize("interleaved", [False, True])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_cache_rows_and_query_rows_of_a_latent(heads, dim, rank, rot, turned, row, latent_row, interleaved, dtype):
+    """Inputs in float32 and in the cache's dtype, through strided views, with and without a query bottleneck; both pairings of
+    the rotation with a factor; rows filled up; queries laid out like the rows."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(rank + rot)
+    q_lens, before, block = [3, 1, 20], [0, 70, 13], 8
+    _, token_seq, positions, ctx = layout(q_lens, before)
+    table, pages = paged(ctx.tolist(), block, g)
+    tokens = sum(q_lens)
+    inv_freq = torch.rand(turned // 2, generator=g) if turned else None
+    wkv = torch.randn(rank, generator=g)
+    kw = dict(kv_rank=rank, rot_dim=rot, rotary_dim=turned, eps=1e-3, write_kv=True, interleaved=interleaved, magnitude=1.3, latent_row=latent_row)
+    for x_dtype in {torch.float32, dtype}:
+        for q_rank in (0, 11):
+            x = torch.randn(tokens, 5 + q_rank + rank + rot, generator=g).to(x_dtype)
+            wq = torch.randn(q_rank, generator=g) if q_rank else None
+            want = [torch.full((pages, 1, block, row), 9.0, dtype=dtype), torch.full((pages, 1, latent_row, block), 9.0, dtype=dtype),
+                    torch.empty(tokens, q_rank, dtype=dtype) if q_rank else None]
+            got = [None if t is None else t.clone().to(DEV) for t in want]
+            refs.latent_norm_rope_write(x[:, 5:], wq, wkv, inv_freq, positions, token_seq, table, *want, q_rank=q_rank, **kw)
+            ops.latent_norm_rope_write(x.to(DEV)[:, 5:], *to_dev(wq, wkv, inv_freq, positions, token_seq, table), *got, q_rank=q_rank, **kw)
+            for a, b in zip(got, want):
+                if b is not None:
+                    close(a, b, dtype)
+    q = torch.randn(tokens, 3 + heads * (dim + rot), generator=g).to(dtype)
+    qa = torch.randn(heads, tokens, latent_row, generator=g).to(dtype)
+    kw = dict(heads=heads, dim=dim, rot_dim=rot, rotary_dim=turned, kv_rank=latent_row, interleaved=interleaved, magnitude=1.3)
+    want = refs.latent_query_pack(q[:, 3:], qa, inv_freq, positions, torch.empty(tokens, heads, row, dtype=dtype), **kw)
+    got = ops.latent_query_pack(q.to(DEV)[:, 3:], *to_dev(qa, inv_freq, positions), torch.full((tokens, heads, row), 5.0, dtype=dtype, device=DEV), **kw)
+    close(got, want, dtype)
+
+
+@pytest.mark.parametrize("heads,tokens,dim", [(1, 1, 8), (3, 5, 12), (8, 70, 64), (5, 9, 7)])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_heads_side_by_side_with_a_gate(heads, tokens, dim, dtype):
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(dim)
+    x = torch.randn(heads, tokens, dim, generator=g).to(dtype)
+    for pad in (8, 3):
+        gate = (torch.randn(tokens, heads * dim + pad, generator=g) * 3.0).to(dtype)
+        for chosen in (gate[:, pad:], None):
+            want = refs.gate_heads(x, chosen, torch.empty(tokens, heads * dim, dtype=dtype))
+            got = ops.gate_heads(x.to(DEV), None if chosen is None else gate.to(DEV)[:, pad:], torch.empty(tokens, heads * dim, dtype=dtype, device=DEV))
+            close(got, want, dtype)
+
+
+@pytest.mark.parametrize("heads,row,latent_row,block", [(4, 96, 64, 8), (3, 160, 128, 16), (16, 192, 128, 32), (6, 320, 256, 16), (16, 576, 512, 16), (5, 20, 14, 4), (2, 112, 96, 16)])
+@pytest.mark.parametrize("window", [1, 7, 32, 100, None])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_one_key_at_the_window_s_edge_over_a_latent(heads, row, latent_row, block, window, dtype):
+    """Keys that stand out just inside and just outside the windows of a portion's first and last token and of single
+    tokens, at page borders, at a tile's border and at the first position; sinks between negligible and dominant; pages ahead of every
+    window given back (their entries say so, and whatever lies in pages that are not the request's is not a number);
+    every count of key runs."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(row + (window or 0))
+    q_lens, before = [30, 1, 2, 1], [201, 150, 0, 3 * block - 1]
+    cu_q, token_seq, positions, ctx = layout(q_lens, before)
+    table, pages = paged(ctx.tolist(), block, g, extra=3)
+    tokens = sum(q_lens)
+    q = torch.randn(tokens, heads, row, generator=g)
+    key_pages = torch.full((pages, 1, block, row), float("nan"))
+    value_pages = torch.full((pages, 1, latent_row, block), float("nan"))
+    for s, (n, b) in enumerate(zip(q_lens, before)):
+        rows = torch.randn(b + n, row, generator=g)
+        direction = q[int(cu_q[s]):int(cu_q[s + 1])].mean((0, 1))
+        loud = {0, block - 1, block, 31, 32}
+        for p in {b, b + n - 1, b + n // 2}:
+            loud |= {p, p - (window or 40), p - (window or 40) + 1}
+        for place in loud:
+            if 0 <= place < b + n:
+                rows[place] = rows[place] * 0.5 + 4.0 * direction / direction.norm()
+        for p in range(b + n):
+            key_pages[table[s, p // block], 0, p % block] = rows[p]
+            value_pages[table[s, p // block], 0, :, p % block] = rows[p, :latent_row]
+        if window is not None:
+            passed = max(0, b - window + 1) // block
+            for page in table[s, :passed].tolist():
+                key_pages[page], value_pages[page] = float("nan"), float("nan")
+            table[s, :passed] = -1
+    key_pages, value_pages, q = key_pages.to(dtype), value_pages.to(dtype), q.reshape(tokens, -1).to(dtype)
+    sink = torch.tensor([[-30.0, 0.0, 3.0, 8.0][h % 4] for h in range(heads)])
+    kw = dict(num_seqs=len(q_lens), max_q_len=max(q_lens), heads=heads, row_dim=row, value_dim=latent_row, scale=row ** -0.5, window=window)
+    for sinks in (sink, None):
+        want = refs.latent_attention(q, key_pages, value_pages, torch.empty(tokens, heads * latent_row, dtype=dtype), cu_q, ctx, table, sink=sinks, **kw)
+        assert bool(torch.isfinite(want.float()).all())
+        moved = to_dev(q, key_pages, value_pages)
+        for splits in (None, 1, 3, 16):
+            out = torch.full((tokens, heads * latent_row), 7.0, dtype=dtype, device=DEV)
+            ops.latent_attention(*moved, out, *to_dev(cu_q, ctx, table), sink=None if sinks is None else sinks.to(DEV), num_decode=2,
+                                 max_ctx=int(ctx.max()), splits=splits, **kw)
+            close(out, want, dtype, loose=2.0)
+
+
+def test_sizes_of_filled_rows():
+    from forge_engine_amd.kernels import ops
+    for row, latent_row in ops.LATENT_ROWS:
+        assert ops.latent_attention_supported(torch.bfloat16, row, latent_row, 16)
+    assert ops.latent_row_sizes(torch.bfloat16, 96, 16) == (160, 128) and ops.latent_row_sizes(torch.bfloat16, 60, 40) == (192, 128)
+    assert ops.latent_row_sizes(torch.bfloat16, 512, 64) == (576, 512) and ops.latent_row_sizes(torch.bfloat16, 512, 65) == (577, 512)
+    assert ops.latent_row_sizes(torch.float32, 60, 40) == (100, 60)
+
+
+# ------------------------------------------------------------------ the model
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    kept = {}
+
+    def of(name, dtype):
+        if (name, dtype) not in kept:
+            kept[(name, dtype)] = bu.write_model(CONFIGS[name], 7, tmp_path_factory.mktemp(f"budanex_{name}"),
+                                                 change=lambda tensors: bu.enlarge(tensors, bu.ENLARGED[dtype]))
+        return kept[(name, dtype)]
+
+    return of
+
+
+@pytest.fixture(scope="module")
+def plain_of(folders):
+    kept = {}
+
+    def of(name, dtype, seed, lengths):
+        key = (name, dtype, seed, lengths)
+        if key not in kept:
+            requests = ru.make_requests({"vocab_size": CONFIGS[name]["vocab"]}, seed, lengths)
+            kept[key] = requests, bu.plain_logits(folders(name, dtype), requests)
+        return kept[key]
+
+    return of
+
+
+TRACES = {"whole": ru.trace_whole, "tail": lambda r: ru.trace_tail(r, 24), "portions": ru.trace_portions,
+          "mixed": lambda r: ru.trace_mixed(r, 5, max_live=4)}
+FRACTION = 0.05
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+@pytest.mark.parametrize("mode", sorted(TRACES))
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_traces_match_the_plain_implementation(name, mode, dtype, folders, plain_of, tmp_path):
+    requests, want = plain_of(name, dtype, 3, LENGTHS[name])
+    got = ru.run_trace(folders(name, dtype), dtype, TRACES[mode](requests), tmp_path, block_size=BLOCKS[name])
+    bu.compare(got, want, dtype, fraction=FRACTION, float32_factor=2.0)
+
+
+def test_matrix_core_kernels_serve_the_medium_sizes(folders):
+    from forge_engine_amd.engine import load_model
+    from forge_engine_amd.kernels import ops
+    _, model = load_model(folders("M", "bfloat16"), dtype="bfloat16", device=DEV)
+    mixers = [block.mixer for block in model.layers]
+    assert [(m.key_row, m.value_row) for m in (mixers[0], mixers[3])] == [(64, 64), (128, 128)]
+    assert [(m.row_dim, m.latent_row) for m in (mixers[1], mixers[4])] == [(160, 128), (192, 128)]
+    assert all(ops.latent_attention_supported(torch.bfloat16, m.row_dim, m.latent_row, 16) for m in (mixers[1], mixers[4]))
+
+
+def sharpen(tensors):
+    """Queries and keys larger, sinks of the scores' size and decays near one: one key of hundreds, and the first token,
+    reach the logits."""
+    bu.enlarge(tensors, 3.0)
+    for name in tensors:
+        if name.endswith((".mix.q.norm", ".mix.k.norm")):
+            tensors[name] = (tensors[name].float() * 1.5).to(tensors[name].dtype)
+        if name.endswith(".sink"):
+            tensors[name] = torch.full_like(tensors[name], 1.0)
+        if name.endswith(".A_log"):
+            tensors[name] = torch.full_like(tensors[name], -4.0)
+        if name.endswith(".dt_bias"):
+            tensors[name] = torch.full_like(tensors[name], -2.0)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_requests_with_sharp_attention_and_a_long_memory(dtype, tmp_path):
+    """Prompts of several hundred tokens: whole, then the last 100 tokens one by one (windows pass over decoded tokens),
+    then in portions, then three at once; and the control that the first token moves the last logits."""
+    folder = bu.write_model(bu.MEDIUM, 32, tmp_path / "sharp", change=sharpen)
+    requests = ru.make_requests({"vocab_size": bu.MEDIUM["vocab"]}, 9, (500, 333, 129))
+    want = bu.plain_logits(folder, requests)
+    cfg, weights = bu.folder_weights(folder)
+    changed = [(requests["r0"][0] + 1) % bu.MEDIUM["vocab"]] + requests["r0"][1:]
+    last = want[("r0", 499)]
+    assert float((plain.forward(cfg, weights, changed)[-1] - last).abs().max()) > 20 * (1e-5 + 1e-4 * float(last.abs().max()))
+    for mode, trace in (("whole", ru.trace_whole(requests)), ("tail", ru.trace_tail(requests, 100)),
+                        ("portions", ru.trace_portions(requests, sizes=(64, 17, 2, 230, 3, 48, 16, 2, 33), want_all=False)),
+                        ("mixed", ru.trace_mixed(requests, 11, max_live=3))):
+        got = ru.run_trace(folder, dtype, trace, tmp_path / mode, block_size=16)
+        bu.compare(got, want, dtype, fraction=0.08, float32_factor=4.0)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_captured_steps_equal_eager_steps_and_long_decoding(dtype, folders, plain_of):
+    """A prompt and then 150 single tokens, two requests side by side: steps replayed from captured graphs against the
+    same steps run eagerly (states move on once a step either way), and both against the plain implementation; then
+    portions whose shape repeats, captured and replayed with other contents."""
+    from forge_engine_amd.engine import ModelRunner, StepEntry, load_model
+    _, model = load_model(folders("M", dtype), dtype=dtype, device=DEV)
+    requests, want = plain_of("M", dtype, 21, (160, 171))
+    results = {}
+    for graphs in (True, False):
+        runner = ModelRunner(model, block_size=16, block_capacity=40, num_state_slots=3, use_graphs=graphs, eager_sightings=1)
+        got = {}
+        for name in requests:
+            runner.begin(name)
+        at = {"r0": 10, "r1": 21}
+        logits = runner.step([StepEntry(n, requests[n][:at[n]], [at[n] - 1]) for n in requests])
+        for row, n in zip(logits, requests):
+            got[(n, at[n] - 1)] = row.cpu().clone()
+        for _ in range(150):
+            logits = runner.step([StepEntry(n, [requests[n][at[n]]], [0]) for n in requests])
+            for row, n in zip(logits, requests):
+                got[(n, at[n])] = row.cpu().clone()
+                at[n] += 1
+        assert runner.graph_replays >= (140 if graphs else 0) and (graphs or runner.graph_replays == 0)
+        for name in requests:
+            runner.end(name)
+            runner.begin(name)
+        replays = runner.portion_graph_replays
+        for start in range(0, 160, 40):          # the same shape four times: eager, captured, replayed
+            logits = runner.step([StepEntry(n, requests[n][start:start + 40], [39]) for n in requests])
+            for row, n in zip(logits, requests):
+                got[(n, start + 39, "portions")] = row.cpu().clone()
+        assert runner.portion_graph_replays - replays >= (2 if graphs else 0)
+        results[graphs] = got
+        bu.compare({key[:2]: row for key, row in got.items() if len(key) == 2}, want, dtype, fraction=FRACTION, float32_factor=2.0)
+        bu.compare({key[:2]: row for key, row in got.items() if len(key) == 3}, want, dtype, fraction=FRACTION, float32_factor=2.0)
+    for key, row in results[True].items():
+        # a graph may cut the keys into other runs; in bfloat16 some positions are sensitive to the rounding of any of them
+        apart, size = ((t.double() ** 2).mean().sqrt() for t in (row - results[False][key], row))
+        assert float(apart) <= (2e-5 if dtype == "float32" else 5e-2) * float(size), key
+
+
+def test_first_tokens_and_slot_reuse(folders):
+    """A request that takes over the state slot and the pages of one that ended starts from nothing in every pass; requests
+    of one and two tokens."""
+    from forge_engine_amd.engine import ModelRunner, StepEntry, load_model
+    folder = folders("A", "float32")
+    _, model = load_model(folder, dtype="float32", device=DEV)
+    runner = ModelRunner(model, block_size=4, block_capacity=16, num_state_slots=1)
+    cfg, weights = bu.folder_weights(folder)
+    for tokens in ([5, 80, 17, 3], [44], [7, 7], [80, 5, 17, 3, 3, 3, 8, 1, 2]):
+        runner.begin("only")
+        rows = [runner.step([StepEntry("only", [token], [0])])[0].cpu().clone() for token in tokens]
+        runner.end("only")
+        for got, row in zip(rows, plain.forward(cfg, weights, tokens)):
+            assert float((got.double() - row).abs().max()) <= 2e-5 + 2e-4 * float(row.abs().max())
+
+
+def test_generation_through_the_entry_point_and_the_command_line(folders):
+    import os
+    import subprocess
+    import sys
+    from conftest import ROOT
+    from forge_engine_amd.config import SchedulerConfig
+    from forge_engine_amd.engine import engine_from_folder
+    from forge_engine_amd.sampling import SamplingParams
+
+    folder = folders("A", "float32")
+    cfg, weights = bu.folder_weights(folder)
+
+    def greedy(prompt, count):
+        tokens = list(prompt)
+        for _ in range(count):
+            tokens.append(int(plain.forward(cfg, weights, tokens)[-1].argmax()))
+        return tokens[len(prompt):]
+
+    prompts = list(ru.make_requests({"vocab_size": bu.SMALL_A["vocab"]}, 13, (11, 3, 25)).values())
+    want = [greedy(prompt, 8) for prompt in prompts]
+    engine = engine_from_folder(folder, scheduler_config=SchedulerConfig(block_size=4, block_capacity=128, token_budget=16),
+                                dtype="float32", eos_token_ids=[])
+    ids = [engine.submit(prompt, sampling_params=SamplingParams(max_new_tokens=8)) for prompt in prompts]
+    engine.run_until_idle()
+    assert [list(engine.request(i).output_token_ids) for i in ids] == want
+    command = [sys.executable, str(ROOT / "bin" / "forge-engine"), "generate", "--model", str(folder), "--dtype", "float32",
+               "--max-new-tokens", "8", "--block-size", "4", "--prompt-ids", ",".join(map(str, prompts[0]))]
+    done = subprocess.run(command, capture_output=True, text=True, timeout=300, env=dict(os.environ))
+    assert done.returncode == 0, done.stderr[-2000:]
+    assert ",".join(map(str, want[0])) in done.stdout.replace(" ", "")
