@@ -14,6 +14,9 @@
 //       the rotated part of every head of q [T, heads, dim + rot_dim], rotated here.
 //   fe_latent_gate_heads: the heads' results x [heads, T, dim] (of a batched product) side by side, [T, heads * dim],
 //       times sigmoid(gate) element by element if there is a gate.
+//   fe_latent_query_step, fe_latent_value_step: a few tokens (up to 16, bfloat16): the product per head and what follows
+//       it in one launch, the weight streamed once on the matrix cores: queries through the key up-projection straight into
+//       the query rows (with the rotated parts), and the attention's results through the value up-projection, gated.
 // Norms, angles, rotations and gates are float32, one rounding at the stores.
 #include "common.h"
 
@@ -162,6 +165,112 @@ extern "C" int fe_latent_query_pack(const void* q, long long q_stride, const voi
   else if (dtype == FE_BF16) LAUNCH(bf16_t);
   else return FE_BAD_ARGUMENT;
 #undef LAUNCH
+  return fe_check_launch();
+}
+
+// ---------------------------------------------------------------- a few tokens: product per head with its ending
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) float floatx4;
+typedef __attribute__((ext_vector_type(4))) unsigned int uintx4;
+
+#define STEP_TOKENS 16
+
+// y[t][n] = sum_k x[t][k] w[n][k] for one head, 16 columns n from n0 on; w [N, K] with K contiguous, a multiple of 8.
+// Block = 4 waves that share K in steps of 32; thread (m, c) = (tid / 16, tid % 16) returns y[m][n0 + c].
+__device__ __forceinline__ float head_tile(const bf16_t* __restrict__ x, size_t token_stride, const bf16_t* __restrict__ w,
+                                           int tokens, int N, int K, int n0, float (*red)[64][4]) {
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lr = lane & 15, lq = lane >> 4;
+  const bool row_ok = lr < tokens, col_ok = n0 + lr < N;
+  const bf16_t* xrow = x + (size_t)(row_ok ? lr : 0) * token_stride + lq * 8;
+  const bf16_t* wrow = w + (size_t)(col_ok ? n0 + lr : 0) * K + lq * 8;
+  const uintx4 none = uintx4{0u, 0u, 0u, 0u};
+  floatx4 acc = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = wave * 32; k < K; k += 128) {
+    const bool in = k + lq * 8 < K;
+    const uintx4 a = in && row_ok ? *(const uintx4*)(xrow + k) : none;
+    const uintx4 b = in && col_ok ? *(const uintx4*)(wrow + k) : none;
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
+  }
+  *(floatx4*)red[wave][lane] = acc;        // lane (lr, lq): rows 4 lq + i of column lr
+  __syncthreads();
+  const int m = tid >> 4, c = tid & 15;
+  float y = 0.f;
+#pragma unroll
+  for (int wv = 0; wv < 4; ++wv) y += red[wv][(m >> 2) * 16 + c][m & 3];
+  return y;
+}
+
+// Blocks (column tile, head); the last column tile's index stands for the head's rotated parts instead.
+__global__ __launch_bounds__(256) void latent_query_step_kernel(
+    const bf16_t* __restrict__ q, size_t q_stride, const bf16_t* __restrict__ uk, const float* __restrict__ inv_freq,
+    const int* __restrict__ positions, bf16_t* __restrict__ out, int tokens, int heads, int dim, int rot_dim, int rotary_dim,
+    int key_row, int value_row, Pairing pairs, float magnitude) {
+  __shared__ __attribute__((aligned(16))) float red[4][64][4];
+  const int h = blockIdx.y, tid = threadIdx.x;
+  const bf16_t* x = q + (size_t)h * (dim + rot_dim);
+  if (blockIdx.x + 1 < gridDim.x) {
+    const int n0 = blockIdx.x * 16;
+    const float y = head_tile(x, q_stride, uk + (size_t)h * value_row * dim, tokens, value_row, dim, n0, red);
+    const int m = tid >> 4, n = n0 + (tid & 15);
+    if (m < tokens && n < value_row) out[((size_t)m * heads + h) * key_row + n] = float_to_bf16(y);
+    return;
+  }
+  const int half = rotary_dim / 2;
+  for (int e = tid; e < tokens * half; e += 256) {
+    const int t = e / half, i = e - t * half;
+    float sn, cs;
+    sincosf((float)positions[t] * inv_freq[i], &sn, &cs);
+    cs *= magnitude;
+    sn *= magnitude;
+    const bf16_t* r = x + (size_t)t * q_stride + dim;
+    bf16_t* turned = out + ((size_t)t * heads + h) * key_row + value_row;
+    const int lo = i * pairs.step, hi = lo + pairs.offset;
+    const float u = bf16_to_float(r[lo]), v = bf16_to_float(r[hi]);
+    turned[lo] = float_to_bf16(u * cs - v * sn);
+    turned[hi] = float_to_bf16(v * cs + u * sn);
+  }
+  const int rest = key_row - value_row - rotary_dim;
+  for (int e = tid; e < tokens * rest; e += 256) {
+    const int t = e / rest, c = rotary_dim + e - t * rest;
+    out[((size_t)t * heads + h) * key_row + value_row + c] = c < rot_dim ? x[(size_t)t * q_stride + dim + c] : (bf16_t)0;
+  }
+}
+
+extern "C" int fe_latent_query_step(const void* q, long long q_stride, const void* uk, const float* inv_freq, const int* positions,
+                                    void* out, int tokens, int heads, int dim, int rot_dim, int rotary_dim, int key_row,
+                                    int value_row, int interleaved, float magnitude, hipStream_t stream) {
+  if (tokens <= 0) return FE_OK;
+  if (tokens > STEP_TOKENS || heads < 1 || heads > 65535 || dim < 8 || dim % 8 || (dim + rot_dim) % 8 || q_stride % 8 || value_row < 1 ||
+      rot_dim < 0 || rotary_dim < 0 || rotary_dim > rot_dim || rotary_dim % 2 || q_stride < (long long)heads * (dim + rot_dim) ||
+      key_row < value_row + rot_dim || !q || !uk || !out || !positions || (rotary_dim && !inv_freq) ||
+      ((((uintptr_t)q) | ((uintptr_t)uk)) & 15))
+    return FE_BAD_ARGUMENT;
+  latent_query_step_kernel<<<dim3((value_row + 15) / 16 + 1, heads), 256, 0, stream>>>(
+      (const bf16_t*)q, (size_t)q_stride, (const bf16_t*)uk, inv_freq, positions, (bf16_t*)out, tokens, heads, dim, rot_dim, rotary_dim,
+      key_row, value_row, pairing(rotary_dim, interleaved), magnitude);
+  return fe_check_launch();
+}
+
+__global__ __launch_bounds__(256) void latent_value_step_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ uv,
+                                                                const bf16_t* __restrict__ gate, size_t gate_stride,
+                                                                bf16_t* __restrict__ out, int tokens, int heads, int latent, int dim) {
+  __shared__ __attribute__((aligned(16))) float red[4][64][4];
+  const int h = blockIdx.y, n0 = blockIdx.x * 16, m = threadIdx.x >> 4, n = n0 + (threadIdx.x & 15);
+  const bool mine = m < tokens && n < dim;
+  const float g = mine && gate ? bf16_to_float(gate[(size_t)m * gate_stride + (size_t)h * dim + n]) : 0.f;
+  const float y = head_tile(x + (size_t)h * latent, (size_t)heads * latent, uv + (size_t)h * dim * latent, tokens, dim, latent, n0, red);
+  if (mine) out[(size_t)m * heads * dim + (size_t)h * dim + n] = float_to_bf16(gate ? y / (1.f + expf(-g)) : y);
+}
+
+extern "C" int fe_latent_value_step(const void* x, const void* uv, const void* gate, long long gate_stride, void* out, int tokens,
+                                    int heads, int latent, int dim, hipStream_t stream) {
+  if (tokens <= 0) return FE_OK;
+  if (tokens > STEP_TOKENS || heads < 1 || heads > 65535 || latent < 8 || latent % 8 || dim < 1 || !x || !uv || !out ||
+      (gate && gate_stride < (long long)heads * dim) || ((((uintptr_t)x) | ((uintptr_t)uv)) & 15))
+    return FE_BAD_ARGUMENT;
+  latent_value_step_kernel<<<dim3((dim + 15) / 16, heads), 256, 0, stream>>>((const bf16_t*)x, (const bf16_t*)uv, (const bf16_t*)gate,
+                                                                           (size_t)gate_stride, (bf16_t*)out, tokens, heads, latent, dim);
   return fe_check_launch();
 }
 

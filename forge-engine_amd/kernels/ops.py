@@ -1617,6 +1617,65 @@ def gate_heads(x: Tensor, gate: Tensor | None, out: Tensor) -> Tensor:
     return out
 
 
+LATENT_STEP_TOKENS = 16      # up to here the products per head around the attention over a latent end in the same launch
+
+
+def latent_step_fits(tokens: int, dtype, dim: int, rot_dim: int, latent_row: int) -> bool:
+    """Whether a step's products per head go through ``latent_query_step`` and ``latent_value_step``."""
+    return tokens <= LATENT_STEP_TOKENS and dtype == torch.bfloat16 and dim % 8 == 0 and rot_dim % 8 == 0 and latent_row % 8 == 0
+
+
+def latent_query_step(q: Tensor, uk: Tensor, inv_freq: Tensor | None, positions: Tensor, out: Tensor, *, heads: int, dim: int,
+                      rot_dim: int, rotary_dim: int, interleaved: bool = False, magnitude: float = 1.0) -> Tensor:
+    """The attention's query rows ``out`` [T, heads, row] (see ``latent_query_pack``) of up to 16 tokens straight from q [T,
+    heads * (dim + rot_dim)] (bfloat16, rows of any stride that is a multiple of 8) and the key up-projection ``uk`` [heads, latent_row, dim]: one
+    launch, the weight read once on the matrix cores, float32 sums."""
+    _gpu(q, "q", torch.bfloat16, contiguous=False)
+    _gpu(uk, "uk", torch.bfloat16)
+    _gpu(out, "out", torch.bfloat16)
+    _gpu(positions, "positions", torch.int32)
+    tokens = q.shape[0]
+    q_stride = _strided_rows(q, "q", heads * (dim + rot_dim))
+    if not latent_step_fits(tokens, q.dtype, dim, rot_dim, 8) or q_stride % 8 or q.data_ptr() % 16:
+        raise KernelError("up to 16 tokens, sizes and strides in multiples of 8, 16-byte alignment")
+    if uk.dim() != 3 or uk.shape[0] != heads or uk.shape[2] != dim:
+        raise KernelError(f"uk must be [{heads}, latent row, {dim}], got {tuple(uk.shape)}")
+    latent_row = uk.shape[1]
+    if out.dim() != 3 or out.shape[:2] != (tokens, heads) or out.shape[2] < latent_row + rot_dim or positions.numel() != tokens:
+        raise KernelError(f"out must be [{tokens}, {heads}, >= {latent_row + rot_dim}]")
+    if rotary_dim % 2 or not 0 <= rotary_dim <= rot_dim:
+        raise KernelError("rotary_dim must be even and at most rot_dim")
+    if rotary_dim:
+        _gpu(inv_freq, "inv_freq", torch.float32)
+        if inv_freq.shape != (rotary_dim // 2,):
+            raise KernelError(f"inv_freq must be [{rotary_dim // 2}]")
+    _call("latent", "fe_latent_query_step", _ptr(q), c_longlong(q_stride), _ptr(uk), _ptr(inv_freq if rotary_dim else None), _ptr(positions),
+          _ptr(out), c_int(tokens), c_int(heads), c_int(dim), c_int(rot_dim), c_int(rotary_dim), c_int(out.shape[2]), c_int(latent_row),
+          c_int(1 if interleaved else 0), c_float(magnitude), _stream())
+    return out
+
+
+def latent_value_step(x: Tensor, uv: Tensor, gate: Tensor | None, out: Tensor) -> Tensor:
+    """``out[t, h * D + d] = (uv[h] x[t, h])[d] * sigmoid(gate[t, h * D + d])`` for up to 16 tokens: x [T, heads, latent_row],
+    uv [heads, D, latent_row], gate [T, heads * D] rows of any stride or None, out [T, heads * D], all bfloat16, float32 sums."""
+    for name, t in (("x", x), ("uv", uv), ("out", out)):
+        _gpu(t, name, torch.bfloat16)
+    if x.dim() != 3 or uv.dim() != 3 or uv.shape[0] != x.shape[1] or uv.shape[2] != x.shape[2]:
+        raise KernelError(f"x must be [T, heads, latent row] and uv [heads, D, latent row], got {tuple(x.shape)} and {tuple(uv.shape)}")
+    tokens, heads, latent_row = x.shape
+    dim = uv.shape[1]
+    if tokens > LATENT_STEP_TOKENS or latent_row % 8 or out.shape != (tokens, heads * dim):
+        raise KernelError(f"up to 16 tokens, latent rows in multiples of 8, out [{tokens}, {heads * dim}]")
+    gate_stride = 0
+    if gate is not None:
+        gate_stride = _strided_rows(gate, "gate", heads * dim)
+        if gate.dtype != x.dtype or gate.shape[0] != tokens:
+            raise KernelError("gate must be in x's dtype with one row a token")
+    _call("latent", "fe_latent_value_step", _ptr(x), _ptr(uv), _ptr(gate), c_longlong(gate_stride), _ptr(out), c_int(tokens), c_int(heads),
+          c_int(latent_row), c_int(dim), _stream())
+    return out
+
+
 LATENT_TARGET_BLOCKS = 512      # blocks the matrix-core attention over a latent aims at before it stops cutting the keys into runs
 LATENT_MIN_TILES = 2            # ... and the fewest tiles a run may have (8 sequences at 1,024 keys, 16 heads, rows of 576, us a call with the
                                 # merge, in a captured graph: 1 run 110, 2 runs 62, 4 runs 36, 8 runs 24, 16 runs 21, 32 runs 25)

@@ -97,6 +97,8 @@ class LatentAttention(Mixer):
         self.uq_weight: Tensor | None = None
         self.uk: Tensor | None = None               # [heads, head_dim, latent_row]
         self.uv_t: Tensor | None = None             # [heads, latent_row, value_dim]
+        self.uk_t: Tensor | None = None             # the same two with the summed dim last, for steps of a few tokens
+        self.uv: Tensor | None = None
         self.o_weight: Tensor | None = None
 
     @property
@@ -147,8 +149,10 @@ class LatentAttention(Mixer):
             self.uq_weight = tensor
         elif key == "uk":
             self.uk = self._filled(tensor.view(self.num_heads, self.head_dim, self.kv_rank))
+            self.uk_t = self.uk.transpose(1, 2).contiguous() if self._steps(1) else None
         elif key == "uv":
-            self.uv_t = self._filled(tensor.view(self.num_heads, self.value_dim, self.kv_rank)).transpose(1, 2).contiguous()
+            uv = self._filled(tensor.view(self.num_heads, self.value_dim, self.kv_rank))
+            self.uv_t, self.uv = uv.transpose(1, 2).contiguous(), uv if self._steps(1) else None
         elif key == "o":
             self.o_weight = tensor
         else:
@@ -157,6 +161,10 @@ class LatentAttention(Mixer):
     def _filled(self, tensor: Tensor) -> Tensor:
         """The last dim filled up from the latent's size to its width in a cache row."""
         return tensor if self.latent_row == self.kv_rank else torch.nn.functional.pad(tensor, (0, self.latent_row - self.kv_rank))
+
+    def _steps(self, tokens: int) -> bool:
+        """Whether a step of so few tokens takes the products per head with their endings in one launch each."""
+        return ops.latent_step_fits(tokens, self.ctx.dtype, self.head_dim, self.rot_dim, self.latent_row)
 
     def cache_needs(self) -> CacheNeeds:
         return CacheNeeds(paged=PagedKV(1, self.row_dim, self.window, self.latent_row))
@@ -190,19 +198,27 @@ class LatentAttention(Mixer):
             q = ops.linear(latent_q, self.uq_weight)                                   # [T, H * (plain | rotated)]
             if self.output_gate:
                 gate = ops.linear(x, self.gate_weight)
-        plain = q.unflatten(1, (heads, self.q_head))[:, :, :self.head_dim]
-        through_keys = ops.heads_product(plain, self.uk)                               # [H, T, latent_row]
+        few = self._steps(tokens) and q.stride(0) % 8 == 0
         rows = torch.empty((tokens, heads, self.row_dim), dtype=x.dtype, device=x.device)
-        ops.latent_query_pack(q, through_keys, inv_freq, batch.positions, rows, heads=heads, dim=self.head_dim,
-                              kv_rank=self.latent_row, **turning)
+        if few:
+            ops.latent_query_step(q, self.uk_t, inv_freq, batch.positions, rows, heads=heads, dim=self.head_dim, **turning)
+        else:
+            plain = q.unflatten(1, (heads, self.q_head))[:, :, :self.head_dim]
+            through_keys = ops.heads_product(plain, self.uk)                           # [H, T, latent_row]
+            ops.latent_query_pack(q, through_keys, inv_freq, batch.positions, rows, heads=heads, dim=self.head_dim,
+                                  kv_rank=self.latent_row, **turning)
         read = torch.empty((tokens, heads * self.latent_row), dtype=x.dtype, device=x.device)
         ops.latent_attention(rows.view(tokens, heads * self.row_dim), cache.key_pages, cache.value_pages, read, batch.cu_q, batch.ctx_len,
                              cache.block_table, num_seqs=batch.num_seqs, max_q_len=batch.max_q_len, heads=heads,
                              row_dim=self.row_dim, value_dim=self.latent_row, scale=self.scale, num_decode=batch.num_decode,
                              max_ctx=batch.max_ctx, window=self.window, sink=self.sink_weight)
-        values = ops.heads_product(read.view(tokens, heads, self.latent_row), self.uv_t)  # [H, T, value_dim]
         attn = torch.empty((tokens, heads * self.value_dim), dtype=x.dtype, device=x.device)
-        return ops.linear_update(ops.gate_heads(values, gate, attn), self.o_weight, stream=stream)
+        read = read.view(tokens, heads, self.latent_row)
+        if few:
+            ops.latent_value_step(read, self.uv, gate, attn)
+        else:
+            ops.gate_heads(ops.heads_product(read, self.uv_t), gate, attn)             # values [H, T, value_dim]
+        return ops.linear_update(attn, self.o_weight, stream=stream)
 
     def token_inputs(self):
         return self.position.token_inputs()

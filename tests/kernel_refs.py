@@ -880,6 +880,20 @@ def gate_heads(x, gate, out):
     return out
 
 
+def latent_step_fits(tokens, dtype, dim, rot_dim, latent_row):
+    return tokens <= 2 and dtype == torch.bfloat16        # so that CPU tests meet both
+
+
+def latent_query_step(q, uk, inv_freq, positions, out, *, heads, dim, rot_dim, **turning):
+    plain = q.reshape(q.shape[0], heads, dim + rot_dim)[:, :, :dim]
+    qa = heads_product(plain, uk.transpose(1, 2))
+    return latent_query_pack(q, qa, inv_freq, positions, out, heads=heads, dim=dim, rot_dim=rot_dim, kv_rank=uk.shape[1], **turning)
+
+
+def latent_value_step(x, uv, gate, out):
+    return gate_heads(heads_product(x, uv.transpose(1, 2)), gate, out)
+
+
 def latent_row_sizes(dtype, kv_rank, rot_dim):
     """A filled-up row in bfloat16, as the kernels would have it, in sizes of its own."""
     return (kv_rank + rot_dim, kv_rank) if dtype == torch.float32 else (kv_rank + 3 + rot_dim + 2, kv_rank + 3)
@@ -939,7 +953,7 @@ def linear_in_parts(x, weight):
 DECODE_SPLITS_TESTED = tuple(range(1, 65))
 
 
-NAMES = ("cap_rows", "gate_heads", "latent_row_sizes", "decode_prepare_supported", "linear_in_parts", "embed_rows", "add_rmsnorm", "add_rows", "swiglu", "gemm_nt_f32", "linear", "linear_update", "linear_swiglu", "gemm_skinny",
+NAMES = ("cap_rows", "gate_heads", "latent_row_sizes", "latent_step_fits", "latent_query_step", "latent_value_step", "decode_prepare_supported", "linear_in_parts", "embed_rows", "add_rmsnorm", "add_rows", "swiglu", "gemm_nt_f32", "linear", "linear_update", "linear_swiglu", "gemm_skinny",
          "qk_norm_rope_write", "paged_attention", "argmax_rows", "sample_filtered_rows",
          "cast_rows", "add_bias", "token_shift", "rmsnorm_update", "rmsnorm_mean", "polynorm", "tanh_rows", "head_norm_gate",
          "conv_rope_norm_write", "masked_attention", "linear_recurrence", "mlstm_gate_scan",

@@ -221,6 +221,34 @@ def test_heads_side_by_side_with_a_gate(heads, tokens, dim, dtype):
             close(got, want, dtype)
 
 
+@pytest.mark.parametrize("heads,dim,rot,turned,rank,row,vdim", [(3, 8, 8, 6, 24, 40, 5), (16, 128, 64, 64, 512, 576, 128), (4, 48, 32, 32, 128, 160, 40), (1, 136, 0, 0, 8, 8, 17),
+                                                                 (5, 64, 16, 16, 57, 73, 1)])
+@pytest.mark.parametrize("tokens", [1, 7, 16])
+def test_products_per_head_of_a_few_tokens(heads, dim, rot, turned, rank, row, vdim, tokens):
+    """Queries through the key up-projection into their rows, results through the value up-projection behind a gate."""
+    from forge_engine_amd.kernels import ops
+    g = torch.Generator().manual_seed(dim + tokens)
+    bf16 = torch.bfloat16
+    size = heads * (dim + rot)
+    q = torch.randn(tokens, size + 24, generator=g).to(bf16)
+    uk = (torch.randn(heads, rank, dim, generator=g) * dim ** -0.5).to(bf16)
+    positions = torch.randint(0, 900, (tokens,), generator=g, dtype=torch.int32)
+    inv_freq = torch.rand(turned // 2, generator=g) if turned else None
+    for interleaved in (False, True):
+        kw = dict(heads=heads, dim=dim, rot_dim=rot, rotary_dim=turned, interleaved=interleaved, magnitude=1.2)
+        want = refs.latent_query_step(q[:, 8:8 + size], uk, inv_freq, positions, torch.empty(tokens, heads, row, dtype=bf16), **kw)
+        got = ops.latent_query_step(q.to(DEV)[:, 8:8 + size], *to_dev(uk, inv_freq, positions), torch.full((tokens, heads, row), 7.0, dtype=bf16, device=DEV), **kw)
+        close(got, want, bf16)
+    if rank % 8:
+        return
+    x, uv = torch.randn(tokens, heads, rank, generator=g).to(bf16), (torch.randn(heads, vdim, rank, generator=g) * rank ** -0.5).to(bf16)
+    gate = torch.randn(tokens, heads * vdim + 3, generator=g).to(bf16)
+    for chosen in (gate[:, 3:], None):
+        want = refs.latent_value_step(x, uv, chosen, torch.empty(tokens, heads * vdim, dtype=bf16))
+        got = ops.latent_value_step(*to_dev(x, uv), None if chosen is None else gate.to(DEV)[:, 3:], torch.empty(tokens, heads * vdim, dtype=bf16, device=DEV))
+        close(got, want, bf16)
+
+
 @pytest.mark.parametrize("heads,row,latent_row,block", [(4, 96, 64, 8), (3, 160, 128, 16), (16, 192, 128, 32), (6, 320, 256, 16), (16, 576, 512, 16), (5, 20, 14, 4), (2, 112, 96, 16)])
 @pytest.mark.parametrize("window", [1, 7, 32, 100, None])
 @pytest.mark.parametrize("dtype", DTYPES)
